@@ -9,7 +9,7 @@
 // as 2 x 2 v_mfma_f32_32x32x16_bf16 accumulators.  Global loads run two K steps ahead of the MFMAs, and
 // loads and LDS stores are spread between the MFMAs of a step: LDS bandwidth (reads of operands plus stores of
 // the next step) and the load path are each about as busy as the matrix cores, so none of them may wait for another.
-// Epilogues: store bfloat16 / float32, add into a float32 residual, or SwiGLU: then the W tile is
+// Epilogues: store bfloat16 / float32, add into a float32 residual, the squared relu in bfloat16 (grouped rows only), or SwiGLU: then the W tile is
 // 64 gate rows and the matching 64 up rows, each wave computes gate and up of the same 64 x 32 outputs,
 // and the block writes a 128 x 64 tile of silu(gate) * up.
 // With 17..128 rows and a long K, K is cut into slices for different blocks and a second kernel adds the slices in
@@ -28,7 +28,7 @@ constexpr int BN = 128, BK = 64;
 constexpr int BM_ROWS = 128;
 constexpr int LDS_ROW = BK + 8;  // bfloat16 elements per LDS row (144 bytes)
 
-enum { G_STORE_BF16 = 0, G_STORE_F32 = 1, G_ACC_F32 = 2, G_SWIGLU = 3, G_PARTIAL = 4 };
+enum { G_STORE_BF16 = 0, G_STORE_F32 = 1, G_ACC_F32 = 2, G_SWIGLU = 3, G_PARTIAL = 4, G_RELU2 = 5 };
 
 template <int BM>
 struct GemmRegs {
@@ -95,7 +95,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
     const int e = grp.tiles[3 * ti], p0 = grp.tiles[3 * ti + 1];
     M = grp.tiles[3 * ti + 2];                       // the tile's rows are all the rows this block knows of
     A += (size_t)p0 * lda;
-    C = (char*)C + (size_t)p0 * ldc * (MODE == G_STORE_BF16 || MODE == G_SWIGLU ? 2 : 4);
+    C = (char*)C + (size_t)p0 * ldc * (MODE == G_STORE_BF16 || MODE == G_SWIGLU || MODE == G_RELU2 ? 2 : 4);
     W += (size_t)e * grp.w_stride;
     if (MODE == G_SWIGLU) W2 += (size_t)e * grp.w_stride;
   } else {
@@ -313,6 +313,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
           if (n >= N) continue;
           const size_t o = (size_t)m * ldc + n;
           if (MODE == G_STORE_BF16) ((bf16_t*)C)[o] = float_to_bf16(acc[a][b][r]);
+          else if (MODE == G_RELU2) ((bf16_t*)C)[o] = float_to_bf16(fmaxf(acc[a][b][r], 0.f) * fmaxf(acc[a][b][r], 0.f));
           else if (MODE == G_STORE_F32) ((float*)C)[o] = acc[a][b][r];
           else if (MODE == G_ACC_F32) ((float*)C)[o] += acc[a][b][r];
           else ((float*)C)[((size_t)blockIdx.z * M + m) * N + n] = acc[a][b][r];
@@ -643,13 +644,13 @@ APC_EXPORT int apc_gemm_bf16(const void* A, int lda, const void* W, void* C, int
 }
 
 // Rows in runs of one matrix each (see GroupedRows): mode G_SWIGLU (W, W2: gate and up; bfloat16 out; act, alpha, limit:
-// the gated unit's activation) or G_STORE_F32.  tile_rows: 64 or 128, the rows `tiles` was cut for.
+// the gated unit's activation), G_RELU2 (the square of max(sum, 0), bfloat16 out) or G_STORE_F32.  tile_rows: 64 or 128, the rows `tiles` was cut for.
 APC_EXPORT int apc_gemm_grouped_bf16(const void* A, int lda, const void* W, const void* W2, size_t w_stride, void* C,
                                      int ldc, const int* tiles, const int* n_tiles, int max_tiles, int tile_rows,
                                      int N, int K, int mode, int act, float alpha, float limit, hipStream_t stream) {
   if (max_tiles <= 0) return 0;
   if (N <= 0 || K <= 0 || K % 8 || lda % 8 || !tiles || !n_tiles || (tile_rows != 64 && tile_rows != 128) ||
-      (mode != G_SWIGLU && mode != G_STORE_F32) || (mode == G_SWIGLU && !W2) || max_tiles > 65535 || act < 0 || act > 1)
+      (mode != G_SWIGLU && mode != G_STORE_F32 && mode != G_RELU2) || (mode == G_SWIGLU && !W2) || max_tiles > 65535 || act < 0 || act > 1)
     return APC_ERR_BAD_ARG;
   if (!aligned16(A) || !aligned16(W) || (W2 && !aligned16(W2))) return APC_ERR_UNSUPPORTED;
   const GroupedRows grp{tiles, n_tiles, w_stride, act, alpha, limit};
@@ -670,6 +671,7 @@ APC_EXPORT int apc_gemm_grouped_bf16(const void* A, int lda, const void* W, cons
     }                                                                        \
   } while (0)
   if (mode == G_SWIGLU) GROUPED_BY(G_SWIGLU);
+  else if (mode == G_RELU2) GROUPED_BY(G_RELU2);
   else GROUPED_BY(G_STORE_F32);
 #undef GROUPED_BY
 #undef GROUPED_LAUNCH

@@ -12,10 +12,14 @@
 constexpr int TM = 64, TN = 64, TK = 16;
 
 // mode 0: C = acc (C of c_dtype)   mode 1: C += acc (C float32)
+// blockIdx.z: one of several products of the same sizes, whose operands lie these many elements apart.
+struct HeadStrides {
+  size_t a = 0, w = 0, c = 0;
+};
 __global__ __launch_bounds__(256) void gemm_plain_kernel(const void* __restrict__ A, int a_dtype, int lda,
                                                          const void* __restrict__ W, int w_dtype, int ldw,
                                                          void* __restrict__ C, int c_dtype, int ldc, int M, int N,
-                                                         int K, int mode) {
+                                                         int K, int mode, HeadStrides hs) {
   __shared__ float As[TK][TM + 4];
   __shared__ float Ws[TK][TN + 4];
   const int tid = threadIdx.x;
@@ -36,8 +40,8 @@ __global__ __launch_bounds__(256) void gemm_plain_kernel(const void* __restrict_
       const int k = k0 + kk;
       float a = 0.f, w = 0.f;
       if (k < K) {
-        if (m0 + r < M) a = load_f(A, a_dtype, (size_t)(m0 + r) * lda + k);
-        if (n0 + r < N) w = load_f(W, w_dtype, (size_t)(n0 + r) * ldw + k);
+        if (m0 + r < M) a = load_f(A, a_dtype, blockIdx.z * hs.a + (size_t)(m0 + r) * lda + k);
+        if (n0 + r < N) w = load_f(W, w_dtype, blockIdx.z * hs.w + (size_t)(n0 + r) * ldw + k);
       }
       As[kk][r] = a;
       Ws[kk][r] = w;
@@ -65,7 +69,7 @@ __global__ __launch_bounds__(256) void gemm_plain_kernel(const void* __restrict_
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
-      const size_t o = (size_t)m * ldc + n;
+      const size_t o = blockIdx.z * hs.c + (size_t)m * ldc + n;
       if (mode == 1) ((float*)C)[o] += acc[i][j];
       else store_f(C, c_dtype, o, acc[i][j]);
     }
@@ -80,7 +84,20 @@ APC_EXPORT int apc_gemm_plain(const void* A, int a_dtype, int lda, const void* W
   const int gy = ceil_div(M, TM);
   if (gy > 65535) return APC_ERR_BAD_ARG;
   hipLaunchKernelGGL(gemm_plain_kernel, dim3(ceil_div(N, TN), gy), dim3(256), 0, stream, A, a_dtype, lda, W, w_dtype,
-                     ldw, C, c_dtype, ldc, M, N, K, mode);
+                     ldw, C, c_dtype, ldc, M, N, K, mode, HeadStrides{});
+  APC_LAUNCH_CHECK();
+  return 0;
+}
+
+// A matrix of its own for every head: C[m][h * c_head + n] = A[m][h * a_head ..] . W[h][n], W [H][N][K] contiguous.
+APC_EXPORT int apc_heads_gemm_plain(const void* A, int a_dtype, int lda, int a_head, const void* W, int w_dtype, void* C,
+                                    int c_dtype, int ldc, int c_head, int M, int H, int N, int K, hipStream_t stream) {
+  if (M <= 0 || H <= 0 || N <= 0) return 0;
+  if (K <= 0 || a_head < K || c_head < N || lda < (H - 1) * a_head + K || ldc < (H - 1) * c_head + N) return APC_ERR_BAD_ARG;
+  const int gy = ceil_div(M, TM);
+  if (gy > 65535 || H > 65535) return APC_ERR_BAD_ARG;
+  hipLaunchKernelGGL(gemm_plain_kernel, dim3(ceil_div(N, TN), gy, H), dim3(256), 0, stream, A, a_dtype, lda, W, w_dtype, K,
+                     C, c_dtype, ldc, M, N, K, 0, HeadStrides{(size_t)a_head, (size_t)N * K, (size_t)c_head});
   APC_LAUNCH_CHECK();
   return 0;
 }

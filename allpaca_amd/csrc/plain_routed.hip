@@ -7,7 +7,11 @@
 //   lower index wins a tie);  weights: s of the chosen
 //   y[t] = sum_k w[t][k] * (expert e = ids[t][k] has matrices ? Wd_e (a(Wg_e h, Wu_e h)) : h)
 //   a(g, u) = silu(g) * u  (`act` 0), or with g' = min(g, limit), u' = clamp(u, -limit, limit):
-//   g' * sigmoid(alpha g') * (u' + 1)  (`act` 1)
+//   g' * sigmoid(alpha g') * (u' + 1)  (`act` 1), or an expert without a gate: the square of max(u, 0)  (`act` 2; the
+//   matrices are then [E][F][D], up rows alone)
+// `groups` > 1: the outputs form that many equal runs of neighbours; a run's score is the sum of the two largest
+// s + correction in it, and only outputs of the `keep` runs with the largest scores (the lower run on a tie) can be
+// chosen.  With `renormalize` the weights are divided by their sum (+ 1e-20); they are multiplied by `w_scale`.
 // With `in_weights` the weight multiplies the expert's input instead of its output: y[t] = sum_k expert(w[t][k] h[t]),
 // formed as a(w g, w u) from the same sums g = Wg h, u = Wu h (the products are linear in h).
 #include "common.h"
@@ -20,8 +24,11 @@ constexpr int MAX_TOP = 32;
 
 __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict__ z, int ldz,
                                                         const float* __restrict__ correction, int N, int K,
-                                                        int renormalize, int score, int* __restrict__ ids,
+                                                        int renormalize, int score, int groups, int keep,
+                                                        float w_scale, int* __restrict__ ids,
                                                         float* __restrict__ weights) {
+  __shared__ float cs[MAX_PER_LANE_R * WAVE];      // groups > 1: the choice scores, and whether a run is kept
+  __shared__ int kept[MAX_PER_LANE_R * WAVE];
   const int t = blockIdx.x, lane = threadIdx.x;
   float s[MAX_PER_LANE_R], c[MAX_PER_LANE_R];
   float mx = -INFINITY;
@@ -46,6 +53,52 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
     const int i = lane + e * WAVE;
     s[e] = s[e] / sum;
     c[e] = i < N ? s[e] + (correction ? correction[i] : 0.f) : -INFINITY;
+  }
+  if (groups > keep) {
+    const int n = N / groups;
+#pragma unroll
+    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+      const int i = lane + e * WAVE;
+      if (i < N) cs[i] = c[e];
+    }
+    __syncthreads();
+    float gs[MAX_PER_LANE_R];
+#pragma unroll
+    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+      const int g = lane + e * WAVE;
+      gs[e] = -INFINITY;
+      if (g >= groups) continue;
+      float a = -INFINITY, b = -INFINITY;          // the largest and the next
+      for (int i = 0; i < n; ++i) {
+        const float v = cs[g * n + i];
+        if (v > a) { b = a; a = v; }
+        else if (v > b) b = v;
+      }
+      gs[e] = n > 1 ? a + b : a;
+      kept[g] = 0;
+    }
+    for (int k = 0; k < keep; ++k) {
+      float best = -INFINITY;
+      int best_g = 0x7fffffff;
+#pragma unroll
+      for (int e = 0; e < MAX_PER_LANE_R; ++e)
+        if (gs[e] > best) { best = gs[e]; best_g = lane + e * WAVE; }
+#pragma unroll
+      for (int o = WAVE / 2; o > 0; o >>= 1) {
+        const float ob = __shfl_xor(best, o, WAVE);
+        const int og = __shfl_xor(best_g, o, WAVE);
+        if (ob > best || (ob == best && og < best_g)) { best = ob; best_g = og; }
+      }
+#pragma unroll
+      for (int e = 0; e < MAX_PER_LANE_R; ++e)
+        if (lane + e * WAVE == best_g) { gs[e] = -INFINITY; kept[best_g] = 1; }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+      const int i = lane + e * WAVE;
+      if (i < N && !kept[i / n]) c[e] = -INFINITY;
+    }
   }
   float total = 0.f;
   float mine = 0.f;      // lane k keeps the k-th weight
@@ -75,13 +128,14 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
     if (lane == k) { mine = w; mine_id = best_i; }
   }
   if (lane < K) {
-    ids[(size_t)t * K + lane] = mine_id;
-    weights[(size_t)t * K + lane] = renormalize ? mine / total : mine;
+    // (a row whose scores are not numbers chooses nothing: the ids stay inside the table)
+    ids[(size_t)t * K + lane] = mine_id < N ? mine_id : N - 1;
+    weights[(size_t)t * K + lane] = (renormalize ? mine / (total + 1e-20f) : mine) * w_scale;
   }
 }
 
 // act[t * K + k][f] = silu(Wg_e[f] . h[t]) * (Wu_e[f] . h[t]) for e = ids[t][k] with matrices;
-// w_gate_up [E][2F][D] (an expert's gate rows, then its up rows).
+// w_gate_up [E][2F][D] (an expert's gate rows, then its up rows); kind 2: [E][F][D], act = relu(W_e[f] . h[t])^2.
 __global__ __launch_bounds__(256) void routed_glu_kernel(const void* __restrict__ h, int h_dtype, int ldh,
                                                          const void* __restrict__ w_gate_up, int w_dtype, int E, int F,
                                                          int D, const int* __restrict__ ids, int K,
@@ -95,6 +149,15 @@ __global__ __launch_bounds__(256) void routed_glu_kernel(const void* __restrict_
   __syncthreads();
   const int f = blockIdx.y * 256 + threadIdx.x;
   if (f >= F) return;
+  if (kind == 2) {
+    const size_t row = ((size_t)e * F + f) * D;
+    float v = 0.f;
+    for (int i = 0; i < D; ++i) v = fmaf(hs[i], load_f(w_gate_up, w_dtype, row + i), v);
+    if (in_weights) v *= in_weights[pair];
+    v = fmaxf(v, 0.f);
+    store_f(act, act_dtype, (size_t)pair * F + f, v * v);
+    return;
+  }
   const size_t gate_row = ((size_t)e * 2 * F + f) * D, up_row = gate_row + (size_t)F * D;
   float g = 0.f, u = 0.f;
   for (int i = 0; i < D; ++i) {
@@ -156,12 +219,14 @@ __global__ __launch_bounds__(256) void routed_down_kernel(const void* __restrict
 }  // namespace
 
 APC_EXPORT int apc_route_topk(const float* z, int ldz, const float* correction, int n_rows, int N, int K,
-                              int renormalize, int score, int* ids, float* weights, hipStream_t stream) {
+                              int renormalize, int score, int groups, int keep, float w_scale, int* ids,
+                              float* weights, hipStream_t stream) {
   if (n_rows <= 0) return 0;
+  if (groups < 1 || keep < 1 || keep > groups || N <= 0 || N % groups || K > keep * (N / groups)) return APC_ERR_BAD_ARG;
   if (N <= 0 || K <= 0 || K > N || ldz < N || !ids || !weights || score < 0 || score > 1) return APC_ERR_BAD_ARG;
   if (N > MAX_PER_LANE_R * WAVE || K > MAX_TOP) return APC_ERR_UNSUPPORTED;
   hipLaunchKernelGGL(route_topk_kernel, dim3(n_rows), dim3(64), 0, stream, z, ldz, correction, N, K, renormalize, score,
-                     ids, weights);
+                     groups, keep, w_scale, ids, weights);
   APC_LAUNCH_CHECK();
   return 0;
 }
@@ -170,7 +235,7 @@ APC_EXPORT int apc_routed_glu(const void* h, int h_dtype, int ldh, const void* w
                               int D, const int* ids, int K, void* act, int act_dtype, int n_rows, int kind, float alpha,
                               float limit, const float* in_weights, hipStream_t stream) {
   if (n_rows <= 0 || E <= 0) return 0;
-  if (F <= 0 || D <= 0 || K <= 0 || ldh < D || kind < 0 || kind > 1) return APC_ERR_BAD_ARG;
+  if (F <= 0 || D <= 0 || K <= 0 || ldh < D || kind < 0 || kind > 2) return APC_ERR_BAD_ARG;
   if ((size_t)D * sizeof(float) > 64 * 1024 || (long)n_rows * K > 0x7fffffffL || ceil_div(F, 256) > 65535)
     return APC_ERR_UNSUPPORTED;
   hipLaunchKernelGGL(routed_glu_kernel, dim3(n_rows * K, ceil_div(F, 256)), dim3(256), (size_t)D * sizeof(float),

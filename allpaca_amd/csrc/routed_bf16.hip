@@ -83,8 +83,8 @@ __global__ __launch_bounds__(1024) void routed_sort_kernel(const int* __restrict
 }
 
 // RT tiles of 16 rows a wave: a weight tile read from memory feeds RT MFMAs (the launches use 1: more rows an expert
-// go to the tiled kernel)
-template <int RT>
+// go to the tiled kernel).  GATED = false: an expert has no gate (w_gate_up is [E][bands(F)][chunks(D)]..), a = max(u, 0)^2
+template <int RT, bool GATED>
 __global__ __launch_bounds__(256) void routed_glu_bf16_kernel(const bf16_t* __restrict__ h, int ldh,
                                                               const bf16_t* __restrict__ w_gate_up, int F, int D,
                                                               const int* __restrict__ order, int K,
@@ -99,8 +99,8 @@ __global__ __launch_bounds__(256) void routed_glu_bf16_kernel(const bf16_t* __re
   const int band = blockIdx.y * 4 + wave;
   if (band >= bands) return;
   const int e = tiles[3 * ti], p0 = tiles[3 * ti + 1], rows = tiles[3 * ti + 2];
-  const bf16_t* wg = w_gate_up + (((size_t)e * 2) * bands + band) * chunks * TILE_ELEMS + lane * 8;
-  const bf16_t* wu = wg + (size_t)bands * chunks * TILE_ELEMS;
+  const bf16_t* wg = w_gate_up + (((size_t)e * (GATED ? 2 : 1)) * bands + band) * chunks * TILE_ELEMS + lane * 8;
+  const bf16_t* wu = GATED ? wg + (size_t)bands * chunks * TILE_ELEMS : wg;
   const bf16_t* arow[RT];
   bool on[RT];
 #pragma unroll
@@ -119,7 +119,7 @@ __global__ __launch_bounds__(256) void routed_glu_bf16_kernel(const bf16_t* __re
     Frag fg[STREAM_U], fu[STREAM_U], a[STREAM_U][RT];
 #pragma unroll
     for (int x = 0; x < STREAM_U; ++x) {
-      fg[x] = load_frag_once(wg + (size_t)(c + x) * TILE_ELEMS);
+      if (GATED) fg[x] = load_frag_once(wg + (size_t)(c + x) * TILE_ELEMS);
       fu[x] = load_frag_once(wu + (size_t)(c + x) * TILE_ELEMS);
 #pragma unroll
       for (int rt = 0; rt < RT; ++rt)
@@ -131,16 +131,17 @@ __global__ __launch_bounds__(256) void routed_glu_bf16_kernel(const bf16_t* __re
     for (int x = 0; x < STREAM_U; ++x)
 #pragma unroll
       for (int rt = 0; rt < RT; ++rt) {
-        g[rt] = mfma16(fg[x], a[x][rt], g[rt]);
+        if (GATED) g[rt] = mfma16(fg[x], a[x][rt], g[rt]);
         u[rt] = mfma16(fu[x], a[x][rt], u[rt]);
       }
   }
   for (; c < chunks; ++c) {
-    const Frag fg = load_frag_once(wg + (size_t)c * TILE_ELEMS), fu = load_frag_once(wu + (size_t)c * TILE_ELEMS);
+    const Frag fg = GATED ? load_frag_once(wg + (size_t)c * TILE_ELEMS) : zero_frag();
+    const Frag fu = load_frag_once(wu + (size_t)c * TILE_ELEMS);
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
       const Frag a = (on[rt] && (c < full || c * 32 + lc * 8 < D)) ? load_frag(arow[rt] + c * 32) : zero_frag();
-      g[rt] = mfma16(fg, a, g[rt]);
+      if (GATED) g[rt] = mfma16(fg, a, g[rt]);
       u[rt] = mfma16(fu, a, u[rt]);
     }
   }
@@ -153,7 +154,10 @@ __global__ __launch_bounds__(256) void routed_glu_bf16_kernel(const bf16_t* __re
     float v[4];
     const float w = in_weights ? in_weights[order[p0 + rt * 16 + li]] : 1.f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = unit_act(g[rt][r] * w, u[rt][r] * w, kind, alpha, limit);
+    for (int r = 0; r < 4; ++r) {
+      const float z = fmaxf(u[rt][r] * w, 0.f);
+      v[r] = GATED ? unit_act(g[rt][r] * w, u[rt][r] * w, kind, alpha, limit) : z * z;
+    }
     if (f0 + 4 <= F && F % 4 == 0) {
       uint2 pk;
       pk.x = pack_bf16x2(v[0], v[1]);
@@ -283,14 +287,15 @@ extern "C" int apc_gemm_grouped_bf16(const void* A, int lda, const void* W, cons
 
 // work: int32 [2 * n_pairs + 3 * max_tiles + 1] (order, place, tiles, the tiles' count); act: bfloat16 [n_pairs, F];
 // ys: float32 [n_pairs, D]; hs: bfloat16 [n_pairs, D] (tiles of 64 and 128 rows only).  tile_rows: 16, 64 or 128.
-// kind, alpha, limit: the activation (0: silu(g) * u; 1: the clamped unit), applied where gate and up are formed.
+// kind, alpha, limit: the activation (0: silu(g) * u; 1: the clamped unit; 2: experts without a gate, max(u, 0)^2, their
+// first matrices [E][bands(F)][chunks(D)][64][8]), applied where gate and up are formed.
 APC_EXPORT int apc_routed_experts_bf16(const void* h, int ldh, const void* w_gate_up, const void* w_down, int E, int F,
                                        int D, const int* ids, const float* weights, int K, int n_rows, int tile_rows,
                                        int* work, void* act, float* ys, void* hs, float* y, int ldy, int kind,
                                        float alpha, float limit, int in_weights, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (!apc_routed_bf16_takes(E, F, D)) return APC_ERR_UNSUPPORTED;
-  if (kind < 0 || kind > 1) return APC_ERR_BAD_ARG;
+  if (kind < 0 || kind > 2) return APC_ERR_BAD_ARG;
   if (K <= 0 || ldh < D || ldy < D || ldh % 8 || (tile_rows != 16 && tile_rows != 64 && tile_rows != 128) || !work ||
       !act || !ys || (tile_rows != 16 && (!hs || ((uintptr_t)hs & 15u))) ||
       ((uintptr_t)h & 15u) || ((uintptr_t)w_gate_up & 15u) || ((uintptr_t)w_down & 15u) || ((uintptr_t)act & 15u) ||
@@ -308,9 +313,13 @@ APC_EXPORT int apc_routed_experts_bf16(const void* h, int ldh, const void* w_gat
   const dim3 g1(max_tiles, ceil_div(ceil_div(F, 16), 4)), g2(max_tiles, ceil_div(ceil_div(D, 16), 4));
   if (g1.y > 65535 || g2.y > 65535) return APC_ERR_UNSUPPORTED;
   if (tile_rows == 16) {
-    hipLaunchKernelGGL(routed_glu_bf16_kernel<1>, g1, dim3(256), 0, stream, (const bf16_t*)h, ldh,
-                       (const bf16_t*)w_gate_up, F, D, order, K, tiles, n_tiles, (bf16_t*)act, kind, alpha, limit,
-                       in_weights ? weights : nullptr);
+#define GLU_LAUNCH(GATED_)                                                                                          \
+  hipLaunchKernelGGL((routed_glu_bf16_kernel<1, GATED_>), g1, dim3(256), 0, stream, (const bf16_t*)h, ldh,           \
+                     (const bf16_t*)w_gate_up, F, D, order, K, tiles, n_tiles, (bf16_t*)act, kind, alpha, limit,     \
+                     in_weights ? weights : nullptr)
+    if (kind == 2) GLU_LAUNCH(false);
+    else GLU_LAUNCH(true);
+#undef GLU_LAUNCH
     APC_LAUNCH_CHECK();
     hipLaunchKernelGGL(routed_down_bf16_kernel<1>, g2, dim3(256), 0, stream, (const bf16_t*)act, F, D,
                        (const bf16_t*)w_down, tiles, n_tiles, ys);
@@ -322,9 +331,11 @@ APC_EXPORT int apc_routed_experts_bf16(const void* h, int ldh, const void* w_gat
     APC_LAUNCH_CHECK();
     const size_t gate_elems = (size_t)ceil_div(F, 16) * ceil_div(D, 32) * TILE_ELEMS;
     const size_t down_elems = (size_t)ceil_div(D, 16) * ceil_div(F, 32) * TILE_ELEMS;
-    int e = apc_gemm_grouped_bf16(hs, D, w_gate_up, (const bf16_t*)w_gate_up + gate_elems, 2 * gate_elems, act, F,
-                                  tiles, n_tiles, max_tiles, tile_rows, F, D, /* gated unit */ 3, kind, alpha, limit,
-                                  stream);
+    int e = kind == 2 ? apc_gemm_grouped_bf16(hs, D, w_gate_up, nullptr, gate_elems, act, F, tiles, n_tiles, max_tiles,
+                                              tile_rows, F, D, /* squared relu */ 5, 0, 1.0f, 0.0f, stream)
+                      : apc_gemm_grouped_bf16(hs, D, w_gate_up, (const bf16_t*)w_gate_up + gate_elems, 2 * gate_elems,
+                                              act, F, tiles, n_tiles, max_tiles, tile_rows, F, D, /* gated unit */ 3,
+                                              kind, alpha, limit, stream);
     if (e) return e;
     e = apc_gemm_grouped_bf16(act, F, w_down, nullptr, down_elems, ys, D, tiles, n_tiles, max_tiles, tile_rows, D, F,
                               /* float32 out */ 1, 0, 1.0f, 0.0f, stream);

@@ -48,10 +48,15 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_linear_attention": [P, I, I, I, I, I, I, I, I, I, P, P, I, P, P, P, P, I, I, P, P, F, P],
         "apc_gated_rmsnorm": [P, I, P, F, P, I, I, P, I, I, I, I, I, I, P],
         "apc_diff_combine": [P, I, F, F, F, P, I, I, P, I, I, I, I, I, P],
-        "apc_route_topk": [P, I, P, I, I, I, I, I, P, P, P],
+        "apc_route_topk": [P, I, P, I, I, I, I, I, I, I, F, P, P, P],
         "apc_routed_glu": [P, I, I, P, I, I, I, I, P, I, P, I, I, I, F, F, P, P],
         "apc_conv_channels": [P, I, I, I, I, P, P, I, P, P, P, P, I, P, I, I, P],
         "apc_selective_scan": [P, I, I, P, I, P, P, P, I, P, P, I, I, P, I, I, I, P, P, P, P, I, I, P],
+        "apc_heads_gemm_plain": [P, I, I, I, P, I, P, I, I, I, I, I, I, I, P],
+        "apc_latent_rows": [P, I, I, I, I, I, I, I, P, F, P, P, P, P, I, P, I, I, P, I, I, I, P],
+        "apc_latent_attention_plain": [P, I, I, P, I, I, I, I, I, I, P, I, I, P, I, P, P, F, P],
+        "apc_tanh_norm": [P, I, I, P, F, P, P, P, I, I, I, I, I, P],
+        "apc_tanh_norm_add": [P, I, P, I, I, F, P, P, F, P, P, P, I, I, I, I, I, P],
         "apc_act_rows": [P, I, I, P, I, I, I, I, I, P],
         "apc_bias_rows": [P, I, P, I, I, P],
         "apc_weighted_pair": [P, I, P, I, F, P, I, F, I, I, P],
@@ -91,6 +96,7 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_selective_scan_bf16": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, P, P, P, I, P, P, P, P, P, I, P],
         "apc_linear_rotate_bf16": [P, I, I, I, I, I, I, P, P, F, I, P],
         "apc_linear_attention_bf16": [P, I, I, I, I, I, I, I, I, P, P, I, P, P, P, I, P, P, P, P, I, P],
+        "apc_heads_gemm_bf16": [P, I, I, P, P, I, I, I, I, I, I, P],
         "apc_attention_masked_takes": [I, I, I, I, I, I],
         "apc_attention_masked_prefill_bf16": [P, I, P, I, I, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, P, P, I, F, I, I, F, P, P, P],
         "apc_attention_masked_decode_bf16": [P, I, P, I, I, I, I, I, I, P, I, P, I, P, P, P, I, I, I, P, P, I, F, I, P, I, I, F, P, P, P],

@@ -767,23 +767,30 @@ ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}
 
 
 def route_topk(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, ids: torch.Tensor,
-               weights: torch.Tensor, renormalize: bool = False, score: str = "softmax") -> None:
+               weights: torch.Tensor, renormalize: bool = False, score: str = "softmax", groups: int = 1,
+               keep_groups: int = 1, weight_scale: float = 1.0) -> None:
     """s = softmax(z) over a row (`score` "sigmoid": s = sigmoid(z), every output for itself); the `top` largest of s + correction are chosen (the lower index wins a tie);
-    weights = s of the chosen (divided by their sum with `renormalize`).  z float32 [rows, n]."""
+    weights = s of the chosen (divided by their sum with `renormalize`) times `weight_scale`.  z float32 [rows, n].
+    `groups` > 1: the outputs form that many equal runs of neighbours, a run's score is the sum of its two largest
+    s + correction, and only outputs of the `keep_groups` best runs can be chosen."""
     _gpu(z, correction, ids, weights)
     T, N = z.shape
     _need(z.dtype == torch.float32 and weights.dtype == torch.float32 and weights.is_contiguous()
           and weights.numel() >= T * top, "route_topk: z float32, weights contiguous float32 [rows, top]")
     _need(score in ROUTER_SCORES, f"route_topk: score {score!r} is not one of {sorted(ROUTER_SCORES)}")
+    _need(1 <= keep_groups <= groups and N % groups == 0 and top <= keep_groups * (N // groups),
+          f"route_topk: top {top} of {keep_groups} of {groups} groups of {N} outputs")
     L = _lib.load("plain")
     _lib.check(L.apc_route_topk(z.data_ptr(), _rows(z, "router logits"), _f32(correction, N, "correction"), T, N,
-                                int(top), 1 if renormalize else 0, ROUTER_SCORES[score], _i32(ids, T * top, "ids"),
-                                weights.data_ptr(), _stream()), "route_topk")
+                                int(top), 1 if renormalize else 0, ROUTER_SCORES[score], int(groups), int(keep_groups),
+                                float(weight_scale), _i32(ids, T * top, "ids"), weights.data_ptr(), _stream()),
+               "route_topk")
 
 
 def prepare_experts(gate_up: torch.Tensor, down: torch.Tensor, run_dtype: torch.dtype):
-    """How the experts' matrices [experts, 2 ff, width] and [experts, width, ff] are kept on the GPU: in the tiled
-    layout of the MFMA kernels for a bfloat16 run whose sizes they take, else as they are."""
+    """How the experts' matrices [experts, 2 ff, width] ([experts, ff, width] without a gate) and [experts, width, ff]
+    are kept on the GPU: in the tiled layout of the MFMA kernels for a bfloat16 run whose sizes they take, else as they
+    are."""
     if run_dtype == torch.bfloat16 and not FORCE_PLAIN and gate_up.is_cuda and gate_up.dtype == torch.bfloat16:
         from . import tuned
         packed = tuned.pack_experts(gate_up, down)
@@ -792,7 +799,8 @@ def prepare_experts(gate_up: torch.Tensor, down: torch.Tensor, run_dtype: torch.
     return gate_up.contiguous(), down.contiguous()
 
 
-EXPERT_ACTIVATIONS = {"silu": 0, "clamped": 1}
+EXPERT_ACTIVATIONS = {"silu": 0, "clamped": 1, "relu2": 2}
+UNGATED_EXPERTS = {"relu2"}      # an expert of these activations is two matrices, Wd a(Wu h)
 
 
 def routed_experts(h: torch.Tensor, w_gate_up, w_down, n_experts: int, ff: int, ids: torch.Tensor,
@@ -802,14 +810,15 @@ def routed_experts(h: torch.Tensor, w_gate_up, w_down, n_experts: int, ff: int, 
     Wd a(Wg h, Wu h) with w_gate_up [n_experts, 2 * ff, width] (gate rows, then up rows) and w_down
     [n_experts, width, ff]; ids from n_experts on are identity experts.  y float32 [rows, width].
     `activation` "silu": a(g, u) = silu(g) * u; "clamped": g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit),
-    u' = clamp(u, -limit, limit).  `weight_input`: the weight multiplies the expert's input instead of its output,
+    u' = clamp(u, -limit, limit); "relu2": experts without a gate, Wd max(Wu h, 0)^2 with w_gate_up [n_experts, ff,
+    width].  `weight_input`: the weight multiplies the expert's input instead of its output,
     y[t] = sum_k expert(weights[t][k] * h[t]) (identity experts then return the weighted row as well)."""
     T, D = h.shape
     E, F, K = int(n_experts), int(ff), int(top)
     _gpu(h, ids, weights, y)
     _need(y.dtype == torch.float32 and y.shape == (T, D), "routed_experts: y float32 [rows, width]")
     _need(activation in EXPERT_ACTIVATIONS, f"routed_experts: activation {activation!r} is not one of {sorted(EXPERT_ACTIVATIONS)}")
-    kind = EXPERT_ACTIVATIONS[activation]
+    kind, n_up = EXPERT_ACTIVATIONS[activation], 1 if activation in UNGATED_EXPERTS else 2
     if not isinstance(w_gate_up, torch.Tensor) and w_gate_up is not None:
         from . import tuned
         tuned.routed_experts_bf16(h, w_gate_up, w_down, E, F, ids, weights, K, y, kind, alpha, limit, weight_input)
@@ -818,7 +827,7 @@ def routed_experts(h: torch.Tensor, w_gate_up, w_down, n_experts: int, ff: int, 
     L = _lib.load("plain")
     if E:
         _gpu(w_gate_up, w_down)
-        _need(w_gate_up.is_contiguous() and tuple(w_gate_up.shape) == (E, 2 * F, D) and w_down.is_contiguous()
+        _need(w_gate_up.is_contiguous() and tuple(w_gate_up.shape) == (E, n_up * F, D) and w_down.is_contiguous()
               and tuple(w_down.shape) == (E, D, F), "routed_experts: matrices [experts, 2 ff, width] and [experts, width, ff]")
         _lib.check(L.apc_routed_glu(h.data_ptr(), _code(h), _rows(h, "h"), w_gate_up.data_ptr(), _code(w_gate_up), E, F,
                                     D, _i32(ids, T * K, "ids"), K, act.data_ptr(), _code(act), T, kind, float(alpha),
@@ -937,3 +946,125 @@ def linear_act(a: torch.Tensor, w, out: torch.Tensor, activation: str) -> None:
     sums = torch.empty((T, n), dtype=torch.float32, device=a.device)
     linear(a, w, sums)
     act_rows(sums, out, activation)
+
+
+# --------------------------------------------------------------------------- tanh norm, attention over cached latents
+def tanh_norm(x: torch.Tensor, norm: tuple, out: torch.Tensor, rows: Optional[torch.Tensor] = None,
+              exact: bool = True) -> None:
+    """out[r] = tanh(alpha * x[r]) * w + b with norm = (alpha, w, b) (of x[rows[r]] with `rows`), in 32-bit.  `exact`:
+    the library's tanh; otherwise one exponential, off by about 1e-7 (bfloat16 runs)."""
+    alpha, w, b = norm
+    _gpu(x, w, b, out, rows)
+    ldx, ldo = _rows(x, "tanh_norm x"), _rows(out, "tanh_norm out")
+    R, D = out.shape[0], x.shape[1]
+    _need(out.shape[1] == D and (x.shape[0] == R if rows is None else True), "tanh_norm: out must be [rows, width]")
+    L = _lib.load("plain")
+    _lib.check(L.apc_tanh_norm(x.data_ptr(), _code(x), ldx, _i32(rows, R, "rows"), float(alpha), _f32(w, D, "norm weight"),
+                               _f32(b, D, "norm bias"), out.data_ptr(), _code(out), ldo, R, D, 1 if exact else 0,
+                               _stream()), "tanh_norm")
+
+
+def tanh_norm_add(x: torch.Tensor, y: torch.Tensor, post: tuple, then: Optional[tuple] = None,
+                  h: Optional[torch.Tensor] = None, exact: bool = True) -> None:
+    """x += tanh(pa * y) * pw + pb with post = (pa, pw, pb), x float32; with then = (alpha, w, b) also
+    h = tanh(alpha * x) * w + b of the new x: one pass over the row."""
+    _gpu(x, y, *post[1:], h)
+    ldx, ldy = _rows(x, "tanh_norm_add x"), _rows(y, "tanh_norm_add y")
+    T, D = x.shape
+    _need(x.dtype == torch.float32 and y.shape == (T, D), "tanh_norm_add: x float32 [rows, width], y of the same shape")
+    _need((then is None) == (h is None) and (h is None or h.shape == (T, D)), "tanh_norm_add: h goes with the next norm")
+    alpha, w, b = then if then is not None else (1.0, None, None)
+    L = _lib.load("plain")
+    _lib.check(L.apc_tanh_norm_add(x.data_ptr(), ldx, y.data_ptr(), _code(y), ldy, float(post[0]),
+                                   _f32(post[1], D, "norm weight"), _f32(post[2], D, "norm bias"), float(alpha),
+                                   _f32(w, D, "next norm's weight"), _f32(b, D, "next norm's bias"),
+                                   h.data_ptr() if h is not None else 0, _code(h) if h is not None else 0,
+                                   _rows(h, "tanh_norm_add h") if h is not None else 0, T, D, 1 if exact else 0,
+                                   _stream()), "tanh_norm_add")
+
+
+def prepare_heads(w: torch.Tensor, run_dtype: torch.dtype, a_head: int, out_head: int):
+    """How a matrix of its own for every head, [heads, out, in], is kept on the GPU for `heads_linear` with these
+    `a_head` and `out_head`: tiled for the MFMA kernels in a bfloat16 run whose sizes they take, else as it is."""
+    if run_dtype == torch.bfloat16 and not FORCE_PLAIN and w.is_cuda and w.dtype == torch.bfloat16:
+        from . import tuned
+        packed = tuned.pack_heads(w, int(a_head), int(out_head))
+        if packed is not None:
+            return packed
+    return w.contiguous()
+
+
+def heads_linear(a: torch.Tensor, a_head: int, w, out: torch.Tensor, out_head: int) -> None:
+    """out[t, h * out_head + n] = sum_k a[t, h * a_head + k] w[h, n, k] for every head h; w [heads, n, k] or its tiled
+    form (`prepare_heads`)."""
+    if not isinstance(w, torch.Tensor):
+        from . import tuned
+        tuned.heads_linear_bf16(a, a_head, w, out, out_head)
+        return
+    _gpu(a, w, out)
+    lda, ldo = _rows(a, "heads_linear a"), _rows(out, "heads_linear out")
+    T = a.shape[0]
+    H, N, K = w.shape
+    _need(w.is_contiguous() and out.shape[0] == T and a_head >= K and out_head >= N and (H - 1) * a_head + K <= a.shape[1]
+          and (H - 1) * out_head + N <= out.shape[1], "heads_linear: head ranges exceed the rows")
+    L = _lib.load("plain")
+    _lib.check(L.apc_heads_gemm_plain(a.data_ptr(), _code(a), lda, int(a_head), w.data_ptr(), _code(w), out.data_ptr(),
+                                      _code(out), ldo, int(out_head), T, H, N, K, _stream()), "heads_gemm_plain")
+
+
+def _latent_pages(pages: torch.Tensor, row: int, page_tokens: int, block_table: torch.Tensor) -> None:
+    if not (pages.dim() == 3 and pages.is_contiguous() and tuple(pages.shape[1:]) == (page_tokens, row)):
+        raise ValueError(f"pages must be [pages, {page_tokens}, {row}], got {tuple(pages.shape)}")
+    _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.is_contiguous(),
+          "block table must be contiguous int32 [segments, blocks]")
+
+
+def latent_rows(proj: torch.Tensor, n_heads: int, head_dim: int, rot_dim: int, c_off: Optional[int], rank: int,
+                norm_w: Optional[torch.Tensor], eps: float, cos_sin: Optional[torch.Tensor], step,
+                block_table: torch.Tensor, pages: torch.Tensor, page_tokens: int, q_out: torch.Tensor) -> None:
+    """Query head h of a row: proj[:, h * (head_dim + rot_dim) ...], whose last rot_dim elements are rotated by the row's
+    position (pairs i, i + rot_dim/2; cos_sin float32 [positions, 2, rot_dim/2]) and go to the end of head h of q_out
+    [rows, heads * (rank + rot_dim)].  With `c_off`: proj[:, c_off : c_off + rank] divided by its root mean square and
+    multiplied with norm_w, and the rot_dim elements behind it, rotated, go into the row's slot of its page
+    [slot][rank + rot_dim]."""
+    _gpu(proj, norm_w, cos_sin, block_table, pages, q_out)
+    T, H, dn, dr, R = proj.shape[0], int(n_heads), int(head_dim), int(rot_dim), int(rank)
+    ld, ldq = _rows(proj, "projected rows"), _rows(q_out, "latent queries")
+    _need(proj.shape[1] >= H * (dn + dr) and q_out.shape == (T, H * (R + dr)), "latent_rows: q heads exceed the row")
+    _need(c_off is None or (norm_w is not None and c_off + R + dr <= proj.shape[1]), "latent_rows: the latent exceeds the row")
+    _latent_pages(pages, R + dr, page_tokens, block_table)
+    if dr:
+        _need(dr % 2 == 0 and cos_sin is not None and cos_sin.dtype == torch.float32 and cos_sin.is_contiguous()
+              and cos_sin.dim() == 3 and tuple(cos_sin.shape[1:]) == (2, dr // 2),
+              "cos/sin table must be float32 [positions, 2, rot/2]")
+    L = _lib.load("plain")
+    _lib.check(L.apc_latent_rows(
+        proj.data_ptr(), _code(proj), ld, H, dn, dr, -1 if c_off is None else int(c_off), R, _f32(norm_w, R, "norm weight"),
+        float(eps), cos_sin.data_ptr() if dr else 0, _i32(step.positions, T, "positions"), _i32(step.row_seg, T, "row_seg"),
+        block_table.data_ptr(), block_table.shape[1], pages.data_ptr(), _code(pages), page_tokens, q_out.data_ptr(),
+        _code(q_out), ldq, T, _stream()), "latent_rows")
+
+
+def latent_attention_plain(q: torch.Tensor, out: torch.Tensor, n_heads: int, rank: int, rot_dim: int,
+                           pages: torch.Tensor, page_tokens: int, block_table: torch.Tensor, positions: torch.Tensor,
+                           row_seg: torch.Tensor, scale: float) -> None:
+    _gpu(q, out, pages, block_table, positions, row_seg)
+    T, H, R, dr = q.shape[0], int(n_heads), int(rank), int(rot_dim)
+    ldq, ldo = _rows(q, "attention q"), _rows(out, "attention out")
+    _need(q.shape[1] == H * (R + dr) and out.shape == (T, H * R), "latent attention: q [rows, heads * (rank + rot_dim)], "
+          "out [rows, heads * rank]")
+    _latent_pages(pages, R + dr, page_tokens, block_table)
+    L = _lib.load("plain")
+    _lib.check(L.apc_latent_attention_plain(
+        q.data_ptr(), _code(q), ldq, out.data_ptr(), _code(out), ldo, T, H, R, dr, pages.data_ptr(), _code(pages),
+        page_tokens, block_table.data_ptr(), block_table.shape[1], _i32(positions, T, "positions"),
+        _i32(row_seg, T, "row_seg"), float(scale), _stream()), "latent_attention_plain")
+
+
+def latent_attention(q: torch.Tensor, out: torch.Tensor, n_heads: int, rank: int, rot_dim: int, pages: torch.Tensor,
+                     page_tokens: int, block_table: torch.Tensor, step, scale: float) -> None:
+    """Causal softmax attention of every head over the cached rows [latent | rotated part] of its request: scores
+    (q_h . row) * scale with q_h = q[:, h * (rank + rot_dim) ...], out[:, h * rank ...] = sum of weights times the rows'
+    first `rank` elements."""
+    latent_attention_plain(q, out, n_heads, rank, rot_dim, pages, page_tokens, block_table, step.positions, step.row_seg,
+                           scale)

@@ -606,8 +606,8 @@ class PackedExperts:
     """The matrices of a layer's experts in the tiled layout of the MFMA kernels: `data` holds, for every expert, the
     tiles of its matrices (`per_expert` of them: gate and up, or down alone), each packed like a `PackedWeight`."""
 
-    def __init__(self, data: torch.Tensor, n_experts: int, N: int, K: int):
-        self.data, self.E, self.N, self.K = data, n_experts, N, K
+    def __init__(self, data: torch.Tensor, n_experts: int, N: int, K: int, per_expert: int = 1):
+        self.data, self.E, self.N, self.K, self.per_expert = data, n_experts, N, K, per_expert
 
 
 # pairs an expert on average from which a row tile holds 64 and 128 rows instead of 16 (and the products run on the
@@ -616,16 +616,18 @@ ROUTED_TILE_64_MIN, ROUTED_TILE_128_MIN = 24, 96
 
 
 def pack_experts(gate_up: torch.Tensor, down: torch.Tensor):
-    """[E, 2 F, D] and [E, D, F] bfloat16 -> (PackedExperts, PackedExperts), or None for sizes the kernels do not take."""
+    """[E, 2 F, D] (gate rows, then up rows; [E, F, D] for experts without a gate) and [E, D, F] bfloat16 ->
+    (PackedExperts, PackedExperts), or None for sizes the kernels do not take."""
     from .packing import pack_mfma
-    E, F2, D = gate_up.shape
-    F = F2 // 2
+    E, D, F = down.shape
+    gated = gate_up.shape[1] == 2 * F
     if not _lib.load("tuned").apc_routed_bf16_takes(E, F, D):
         return None
-    gu = torch.stack([torch.stack([pack_mfma(gate_up[e, :F].contiguous()).data,
-                                   pack_mfma(gate_up[e, F:].contiguous()).data]) for e in range(E)]).contiguous()
+    firsts = (slice(0, F), slice(F, 2 * F)) if gated else (slice(0, F),)
+    gu = torch.stack([torch.stack([pack_mfma(gate_up[e, s].contiguous()).data for s in firsts])
+                      for e in range(E)]).contiguous()
     dn = torch.stack([pack_mfma(down[e].contiguous()).data for e in range(E)]).contiguous()
-    return PackedExperts(gu, E, F, D), PackedExperts(dn, E, D, F)
+    return PackedExperts(gu, E, F, D, len(firsts)), PackedExperts(dn, E, D, F)
 
 
 def routed_experts_bf16(h, w_gate_up: PackedExperts, w_down: PackedExperts, E: int, F: int, ids, weights, K: int,
@@ -635,7 +637,7 @@ def routed_experts_bf16(h, w_gate_up: PackedExperts, w_down: PackedExperts, E: i
     T, D = h.shape
     _ops._gpu(h, w_gate_up.data, w_down.data, ids, weights, y)
     _ops._need(h.dtype == torch.bfloat16 and (w_gate_up.E, w_gate_up.N, w_gate_up.K) == (E, F, D)
-               and (w_down.E, w_down.N, w_down.K) == (E, D, F), "routed experts: matrices do not fit the sizes")
+               and (w_down.E, w_down.N, w_down.K) == (E, D, F) and w_gate_up.per_expert == (1 if kind == 2 else 2), "routed experts: matrices do not fit the sizes")
     L = _lib.load("tuned")
     n_pairs = T * K
     tile_rows = 128 if n_pairs >= ROUTED_TILE_128_MIN * E else 64 if n_pairs >= ROUTED_TILE_64_MIN * E else 16
@@ -679,3 +681,35 @@ def rotary_pages_bf16(q, ldq, q_off, H, dq, q_rot0, q_out, ldqo, ka, ldka, ka_of
         block_table.shape[1], cache.data_ptr(), page_tokens, T, _ops._f32(q_norm_w, dq, "q norm weight"),
         _ops._f32(k_norm_w, da + db, "k norm weight"), float(norm_eps), _ops._stream()), "rotary_pages_bf16")
     return True
+
+
+# --------------------------------------------------------------------------- a matrix of its own for every head
+class PackedHeads:
+    """[heads, N, K] matrices in the tiled layout: `data` [heads, bands, chunks, 64, 8]."""
+
+    def __init__(self, data: torch.Tensor, H: int, N: int, K: int):
+        self.data, self.H, self.N, self.K = data, H, N, K
+
+
+def pack_heads(w: torch.Tensor, a_head: int, out_head: int):
+    """[H, N, K] bfloat16 -> PackedHeads, or None where the kernel does not take the heads' places in the rows (`a_head`
+    elements apart in the product's input, `out_head` in its output)."""
+    from .packing import can_pack, pack_mfma
+    if not can_pack(w[0]) or a_head % 8 or out_head % 4:
+        return None
+    H, N, K = w.shape
+    return PackedHeads(torch.stack([pack_mfma(w[h].contiguous()).data for h in range(H)]).contiguous(), H, N, K)
+
+
+def heads_linear_bf16(a: torch.Tensor, a_head: int, w: PackedHeads, out: torch.Tensor, out_head: int) -> None:
+    _ops._gpu(a, w.data, out)
+    lda, ldo = _ops._rows(a, "heads_linear a"), _ops._rows(out, "heads_linear out")
+    T = a.shape[0]
+    _ops._need(a.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and out.shape[0] == T
+               and (w.H - 1) * a_head + w.K <= a.shape[1] and (w.H - 1) * out_head + w.N <= out.shape[1],
+               "heads_linear: bfloat16 rows that hold the heads' ranges")
+    _ops._need(lda % 8 == 0 and ldo % 4 == 0 and _aligned(a) and out.data_ptr() % 8 == 0,
+               "heads_linear_bf16: rows of a stride that is a multiple of 8 (out: 4), aligned")
+    L = _lib.load("tuned")
+    _lib.check(L.apc_heads_gemm_bf16(a.data_ptr(), lda, int(a_head), w.data.data_ptr(), out.data_ptr(), ldo, int(out_head),
+                                     T, w.H, w.N, w.K, _ops._stream()), "heads_gemm_bf16")

@@ -8,6 +8,7 @@ does not know which model it is in.  It names the tensors it wants
 Interfaces
 ----------
 Norm            forward(x[T,D] float32 residual or activations, out[T,D]) ; forward_rows(x, rows, out)
+                add_normed(x, y, then, h): x += norm(y), h = then(x)
 PositionEncoding  table-driven rotation or any in-place transform of q and k by per-row positions
 Mixer           cache_need() -> PagedKV | FixedState | None
                 forward_add(h[T,D], step, cache, residual[T,D] float32): residual += mixer(h)
@@ -71,6 +72,20 @@ class PagedKeysValues:
 
     def page_shape(self, page_tokens: int) -> Tuple[int, ...]:
         return (self.kv_heads, page_tokens * (self.key_dim + self.value_dim))
+
+
+@dataclass(frozen=True)
+class PagedLatents:
+    """One row of `rank` + `rot_dim` elements a position, whatever the number of heads: the latent that keys and values
+    are formed from, then the rotated key part all heads share.  A page holds its positions' rows one after the other."""
+    rank: int
+    rot_dim: int
+    window: Optional[int] = None
+    kind = "pages"
+    dtype = None
+
+    def page_shape(self, page_tokens: int) -> Tuple[int, ...]:
+        return (page_tokens, self.rank + self.rot_dim)
 
 
 @dataclass(frozen=True)
@@ -143,6 +158,17 @@ class Norm(Part):
         """(weight, eps) if this norm is x / sqrt(mean(x^2) + eps) * weight, which the products around it can
         fold in; None for any other norm."""
         return None
+
+    def add_normed(self, x: torch.Tensor, y: torch.Tensor, then: Optional["Norm"] = None,
+                   h: Optional[torch.Tensor] = None) -> None:
+        """x += norm(y) in 32-bit (x [T,D] float32); with `then`, also h = then(new x).  A norm that has a kernel for
+        both overrides this."""
+        from ..kernels import ops
+        z = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+        self.forward(y, z)
+        ops.add_into(x, z)
+        if then is not None:
+            then.forward(x, h)
 
 
 class NormEmit:

@@ -80,15 +80,16 @@ class Block:
 
 
 class NormedLeft:
-    """What a pre-norm layer with a scaled sum leaves for the next one: the next layer's first input, already
-    normalised (the sum of this layer's last output and that norm are one pass over the row)."""
+    """What a layer whose last sum is fused with a norm (pre-norm with a scaled sum, or norms on both sides of a
+    sublayer) leaves for the next one: the next layer's first input, already normalised (the sum of this layer's last
+    output and that norm are one pass over the row)."""
 
     def __init__(self, norm, h: torch.Tensor):
         self.norm, self.h = norm, h
 
 
 class ScaledFirst:
-    """What such a layer shows the layer before it: the norm of its first read."""
+    """What such a layer shows the layer before it: the norm of its first read, which is given as a `NormedLeft`."""
 
     def __init__(self, norm):
         self.norm = norm
@@ -300,3 +301,43 @@ class SublayerNorm:
             h = copy() if wants else None
             ops.rmsnorm_add(y, w, eps, mult, x, h)
         return RowsLeft(h) if (wants and narrow) else None
+
+
+@ARRANGEMENTS.register("sandwich_norm")
+class SandwichNorm:
+    """A norm ahead of each sublayer and one on its output:
+       x <- x + post1(mixer(norm1(x)));  x <- x + post2(ffn(norm2(x)))      (a layer may have no feed-forward)
+    The output's norm, the sum and the norm of whoever reads x next are `Norm.add_normed`: one kernel where the norms
+    have one."""
+    registries = {"mixer_norm": NORMS, "mixer": MIXERS, "mixer_post": NORMS,
+                  "ffn_norm": NORMS, "ffn": FEED_FORWARDS, "ffn_post": NORMS}
+    chains_norms = True
+
+    @staticmethod
+    def first_norm(parts):
+        return ScaledFirst(parts["mixer_norm"])
+
+    @staticmethod
+    def run(parts, x: torch.Tensor, step, cache, pre=None, next_norm=None):
+        mixer, ffn, norm1 = parts["mixer"], parts.get("ffn"), parts["mixer_norm"]
+        rt = mixer.rt
+
+        def buffer():
+            return torch.empty(x.shape, dtype=rt.dtype, device=x.device)
+
+        if isinstance(pre, NormedLeft) and pre.norm is norm1:
+            h = pre.h
+        else:
+            h = buffer()
+            norm1.forward(x, h)
+        y, post = mixer.forward(h, step, cache), parts["mixer_post"]
+        if ffn is not None:
+            h = buffer()
+            post.add_normed(x, y, parts["ffn_norm"], h)
+            y, post = ffn.forward(h, step), parts["ffn_post"]
+        if isinstance(next_norm, ScaledFirst):
+            h = buffer()
+            post.add_normed(x, y, next_norm.norm, h)
+            return NormedLeft(next_norm.norm, h)
+        post.add_normed(x, y)
+        return None
