@@ -1,0 +1,447 @@
+// Attention of all heads over cached latents, bfloat16 on MFMA with float32 softmax.
+//
+//   A position's cached row is [c | kr]: R + dr elements, one row for all heads.  Head h of a row of the step has a query
+//   of the same size;  s = (q . row) * scale over the positions up to the row's own;  out = sum softmax(s) * row[:R].
+//   Pages: [slot][R + dr], a page is P * (R + dr) elements.
+//
+// (row of the step, head) pairs are one axis: pair = row * H + head, and the queries are a [pairs][R + dr] matrix as they
+// lie.  Since every head reads the same keys, a block takes any PT * 32 consecutive pairs of one request (two rows of 32
+// heads, 8 rows of 8, 32 of the heads of one decoded row), and keys are shared by all of them.  The values are the keys'
+// first R elements: a tile of keys is brought into LDS once and read twice, along the row for the scores and across the
+// rows, by the LDS's transposing read, for the values.
+//
+// A tile of 64 keys lies in LDS as blocks of 32 elements: [block][key][64 bytes], the 16-byte piece p of key t at place
+// p ^ ((t / 4) % 4).  Direct loads fill it 1 KiB an instruction (16 keys x 64 bytes; a lane keeps the address of its key's
+// row for the whole tile), operand reads of 16 keys and transposing reads of 4 keys x 32 elements are free of bank
+// conflicts, and nothing is padded.  Two such buffers take turns: the loads of a tile run during the pass before.
+// The direct loads are written as instructions: left to the compiler, every LDS read behind one waits until all of them
+// have landed (it cannot tell that they fill the other buffer).  What keeps reads and loads apart are the barriers of a
+// pass: a buffer is filled behind the barrier that all its readers have passed, and read behind one that stands behind
+// `vmcnt(0)` of every wave.
+//
+// A pass over a tile, 4 waves:
+//   scores   S^T = K Q^T on 16 x 16 x 32: a wave PT * 16 keys x 32 pairs; its queries stay in registers
+//   maxima   of the tile through LDS (every wave of a pair group has some of its keys); the reference a score is
+//            subtracted from moves only when a maximum exceeds it by more than 2^8, and only then are sums rescaled
+//   weights  exp to LDS in bfloat16, [pair][key]
+//   values   O^T += V^T P^T on 32 x 32 x 16: a wave every fourth block of 32 value elements, all pairs
+// The keys of an item may be cut into ranges of whole tiles, a block each (decoded rows; few prompt rows over many keys):
+// a block then leaves O, its reference and its sum in 32 bits, and `latent_merge_kernel` adds the ranges.
+#include "mfma.h"
+#include <math.h>
+
+namespace {
+
+constexpr int KT = 64;                 // keys a tile
+constexpr int PROW = KT + 8;           // bfloat16 elements of a pair's row of weights in LDS
+constexpr float RISE = 8.f;            // by how much (in powers of 2) a score may exceed its pair's reference
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr float NO_KEY = -1e30f;
+
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) s16x4* lds_s16x4;
+
+struct LatentItems {
+  const int* row0;      // first row of every item (null: item i is row i)
+  const int* rows;      // its rows (null: 1)
+  int n;                // items
+  int blocks;           // blocks an item (for the item with the most rows)
+};
+
+// everything of this wave in LDS, then the block; `asm volatile` with a memory clobber keeps the compiler's accesses on
+// their side
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+// the same behind this wave's direct loads
+__device__ __forceinline__ void loads_barrier() { asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// 16 bytes a lane from `src` (a lane's own address) to LDS at `lds` + 16 * lane (the same `lds` for the wave).  m0 is a
+// register the compiler sets right ahead of an instruction of its own that reads it and never keeps anything in.
+__device__ __forceinline__ void load_to_lds(const bf16_t* src, int lds) {
+  asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(src), "s"(lds));
+}
+__device__ __forceinline__ int lds_address(const void* p) {
+  return (int)(uintptr_t)(const __attribute__((address_space(3))) void*)p;
+}
+
+// c = a . q and c += a . q with q, the queries of the wave's pairs, which only these read, in accumulation registers:
+// 8 NB registers of them, beside O in the vector registers, where a rescaling wants it.  Written as instructions, because
+// left to itself the compiler copies them there in every pass; it does not know the instruction, so what waits for the
+// results is `scores_done`.
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ void mfma16_set(floatx4& c, const Frag& a, const u32x4& q) {
+  asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, 0" : "=&v"(c) : "v"(__builtin_bit_cast(u32x4, a)), "a"(q));
+}
+__device__ __forceinline__ void mfma16_add(floatx4& c, const Frag& a, const u32x4& q) {
+  asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+v"(c) : "v"(__builtin_bit_cast(u32x4, a)), "a"(q));
+}
+template <int PT>
+__device__ __forceinline__ void scores_done(floatx4 (&s)[PT][2]) {
+  if constexpr (PT == 1) asm volatile("s_nop 15\n\ts_nop 3" : "+v"(s[0][0]), "+v"(s[0][1]));
+  else asm volatile("s_nop 15\n\ts_nop 3" : "+v"(s[0][0]), "+v"(s[0][1]), "+v"(s[1][0]), "+v"(s[1][1]));
+}
+// nothing moves across: LDS reads stay as far ahead of what takes them as they are written
+__device__ __forceinline__ void in_order() { __builtin_amdgcn_sched_barrier(0); }
+
+// RT: blocks of 32 value elements, NB: blocks of 32 elements of a row, PT: 32-pair groups a block of threads takes
+template <int RT, int NB, int PT>
+__global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
+    const bf16_t* __restrict__ q, bf16_t* __restrict__ out, int H, int R, int L, const bf16_t* __restrict__ pages,
+    int pshift, const int* __restrict__ block_table, int max_blocks, const int* __restrict__ positions,
+    const int* __restrict__ row_seg, LatentItems items, int n_splits, float scale2, float* __restrict__ parts,
+    float* __restrict__ ml) {
+  static_assert(PT == 1 || PT == 2, "a wave's scores are PT * 16 keys x 32 pairs");
+  constexpr int NP = PT * 32, NG = 4 / PT;      // pairs of a block; waves that share a pair's keys
+  constexpr int NV = (RT + 3) / 4;              // value blocks a wave
+  __shared__ __attribute__((aligned(1024))) bf16_t buf0[NB * KT * 32];
+  __shared__ __attribute__((aligned(1024))) bf16_t buf1[NB * KT * 32];
+  __shared__ __attribute__((aligned(16))) bf16_t ps[NP * PROW];
+  __shared__ float mx[NG * NP];
+  const int lane = threadIdx.x % WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+  const int li = lane % 16, lc = lane / 16, l32 = lane % 32, hh = lane / 32;
+
+  const int split = blockIdx.x % n_splits, rest = blockIdx.x / n_splits;
+  const int item = items.n - 1 - rest / items.blocks;            // (later rows of a prompt see more keys: they go first)
+  const int row0 = items.row0 ? items.row0[item] : item;
+  const int n_pairs = (items.rows ? items.rows[item] : 1) * H;
+  const int pair0 = (rest % items.blocks) * NP;
+  if (pair0 >= n_pairs) return;
+  const int pos0 = positions[row0];
+  const int* bt = block_table + (size_t)row_seg[row0] * max_blocks;
+  const int last = pos0 + (min(pair0 + NP, n_pairs) - 1) / H;     // the last key any pair of the block sees
+  const int first_last = pos0 + pair0 / H;                        // ... and the last one that all of them see
+  const int n_tiles = last / KT + 1, per = (n_tiles + n_splits - 1) / n_splits;
+  const int j0 = split * per, j1 = min(j0 + per, n_tiles);
+
+  const int kb = PT == 1 ? wave * 16 : (wave % 2) * 32, pb = PT == 1 ? 0 : (wave / 2) * 32;
+  const int group = PT == 1 ? wave : wave % 2;
+  // this lane's pairs of the scores: pb + li and pb + 16 + li
+  u32x4 qf[2][NB];
+  int posq[2];
+#pragma unroll
+  for (int p = 0; p < 2; ++p) {
+    const int pair = min(pair0 + pb + p * 16 + li, n_pairs - 1);
+    posq[p] = pos0 + pair / H;
+    const bf16_t* src = q + ((size_t)row0 * H + pair) * L;
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int e = b * 32 + lc * 8;
+      Frag f = load_frag(src + min(e, L - 8));
+#pragma unroll
+      for (int k = 0; k < 4; ++k) f.w[k] = e < L ? f.w[k] : 0u;
+      qf[p][b] = __builtin_bit_cast(u32x4, f);
+    }
+  }
+#pragma unroll
+  for (int p = 0; p < 2; ++p)
+#pragma unroll
+    for (int b = 0; b < NB; ++b) asm volatile("" : "+a"(qf[p][b]));
+
+  // direct loads: this wave brings keys 16 wave .. + 15 of a tile; a lane the piece (lane % 4) ^ (lane / 16) of every
+  // block of key 16 wave + lane / 4.  Pieces behind the row's end bring the row's first one, whose products meet zeros.
+  const int key_of_lane = wave * 16 + lane / 4, piece = (lane % 4) ^ lc;
+  auto row_of = [&](int j, int page) {
+    const int t = min(j * KT + key_of_lane, last);
+    return pages + (((size_t)page << pshift) + (t & ((1 << pshift) - 1))) * L;
+  };
+  auto page_of = [&](int j) { return bt[min(j * KT + key_of_lane, last) >> pshift]; };
+  auto fill = [&](const bf16_t* dst, const bf16_t* row) {
+    const int at = __builtin_amdgcn_readfirstlane(lds_address(dst) + wave * 1024);
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int e = b * 32 + piece * 8;
+      load_to_lds(row + (e < L ? e : 0), at + b * (KT * 64));
+    }
+  };
+
+  floatx16 o[NV][PT];
+#pragma unroll
+  for (int v = 0; v < NV; ++v)
+#pragma unroll
+    for (int t = 0; t < PT; ++t)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) o[v][t][r] = 0.f;
+  float m[2] = {NO_KEY, NO_KEY}, l[2] = {0.f, 0.f};     // of the pairs of the scores
+  float mo[PT];                                         // the same references for the pairs t * 32 + l32 of O
+#pragma unroll
+  for (int t = 0; t < PT; ++t) mo[t] = NO_KEY;
+
+  const int k_at = (kb + li) * 32 + (lc ^ (li / 4)) * 8;                // element in a block of 32 x 64 keys
+  const int v_col = ((lane / 16) % 2) * 2 + (lane % 4) / 2;             // the 16-byte piece of this lane's 4 elements
+  const int v_key = 8 * hh + (lane % 16) / 4;
+  const int v_at0 = v_key * 32 + (v_col ^ (2 * hh)) * 8 + (lane % 2) * 4;
+  const int v_at1 = (v_key + 4) * 32 + (v_col ^ (2 * hh + 1)) * 8 + (lane % 2) * 4;
+
+  int next_page = 0;
+  auto pass = [&](bf16_t* cur, bf16_t* nxt, int j) {
+    if (j + 1 < j1) {
+      fill(nxt, row_of(j + 1, next_page));
+      if (j + 2 < j1) next_page = page_of(j + 2);
+    }
+    // scores
+    floatx4 s[PT][2];
+    {
+      constexpr int N = NB * PT, AHEAD = N < 6 ? N : 6;
+      Frag kf[AHEAD];
+      auto key = [&](int i) {
+        return *reinterpret_cast<const Frag*>(cur + (i / PT) * (KT * 32) + (i % PT) * (16 * 32) + k_at);
+      };
+#pragma unroll
+      for (int i = 0; i < AHEAD; ++i) kf[i] = key(i);
+      in_order();
+#pragma unroll
+      for (int i = 0; i < N; ++i) {
+#pragma unroll
+        for (int p = 0; p < 2; ++p) {
+          if (i < PT) mfma16_set(s[i % PT][p], kf[i % AHEAD], qf[p][i / PT]);
+          else mfma16_add(s[i % PT][p], kf[i % AHEAD], qf[p][i / PT]);
+        }
+        if (i + AHEAD < N) kf[i % AHEAD] = key(i + AHEAD);
+        in_order();
+      }
+    }
+    scores_done<PT>(s);
+    const bool masked = j * KT + KT - 1 > first_last;
+    float tm[2];
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      tm[p] = -INFINITY;
+#pragma unroll
+      for (int kt = 0; kt < PT; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          float v = s[kt][p][r] * scale2;
+          if (masked && j * KT + kb + kt * 16 + lc * 4 + r > posq[p]) v = -INFINITY;
+          s[kt][p][r] = v;
+          tm[p] = fmaxf(tm[p], v);
+        }
+      tm[p] = fmaxf(tm[p], __shfl_xor(tm[p], 16, WAVE));
+      tm[p] = fmaxf(tm[p], __shfl_xor(tm[p], 32, WAVE));
+      if (lc == 0) mx[group * NP + pb + p * 16 + li] = tm[p];
+    }
+    lds_barrier();
+    bool rise = false;
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+#pragma unroll
+      for (int g = 0; g < NG; ++g) tm[p] = fmaxf(tm[p], mx[g * NP + pb + p * 16 + li]);
+      rise = rise || tm[p] > m[p] + RISE;
+    }
+    if (__any(rise)) {
+#pragma unroll
+      for (int p = 0; p < 2; ++p) {
+        const float mn = fmaxf(m[p], tm[p]);
+        l[p] *= __builtin_amdgcn_exp2f(m[p] - mn);
+        m[p] = mn;
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < PT; ++t) {
+      float to = mx[t * 32 + l32];
+#pragma unroll
+      for (int g = 1; g < NG; ++g) to = fmaxf(to, mx[g * NP + t * 32 + l32]);
+      if (__any(to > mo[t] + RISE)) {
+        const float mn = fmaxf(mo[t], to), f = __builtin_amdgcn_exp2f(mo[t] - mn);
+        mo[t] = mn;
+#pragma unroll
+        for (int v = 0; v < NV; ++v)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) o[v][t][r] *= f;
+      }
+    }
+    // weights
+#pragma unroll
+    for (int p = 0; p < 2; ++p)
+#pragma unroll
+      for (int kt = 0; kt < PT; ++kt) {
+        float w[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          w[r] = __builtin_amdgcn_exp2f(s[kt][p][r] - m[p]);
+          l[p] += w[r];
+        }
+        uint2 pk;
+        pk.x = pack_bf16x2(w[0], w[1]);
+        pk.y = pack_bf16x2(w[2], w[3]);
+        *reinterpret_cast<uint2*>(ps + (pb + p * 16 + li) * PROW + kb + kt * 16 + lc * 4) = pk;
+      }
+    lds_barrier();
+    // values: steps of one block of value elements over 16 keys, the weights of 16 keys shared by the blocks
+    {
+      constexpr int K = KT / 16, N = K * NV, AHEAD = N < 6 ? N : 6;
+      Frag vf[AHEAD], pf[2][PT];
+      auto weights = [&](int k) {
+#pragma unroll
+        for (int t = 0; t < PT; ++t)
+          pf[k % 2][t] = *reinterpret_cast<const Frag*>(ps + (t * 32 + l32) * PROW + k * 16 + hh * 8);
+      };
+      auto value = [&](int i) {
+        // (a wave without a block of its own reads another's and drops what it makes)
+        const bf16_t* base = cur + min(wave + 4 * (i % NV), RT - 1) * (KT * 32) + (i / NV) * (16 * 32);
+        const uint2 a = __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(base + v_at0)));
+        const uint2 b = __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(base + v_at1)));
+        Frag f;
+        f.w[0] = a.x; f.w[1] = a.y; f.w[2] = b.x; f.w[3] = b.y;
+        return f;
+      };
+      weights(0);
+#pragma unroll
+      for (int i = 0; i < AHEAD; ++i) vf[i] = value(i);
+      in_order();
+#pragma unroll
+      for (int i = 0; i < N; ++i) {
+        const int k = i / NV, v = i % NV;
+        if (v == 0 && k + 1 < K) weights(k + 1);
+#pragma unroll
+        for (int t = 0; t < PT; ++t) o[v][t] = mfma32(vf[i % AHEAD], pf[k % 2][t], o[v][t]);
+        if (i + AHEAD < N) vf[i % AHEAD] = value(i + AHEAD);
+        in_order();
+      }
+    }
+    loads_barrier();
+  };
+
+  if (j0 < j1) {
+    fill(buf0, row_of(j0, page_of(j0)));
+    if (j0 + 1 < j1) next_page = page_of(j0 + 1);
+    loads_barrier();
+    for (int j = j0; j < j1; j += 2) {
+      pass(buf0, buf1, j);
+      if (j + 1 < j1) pass(buf1, buf0, j + 1);
+    }
+  }
+  // sums of the pairs' weights over all their keys
+#pragma unroll
+  for (int p = 0; p < 2; ++p) {
+    l[p] += __shfl_xor(l[p], 16, WAVE);
+    l[p] += __shfl_xor(l[p], 32, WAVE);
+    if (lc == 0) mx[group * NP + pb + p * 16 + li] = l[p];
+  }
+  lds_barrier();
+#pragma unroll
+  for (int t = 0; t < PT; ++t) {
+    const int pair = pair0 + t * 32 + l32;
+    float sum = mx[t * 32 + l32];
+#pragma unroll
+    for (int g = 1; g < NG; ++g) sum += mx[g * NP + t * 32 + l32];
+    if (pair >= n_pairs) continue;
+    const size_t gp = (size_t)row0 * H + pair;
+    if (n_splits > 1) {
+      if (wave == 0 && hh == 0) {
+        ml[(gp * n_splits + split) * 2] = mo[t];
+        ml[(gp * n_splits + split) * 2 + 1] = sum;
+      }
+      if (j0 >= j1) continue;
+      float* dst = parts + (gp * n_splits + split) * R;
+#pragma unroll
+      for (int v = 0; v < NV; ++v)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+          const int r = (wave + 4 * v) * 32 + k * 8 + hh * 4;
+          if (r < R) *reinterpret_cast<floatx4*>(dst + r) =
+              floatx4{o[v][t][k * 4], o[v][t][k * 4 + 1], o[v][t][k * 4 + 2], o[v][t][k * 4 + 3]};
+        }
+    } else {
+      const float inv = 1.0f / sum;
+      bf16_t* dst = out + gp * R;
+#pragma unroll
+      for (int v = 0; v < NV; ++v)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+          const int r = (wave + 4 * v) * 32 + k * 8 + hh * 4;
+          if (r >= R) continue;
+          uint2 pk;
+          pk.x = pack_bf16x2(o[v][t][k * 4] * inv, o[v][t][k * 4 + 1] * inv);
+          pk.y = pack_bf16x2(o[v][t][k * 4 + 2] * inv, o[v][t][k * 4 + 3] * inv);
+          *reinterpret_cast<uint2*>(dst + r) = pk;
+        }
+    }
+  }
+}
+
+// a block: one pair of an item; 4 value elements a thread
+__global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ parts, const float* __restrict__ ml,
+                                                           int n_splits, int H, int R, LatentItems items,
+                                                           bf16_t* __restrict__ out) {
+  const int item = blockIdx.x / items.blocks, pair = blockIdx.x % items.blocks;
+  if (pair >= (items.rows ? items.rows[item] : 1) * H) return;
+  const size_t gp = (size_t)(items.row0 ? items.row0[item] : item) * H + pair;
+  const float* g = ml + gp * n_splits * 2;
+  float m = NO_KEY;
+  for (int s = 0; s < n_splits; ++s)
+    if (g[2 * s + 1] > 0.f) m = fmaxf(m, g[2 * s]);
+  float sum = 0.f;
+  for (int s = 0; s < n_splits; ++s)
+    if (g[2 * s + 1] > 0.f) sum += g[2 * s + 1] * __builtin_amdgcn_exp2f(g[2 * s] - m);
+  const float inv = 1.0f / sum;
+  for (int r = threadIdx.x * 4; r < R; r += 512) {
+    floatx4 acc = floatx4{0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < n_splits; ++s) {
+      if (!(g[2 * s + 1] > 0.f)) continue;              // a range without a key of this pair has left nothing
+      const float f = __builtin_amdgcn_exp2f(g[2 * s] - m);
+      const floatx4 v = *reinterpret_cast<const floatx4*>(parts + (gp * n_splits + s) * R + r);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) acc[k] = fmaf(f, v[k], acc[k]);
+    }
+    uint2 pk;
+    pk.x = pack_bf16x2(acc[0] * inv, acc[1] * inv);
+    pk.y = pack_bf16x2(acc[2] * inv, acc[3] * inv);
+    *reinterpret_cast<uint2*>(out + gp * R + r) = pk;
+  }
+}
+
+// the smallest kernel whose value blocks hold R elements and whose row blocks hold R + dr; 0: none
+int value_blocks(int R, int L) {
+  for (int rt = 2; rt <= 16; rt *= 2)
+    if (R <= rt * 32 && L <= (rt + 2) * 32) return rt;
+  return 0;
+}
+
+}  // namespace
+
+APC_EXPORT int apc_latent_attention_takes(int H, int R, int dr, int page_tokens) {
+  return (H > 0 && R > 0 && dr >= 0 && R % 8 == 0 && dr % 8 == 0 && value_blocks(R, R + dr) && page_tokens > 0 &&
+          (page_tokens & (page_tokens - 1)) == 0) ? 1 : 0;
+}
+
+// Items (row0 [n_items], rows [n_items] or null for single rows; max_rows: the most rows of one) of consecutive rows of
+// one request.  q [T][H * (R + dr)] and out [T][H * R] contiguous.  n_splits > 1: parts float32 [T * H][n_splits][R] and
+// ml float32 [T * H][n_splits][2].
+APC_EXPORT int apc_latent_attention_bf16(const void* q, void* out, int H, int R, int dr, const void* pages,
+                                         int page_tokens, const int* block_table, int max_blocks, const int* positions,
+                                         const int* row_seg, const int* row0, const int* rows, int n_items, int max_rows,
+                                         int n_splits, float* parts, float* ml, float scale, hipStream_t stream) {
+  if (n_items <= 0) return 0;
+  if (!apc_latent_attention_takes(H, R, dr, page_tokens)) return APC_ERR_UNSUPPORTED;
+  if (max_blocks <= 0 || max_rows <= 0 || n_splits < 1 || (n_splits > 1 && (!parts || !ml)) || (max_rows > 1 && !rows) ||
+      ((uintptr_t)q & 15u) || ((uintptr_t)out & 7u) || ((uintptr_t)pages & 15u) || ((uintptr_t)parts & 15u))
+    return APC_ERR_BAD_ARG;
+  const int L = R + dr, rt = value_blocks(R, L), pairs = max_rows * H;
+  const int two = pairs > 32 ? 1 : 0;
+  const int blocks = ceil_div(pairs, two ? 64 : 32);
+  if ((long)blocks * n_items * n_splits > 0x7fffffffL || (long)pairs * n_items > 0x7fffffffL) return APC_ERR_UNSUPPORTED;
+  const LatentItems items{row0, rows, n_items, blocks};
+  const int pshift = __builtin_ctz(page_tokens);
+#define LATENT_LAUNCH(RT_, PT_)                                                                                         \
+  hipLaunchKernelGGL((latent_attention_kernel<RT_, RT_ + 2, PT_>), dim3(blocks * n_items * n_splits), dim3(256), 0,     \
+                     stream, (const bf16_t*)q, (bf16_t*)out, H, R, L, (const bf16_t*)pages, pshift, block_table,        \
+                     max_blocks, positions, row_seg, items, n_splits, scale * LOG2E, parts, ml)
+#define LATENT_BY(RT_)               \
+  do {                               \
+    if (two) LATENT_LAUNCH(RT_, 2);  \
+    else LATENT_LAUNCH(RT_, 1);      \
+  } while (0)
+  if (rt == 2) LATENT_BY(2);
+  else if (rt == 4) LATENT_BY(4);
+  else if (rt == 8) LATENT_BY(8);
+  else LATENT_BY(16);
+#undef LATENT_BY
+#undef LATENT_LAUNCH
+  APC_LAUNCH_CHECK();
+  if (n_splits > 1) {
+    const LatentItems per_pair{row0, rows, n_items, pairs};
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(pairs * n_items), dim3(128), 0, stream, parts, ml, n_splits, H, R,
+                       per_pair, (bf16_t*)out);
+    APC_LAUNCH_CHECK();
+  }
+  return 0;
+}

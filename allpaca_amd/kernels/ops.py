@@ -1066,5 +1066,9 @@ def latent_attention(q: torch.Tensor, out: torch.Tensor, n_heads: int, rank: int
     """Causal softmax attention of every head over the cached rows [latent | rotated part] of its request: scores
     (q_h . row) * scale with q_h = q[:, h * (rank + rot_dim) ...], out[:, h * rank ...] = sum of weights times the rows'
     first `rank` elements."""
+    if _tuned_ok(q, out, pages):
+        from . import tuned
+        if tuned.latent_attention_bf16(q, out, n_heads, rank, rot_dim, pages, page_tokens, block_table, step, scale):
+            return
     latent_attention_plain(q, out, n_heads, rank, rot_dim, pages, page_tokens, block_table, step.positions, step.row_seg,
                            scale)

@@ -713,3 +713,50 @@ def heads_linear_bf16(a: torch.Tensor, a_head: int, w: PackedHeads, out: torch.T
     L = _lib.load("tuned")
     _lib.check(L.apc_heads_gemm_bf16(a.data_ptr(), lda, int(a_head), w.data.data_ptr(), out.data_ptr(), ldo, int(out_head),
                                      T, w.H, w.N, w.K, _ops._stream()), "heads_gemm_bf16")
+
+
+LATENT_BLOCKS = 256          # blocks that the keys of few rows are cut for (a block a compute unit at a latent of 512)
+LATENT_SPLITS_MAX = 32
+LATENT_RANGE_TILES = 8       # key tiles (of 64) that a range of a prompt tile's keys must keep
+
+
+def latent_attention_bf16(q, out, n_heads: int, rank: int, rot_dim: int, pages, page_tokens: int, block_table, step,
+                          scale: float) -> bool:
+    """Attention of all heads over cached latents on MFMA: tiles of prompt rows, then single rows.  False (nothing done)
+    for sizes the kernel does not take."""
+    _ops._gpu(q, out, pages, block_table)
+    T, H, R, dr = q.shape[0], int(n_heads), int(rank), int(rot_dim)
+    L = _lib.load("tuned")
+    if (q.dtype != torch.bfloat16 or pages.dtype != torch.bfloat16 or out.dtype != torch.bfloat16
+            or not q.is_contiguous() or not out.is_contiguous() or not _aligned(q, out, pages)
+            or not L.apc_latent_attention_takes(H, R, dr, page_tokens)):
+        return False
+    _ops._need(tuple(q.shape) == (T, H * (R + dr)) and tuple(out.shape) == (T, H * R), "latent attention: q [rows, heads * "
+               "(rank + rot_dim)], out [rows, heads * rank]")
+    _ops._latent_pages(pages, R + dr, page_tokens, block_table)
+    _ops._need(step.positions.numel() >= T and step.row_seg.numel() >= T, "step rows differ from q rows")
+
+    def run(row0, rows, n: int, max_rows: int, splits: int, what: str) -> None:
+        parts = ml = None
+        if splits > 1:
+            parts = torch.empty((T * H, splits, R), dtype=torch.float32, device=q.device)
+            ml = torch.empty((T * H, splits, 2), dtype=torch.float32, device=q.device)
+        _lib.check(L.apc_latent_attention_bf16(
+            q.data_ptr(), out.data_ptr(), H, R, dr, pages.data_ptr(), page_tokens, block_table.data_ptr(),
+            block_table.shape[1], step.positions.data_ptr(), step.row_seg.data_ptr(),
+            row0.data_ptr() if row0 is not None else 0, rows.data_ptr() if rows is not None else 0, n, max_rows, splits,
+            parts.data_ptr() if parts is not None else 0, ml.data_ptr() if ml is not None else 0, float(scale),
+            _ops._stream()), what)
+
+    if step.n_tiles:
+        most = min(step.max_rows, _ops.attention_tile_rows(torch.bfloat16))
+        blocks = step.n_tiles * -(-most * H // 64)
+        keys = max([p + n for p, n in zip(step.host_pos0, step.host_rows) if n > 1] or [step.max_context])
+        splits = max(1, min(LATENT_BLOCKS // blocks, -(-keys // 64) // LATENT_RANGE_TILES, LATENT_SPLITS_MAX))
+        run(step.tile_row0, step.tile_rows, step.n_tiles, most, splits, "latent_attention_bf16 (prompt rows)")
+    if step.n_decode_rows:
+        n = step.n_decode_rows
+        blocks = n * -(-H // (64 if H > 32 else 32))
+        splits = max(1, min(LATENT_BLOCKS // blocks, -(-step.max_decode_context // 64), LATENT_SPLITS_MAX))
+        run(step.decode_rows, None, n, 1, splits, "latent_attention_bf16 (decoded rows)")
+    return True
