@@ -727,54 +727,55 @@ def seredra_configs(size: str, context: int):
     return {"seredra": seredra, "llama": design_configs(size, 4, 2 * context)["llama"]}
 
 
+def seredra_work(size, name, rows, keys_sum, prefill):
+    """(bytes, flops) of all launches of entry point `name` in a step of the Seredra model (or, for an entry point of the
+    llama decoder, of that one)."""
+    D, H, G, d, F, V = DESIGN_SIZES[size]
+    Fe, E, K, N, C = F // SEREDRA_TOP, SEREDRA_EXPERTS, SEREDRA_TOP, SEREDRA_STATES, 2 * D
+    if name == "apc_conv_heads_bf16":        # an owner (q, k, v) and a borrower (q): rows read, q and pages written
+        return 2 * rows * ((H + 2 * G) * d + H * d) * 2 * 2 - 2 * rows * 2 * G * d * 2 * 2 // 2, 0
+    if name == "apc_rotary_pages_bf16":      # q and k read, q and the pages' keys and values written
+        return rows * ((H + G) * d + H * d + 2 * G * d) * 2, 0
+    if name in ("apc_rope_kv_write_bf16", "apc_rope_kv_write"):
+        return 4 * rows * ((H + 2 * G) * d + H * d + 2 * G * d) * 2, 0
+    if name == "apc_attention_masked_prefill_bf16":      # three attentions over all earlier keys
+        return 0, 3 * keys_sum * H * 4 * d
+    if name == "apc_attention_prefill_bf16":
+        return 0, 4 * 4 * keys_sum * H * d
+    if name == "apc_attention_masked_decode_bf16":
+        return 3 * keys_sum * G * 2 * d * 2, 0
+    if name == "apc_attention_decode_bf16":
+        return 4 * keys_sum * G * 2 * d * 2, 0
+    if name == "apc_linear_attention_bf16":  # a row: scores and weights over half a chunk of 64, 2 dk dv for the state
+        return 0, rows * H * (2 * 32 * 2 * d + 2 * 2 * d * d)
+    if name == "apc_linear_attention":       # the state of every row read and written
+        return rows * H * d * d * 4 * 2, 0
+    if name in ("apc_selective_scan", "apc_selective_scan_bf16"):
+        # x, z, the step sizes read, y written; decoded rows: the state both ways
+        return rows * C * (2 + 2 + 4 + 2) + (0 if prefill else rows * C * N * 4 * 2), 0
+    if name == "apc_conv_channels":
+        return rows * C * (2 + 2), 0
+    if name == "apc_routed_experts_bf16":
+        used = min(E, rows * K)
+        return 2 * used * 3 * Fe * D * 2, 2 * rows * K * 3 * 2 * Fe * D
+    if name in ("apc_gemm_swiglu_bf16", "apc_skinny_swiglu_bf16", "apc_skinny_swiglu_pre_bf16"):
+        return 4 * 2 * F * D * 2, 4 * rows * 2 * 2 * F * D
+    if name == "apc_act_rows":               # the float32 sums read, the activations written
+        return 2 * rows * F * (4 + 2), 0
+    if name == "apc_streams_step":           # y and x read, x and the next reader's 16-bit copy written
+        return 9 * rows * D * (4 + 4 + 4 + 2), 0
+    if name == "apc_rmsnorm_rows":
+        return 9 * rows * D * (4 + 2), 0
+    if name == "apc_gated_rmsnorm":
+        return rows * H * d * (4 + 2 + 2), 0
+    if name == "apc_weighted_pair":
+        return rows * D * 12, 0
+    return None
+
+
 def seredra_rooflines(size, batch, context, T, points):
     """For the kernels the design adds and their like kernels of the llama decoder: the bytes or the arithmetic of the
     launches of a step over the measured time, as a share of the GPU's peak (8 TB/s, 2.5 PFLOP/s)."""
-    D, H, G, d, F, V = DESIGN_SIZES[size]
-    Fe, E, K, N, C = F // SEREDRA_TOP, SEREDRA_EXPERTS, SEREDRA_TOP, SEREDRA_STATES, 2 * D
-
-    def work(name, rows, keys_sum, prefill):
-        """(bytes, flops) of all of a step's launches of entry point `name`."""
-        if name == "apc_conv_heads_bf16":        # an owner (q, k, v) and a borrower (q): rows read, q and pages written
-            return 2 * rows * ((H + 2 * G) * d + H * d) * 2 * 2 - 2 * rows * 2 * G * d * 2 * 2 // 2, 0
-        if name == "apc_rotary_pages_bf16":      # q and k read, q and the pages' keys and values written
-            return rows * ((H + G) * d + H * d + 2 * G * d) * 2, 0
-        if name in ("apc_rope_kv_write_bf16", "apc_rope_kv_write"):
-            return 4 * rows * ((H + 2 * G) * d + H * d + 2 * G * d) * 2, 0
-        if name == "apc_attention_masked_prefill_bf16":      # three attentions over all earlier keys
-            return 0, 3 * keys_sum * H * 4 * d
-        if name == "apc_attention_prefill_bf16":
-            return 0, 4 * 4 * keys_sum * H * d
-        if name == "apc_attention_masked_decode_bf16":
-            return 3 * keys_sum * G * 2 * d * 2, 0
-        if name == "apc_attention_decode_bf16":
-            return 4 * keys_sum * G * 2 * d * 2, 0
-        if name == "apc_linear_attention_bf16":  # a row: scores and weights over half a chunk of 64, 2 dk dv for the state
-            return 0, rows * H * (2 * 32 * 2 * d + 2 * 2 * d * d)
-        if name == "apc_linear_attention":       # the state of every row read and written
-            return rows * H * d * d * 4 * 2, 0
-        if name in ("apc_selective_scan", "apc_selective_scan_bf16"):
-            # x, z, the step sizes read, y written; decoded rows: the state both ways
-            return rows * C * (2 + 2 + 4 + 2) + (0 if prefill else rows * C * N * 4 * 2), 0
-        if name == "apc_conv_channels":
-            return rows * C * (2 + 2), 0
-        if name == "apc_routed_experts_bf16":
-            used = min(E, rows * K)
-            return 2 * used * 3 * Fe * D * 2, 2 * rows * K * 3 * 2 * Fe * D
-        if name in ("apc_gemm_swiglu_bf16", "apc_skinny_swiglu_bf16", "apc_skinny_swiglu_pre_bf16"):
-            return 4 * 2 * F * D * 2, 4 * rows * 2 * 2 * F * D
-        if name == "apc_act_rows":               # the float32 sums read, the activations written
-            return 2 * rows * F * (4 + 2), 0
-        if name == "apc_streams_step":           # y and x read, x and the next reader's 16-bit copy written
-            return 9 * rows * D * (4 + 4 + 4 + 2), 0
-        if name == "apc_rmsnorm_rows":
-            return 9 * rows * D * (4 + 2), 0
-        if name == "apc_gated_rmsnorm":
-            return rows * H * d * (4 + 2 + 2), 0
-        if name == "apc_weighted_pair":
-            return rows * D * 12, 0
-        return None
-
     table = {}
     for phase, rows, keys_sum in (("prefill", T, T * (T + 1) // 2), ("decode", batch, batch * context)):
         for new, likes in SEREDRA_LIKE_KERNELS.items():
@@ -785,7 +786,7 @@ def seredra_rooflines(size, batch, context, T, points):
                 name = next((n for n in names if n in times), None)
                 if not us or name is None:
                     continue
-                w = work(name, rows, keys_sum, phase == "prefill")
+                w = seredra_work(size, name, rows, keys_sum, phase == "prefill")
                 row[model] = {"us": round(us, 1)}
                 if w:
                     row[model]["share_of_peak"] = round(max(w[0] / (us * 1e-6) / (HBM_PEAK_GBS * 1e9),
@@ -814,6 +815,122 @@ def seredra_run(args) -> int:
             "prefill_seredra_over_llama": round(points["seredra"]["prefill_tok_s"] / points["llama"]["prefill_tok_s"], 3),
             "decode_seredra_over_llama": round(points["seredra"]["decode_tok_s"] / points["llama"]["decode_tok_s"], 3),
             "like_kernels": seredra_rooflines(size, batch, context, T, points)}
+    print(json.dumps(out), flush=True)
+    return 0
+
+
+# ---- the Muvorax design beside the llama and Seredra decoders at equal sizes ---------------------------------------
+# like kernels: of the llama decoder, and of Seredra (which shares the scan, the linear attention and the router)
+MUVORAX_LIKE_KERNELS = {
+    "apc_latent_attention_bf16": (["apc_attention_prefill_bf16", "apc_attention_decode_bf16"],
+                                  ["apc_attention_masked_prefill_bf16", "apc_attention_masked_decode_bf16"]),
+    "apc_latent_rows_bf16": (["apc_rope_kv_write_bf16", "apc_rope_kv_write"], ["apc_rotary_pages_bf16"]),
+    "apc_heads_gemm_bf16": (["apc_gemm_bf16", "apc_skinny_gemm_bf16"], []),
+    "apc_tanh_norm_add": (["apc_rmsnorm_rows"], ["apc_streams_step"]),
+    "apc_act_rows": ([], ["apc_act_rows"]),
+    "apc_routed_experts_bf16": (["apc_gemm_swiglu_bf16", "apc_gemm_pre_bf16", "apc_skinny_swiglu_pre_bf16"],
+                                ["apc_routed_experts_bf16"]),
+    "apc_route_topk": ([], ["apc_route_topk"]),
+    "apc_linear_attention_bf16": (["apc_attention_prefill_bf16"], ["apc_linear_attention_bf16"]),
+    "apc_linear_attention": (["apc_attention_decode_bf16"], ["apc_linear_attention"]),
+    "apc_selective_scan_bf16": (["apc_attention_prefill_bf16"], ["apc_selective_scan_bf16"]),
+    "apc_selective_scan": (["apc_attention_decode_bf16"], ["apc_selective_scan"]),
+    "apc_conv_channels": (["apc_rope_kv_write_bf16"], ["apc_conv_channels"]),
+    "apc_gated_rmsnorm": ([], ["apc_gated_rmsnorm"]),
+}
+MUVORAX_EXPERTS, MUVORAX_TOP, MUVORAX_STATES, MUVORAX_TAPS = 8, 2, 16, 4
+
+
+def muvorax_configs(size: str, context: int):
+    """Four layers: an attention over cached latents (H heads of d unrotated and d/2 rotated elements, a latent of 4 d)
+    with the dense feed-forward; a selective scan of 2 x width channels with 16 states and a lightning attention (heads
+    of d), both with routed experts (2 of 8 in 4 groups of which 2 are kept, each half as wide as the dense
+    feed-forward); an attention on the first layer's latents with the dense feed-forward.  The llama decoder and the
+    Seredra decoder (see there) with four layers of the same widths."""
+    D, H, G, d, F, V = DESIGN_SIZES[size]
+    lat = dict(heads=H, dim=d, rot_dim=d // 2, vdim=d, kv_rank=4 * d, scale=(d + d // 2) ** -0.5,
+               rot=dict(base=500000.0, dims=d // 2, scaling=dict(factor=4.0, original=2048, fast=32.0, slow=1.0)))
+    scan = dict(inner=2 * D, state=MUVORAX_STATES, dt_rank=D // 16, conv=MUVORAX_TAPS)
+    lig = dict(heads=H, dim=d, vdim=d, decay=[1.0 - 2.0 ** (-5 - 5 * h / H) for h in range(H)])
+    moe = dict(kind="moe", expert=dict(ff=F // MUVORAX_TOP),
+               router=dict(experts=MUVORAX_EXPERTS, top=MUVORAX_TOP, scale=1.5, groups=dict(count=4, keep=2)))
+    dense = dict(kind="dense", ff=F)
+    muvorax = dict(architecture="Muvorax", vocab=V, width=D, norm=dict(eps=1e-6), max_positions=2 * context + 4096,
+                   layers=[dict(type="latent_attention", mixer=lat, mlp=dense), dict(type="mamba1", mixer=scan, mlp=moe),
+                           dict(type="lightning", mixer=lig, mlp=moe),
+                           dict(type="latent_attention", mixer=dict(lat, kv_from=0), mlp=dense)])
+    return {"muvorax": muvorax, **seredra_configs(size, context)}
+
+
+def muvorax_rooflines(size, batch, context, T, points):
+    """For the kernels the design uses beside plain products and their like kernels: the bytes or the arithmetic of the
+    launches of a step over the measured time, as a share of the GPU's peak (8 TB/s, 2.5 PFLOP/s)."""
+    D, H, G, d, F, V = DESIGN_SIZES[size]
+    R, dr = 4 * d, d // 2
+    Fe, E, K, N, C = F // MUVORAX_TOP, MUVORAX_EXPERTS, MUVORAX_TOP, MUVORAX_STATES, 2 * D
+
+    def work(model, name, rows, keys_sum, prefill):
+        """(bytes, flops) of all of a step's launches of entry point `name`."""
+        if name == "apc_latent_attention_bf16":  # two layers; decoded rows: the cached rows of their requests
+            return (0, 2 * keys_sum * H * 2 * (2 * R + dr)) if prefill else (2 * keys_sum * (R + dr) * 2,
+                                                                            2 * keys_sum * H * 2 * (2 * R + dr))
+        if name == "apc_latent_rows_bf16":       # the rotated parts of q in two layers, latents and key part of one
+            return rows * (2 * H * dr * 2 + (R + dr) * 2) * 2, 0
+        if name == "apc_heads_gemm_bf16":        # queries and outputs of two layers
+            return (2 * 2 * H * d * R * 2 + 2 * rows * H * (d + 2 * R + dr + d) * 2, 2 * 2 * rows * H * 2 * d * R)
+        if name == "apc_tanh_norm_add":          # x and y read, x and the next reader's 16-bit copy written
+            return 8 * rows * D * (4 + 4 + 4 + 2), 0
+        if name == "apc_routed_experts_bf16" and model == "muvorax":
+            return 2 * min(E, rows * K) * 2 * Fe * D * 2, 2 * rows * K * 2 * 2 * Fe * D
+        if name == "apc_gemm_pre_bf16":          # llama: the gate and up products of four layers (and q, k, v of three)
+            return 4 * 2 * F * D * 2 + 3 * (H + 2 * G) * d * D * 2, rows * 2 * (4 * 2 * F * D + 3 * (H + 2 * G) * d * D)
+        if name == "apc_gemm_bf16" and model == "llama":         # q, k, v of the first layer
+            return 0, rows * 2 * (H + 2 * G) * d * D
+        if name == "apc_skinny_gemm_bf16" and model == "llama":  # the head
+            return V * D * 2, 0
+        if name == "apc_gated_rmsnorm":
+            return rows * H * d * (4 + 2 + 2), 0
+        return seredra_work(size, name, rows, keys_sum, prefill)
+
+    table = {}
+    for phase, rows, keys_sum in (("prefill", T, T * (T + 1) // 2), ("decode", batch, batch * context)):
+        for new, (llama, seredra) in MUVORAX_LIKE_KERNELS.items():
+            row = {}
+            for model, names in (("muvorax", [new]), ("llama", llama), ("seredra", seredra)):
+                times = points[model][phase + "_kernels_us"]
+                name = next((n for n in names if n in times), None)
+                if name is None or not times[name]:
+                    continue
+                us = times[name]
+                w = work(model, name, rows, keys_sum, phase == "prefill")
+                row[model] = {"us": round(us, 1)}
+                if w:
+                    row[model]["share_of_peak"] = round(max(w[0] / (us * 1e-6) / (HBM_PEAK_GBS * 1e9),
+                                                            w[1] / (us * 1e-6) / PEAK_FLOPS["bf16"]), 4)
+            if "muvorax" in row:
+                table[f"{phase}: {new}"] = row
+    return table
+
+
+def muvorax_run(args) -> int:
+    T, batch, context = 2048, args.batch, args.context
+    out = {"metric": "Muvorax beside the llama and Seredra decoders at equal sizes: prefill tok/s (one prompt of 2048 "
+                     f"tokens) and decode tok/s (batch {batch}, context {context})", "unit": "tok/s", "n_gpus": 1,
+           "dtype": args.dtype, "data": "synthetic: random N(0, 0.02) weights, uniform random token ids",
+           "config": {"layers": "latent attention + dense, selective scan + experts, lightning + experts, borrowing "
+                                "latent attention + dense",
+                      "experts": MUVORAX_EXPERTS, "top": MUVORAX_TOP, "states": MUVORAX_STATES, "taps": MUVORAX_TAPS,
+                      "page_tokens": 16},
+           "sizes": {}}
+    for size in args.design_sizes.split(","):
+        cfgs = muvorax_configs(size, context)
+        points = {m: design_point(c, args.dtype, batch, context, args.steps, args.warmup, T) for m, c in cfgs.items()}
+        out["sizes"][size] = {
+            "shape": dict(zip(("width", "heads", "kv_heads", "head_size", "ff", "vocab"), DESIGN_SIZES[size])),
+            **points,
+            **{f"{phase}_muvorax_over_{m}": round(points["muvorax"][phase + "_tok_s"] / points[m][phase + "_tok_s"], 3)
+               for phase in ("prefill", "decode") for m in ("llama", "seredra")},
+            "like_kernels": muvorax_rooflines(size, batch, context, T, points)}
     print(json.dumps(out), flush=True)
     return 0
 
@@ -983,7 +1100,7 @@ def main() -> int:
                     help="for profiling: only the decode steps at --batch (as --no-points), only the 2,048-token "
                          "prefill (prints its figures as the line's value), or only the sampler over the preset's "
                          "vocabulary (microseconds a step's rows take on the GPU and on the host)")
-    ap.add_argument("--design", choices=["risizen", "gulidra", "lesarax", "seredra"], default=None,
+    ap.add_argument("--design", choices=["risizen", "gulidra", "lesarax", "seredra", "muvorax"], default=None,
                     help="instead of the default workload: the named design beside the llama decoder at equal sizes "
                          "(--design-sizes), prefill and decode throughput and the times of their like kernels")
     ap.add_argument("--design-sizes", default="1b,8b", help="with --design: sizes of the comparison, of " + ",".join(DESIGN_SIZES))
@@ -1008,6 +1125,8 @@ def main() -> int:
         return lesarax_run(args)
     if args.design == "seredra":
         return seredra_run(args)
+    if args.design == "muvorax":
+        return muvorax_run(args)
     if args.design:
         return design_run(args)
     if args.kernel_times:
