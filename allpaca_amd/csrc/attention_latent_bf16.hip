@@ -358,33 +358,52 @@ __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
   }
 }
 
-// a block: one pair of an item; 4 value elements a thread
+// a block: one pair of an item; 4 value elements a thread.  The ranges' factors are made once, by the first wave.
+constexpr int SPLITS_MAX = 256, SPLITS_LANE = SPLITS_MAX / WAVE;
 __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ parts, const float* __restrict__ ml,
                                                            int n_splits, int H, int R, LatentItems items,
                                                            bf16_t* __restrict__ out) {
+  __shared__ float factor[SPLITS_MAX];
   const int item = blockIdx.x / items.blocks, pair = blockIdx.x % items.blocks;
   if (pair >= (items.rows ? items.rows[item] : 1) * H) return;
   const size_t gp = (size_t)(items.row0 ? items.row0[item] : item) * H + pair;
-  const float* g = ml + gp * n_splits * 2;
-  float m = NO_KEY;
-  for (int s = 0; s < n_splits; ++s)
-    if (g[2 * s + 1] > 0.f) m = fmaxf(m, g[2 * s]);
-  float sum = 0.f;
-  for (int s = 0; s < n_splits; ++s)
-    if (g[2 * s + 1] > 0.f) sum += g[2 * s + 1] * __builtin_amdgcn_exp2f(g[2 * s] - m);
-  const float inv = 1.0f / sum;
+  if (threadIdx.x < WAVE) {
+    float m[SPLITS_LANE], l[SPLITS_LANE], top = NO_KEY, sum = 0.f;
+#pragma unroll
+    for (int k = 0; k < SPLITS_LANE; ++k) {
+      const int s = threadIdx.x + k * WAVE;
+      m[k] = s < n_splits ? ml[(gp * n_splits + s) * 2] : NO_KEY;
+      l[k] = s < n_splits ? ml[(gp * n_splits + s) * 2 + 1] : 0.f;
+      if (l[k] > 0.f) top = fmaxf(top, m[k]);
+    }
+    top = wave_max(top);
+#pragma unroll
+    for (int k = 0; k < SPLITS_LANE; ++k) {
+      m[k] = l[k] > 0.f ? __builtin_amdgcn_exp2f(m[k] - top) : 0.f;        // a range without a key of this pair: 0
+      sum = fmaf(l[k], m[k], sum);
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int k = 0; k < SPLITS_LANE; ++k) factor[threadIdx.x + k * WAVE] = m[k] / sum;
+  }
+  __syncthreads();
+  const float* src = parts + gp * n_splits * R;
   for (int r = threadIdx.x * 4; r < R; r += 512) {
     floatx4 acc = floatx4{0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < n_splits; ++s) {
-      if (!(g[2 * s + 1] > 0.f)) continue;              // a range without a key of this pair has left nothing
-      const float f = __builtin_amdgcn_exp2f(g[2 * s] - m);
-      const floatx4 v = *reinterpret_cast<const floatx4*>(parts + (gp * n_splits + s) * R + r);
+    for (int s0 = 0; s0 < n_splits; s0 += 8) {
+      floatx4 v[8];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) acc[k] = fmaf(f, v[k], acc[k]);
+      for (int k = 0; k < 8; ++k) v[k] = *reinterpret_cast<const floatx4*>(src + (size_t)min(s0 + k, n_splits - 1) * R + r);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        const float f = s0 + k < n_splits ? factor[s0 + k] : 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[e] = f != 0.f ? fmaf(f, v[k][e], acc[e]) : acc[e];    // (0: nothing was left)
+      }
     }
     uint2 pk;
-    pk.x = pack_bf16x2(acc[0] * inv, acc[1] * inv);
-    pk.y = pack_bf16x2(acc[2] * inv, acc[3] * inv);
+    pk.x = pack_bf16x2(acc[0], acc[1]);
+    pk.y = pack_bf16x2(acc[2], acc[3]);
     *reinterpret_cast<uint2*>(out + gp * R + r) = pk;
   }
 }
@@ -412,7 +431,7 @@ APC_EXPORT int apc_latent_attention_bf16(const void* q, void* out, int H, int R,
                                          int n_splits, float* parts, float* ml, float scale, hipStream_t stream) {
   if (n_items <= 0) return 0;
   if (!apc_latent_attention_takes(H, R, dr, page_tokens)) return APC_ERR_UNSUPPORTED;
-  if (max_blocks <= 0 || max_rows <= 0 || n_splits < 1 || (n_splits > 1 && (!parts || !ml)) || (max_rows > 1 && !rows) ||
+  if (max_blocks <= 0 || max_rows <= 0 || n_splits < 1 || n_splits > SPLITS_MAX || (n_splits > 1 && (!parts || !ml)) || (max_rows > 1 && !rows) ||
       ((uintptr_t)q & 15u) || ((uintptr_t)out & 7u) || ((uintptr_t)pages & 15u) || ((uintptr_t)parts & 15u))
     return APC_ERR_BAD_ARG;
   const int L = R + dr, rt = value_blocks(R, L), pairs = max_rows * H;

@@ -1,4 +1,5 @@
-// Products with a matrix of its own for every head, bfloat16 on MFMA (the up-projections of an attention over cached
+// What an attention over cached latents does to the projected rows ahead of its products (`latent_rows_bf16_kernel`), and
+// products with a matrix of its own for every head, bfloat16 on MFMA (the up-projections of an attention over cached
 // latents, applied to its queries and to its outputs):
 //   C[m][h * c_head + n] = sum_k A[m][h * a_head + k] W[h][n][k]
 // W: every head's matrix in tiles of 16 rows x 32 columns in the lane order of the MFMA operand (see gemm_bf16.hip).
@@ -103,7 +104,110 @@ __global__ __launch_bounds__(256) void heads_gemm_kernel(const bf16_t* __restric
   }
 }
 
+__device__ __forceinline__ void unpack8(const Frag& f, float (&v)[8]) {
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    v[2 * k] = __uint_as_float(f.w[k] << 16);
+    v[2 * k + 1] = __uint_as_float(f.w[k] & 0xffff0000u);
+  }
+}
+__device__ __forceinline__ Frag pack8(const float (&v)[8]) {
+  Frag f;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) f.w[k] = pack_bf16x2(v[2 * k], v[2 * k + 1]);
+  return f;
+}
+// 8 pairs (j, j + half) of a rotated part
+__device__ __forceinline__ void rotate8(const bf16_t* src, bf16_t* dst, const float* cs, int j, int half) {
+  float u[8], v[8], a[8], b[8];
+  unpack8(load_frag(src + j), u);
+  unpack8(load_frag(src + half + j), v);
+#pragma unroll
+  for (int e = 0; e < 8; e += 4) {
+    const float4 c = *reinterpret_cast<const float4*>(cs + j + e), s = *reinterpret_cast<const float4*>(cs + half + j + e);
+    const float cc[4] = {c.x, c.y, c.z, c.w}, ss[4] = {s.x, s.y, s.z, s.w};
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      a[e + k] = u[e + k] * cc[k] - v[e + k] * ss[k];
+      b[e + k] = v[e + k] * cc[k] + u[e + k] * ss[k];
+    }
+  }
+  *reinterpret_cast<Frag*>(dst + j) = pack8(a);
+  *reinterpret_cast<Frag*>(dst + half + j) = pack8(b);
+}
+
+// A block: one row.  The first wave norms the latent and rotates the shared key part into the row's place in its page
+// (8 elements a lane); the other waves rotate the queries' parts, 8 pairs a lane.  Sizes and strides are multiples of 8,
+// the rotated part of 16.  c_off < 0: queries only.
+__global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __restrict__ proj, int ld, int H, int dn,
+                                                               int dr, int c_off, int R, const float* __restrict__ norm_w,
+                                                               float eps, const float* __restrict__ cos_sin,
+                                                               const int* __restrict__ positions,
+                                                               const int* __restrict__ row_seg,
+                                                               const int* __restrict__ block_table, int max_blocks,
+                                                               bf16_t* __restrict__ pages, int P, bf16_t* __restrict__ q,
+                                                               int ldq) {
+  const int r = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, half = dr / 2, L = R + dr;
+  const int pos = positions[r];
+  const float* cs = cos_sin + (size_t)pos * dr;
+  const bf16_t* row = proj + (size_t)r * ld;
+  int first = threadIdx.x, step = 256;
+  if (c_off >= 0) {
+    if (wave == 0) {
+      const bf16_t* src = row + c_off;
+      const int page = block_table[(size_t)row_seg[r] * max_blocks + pos / P];
+      bf16_t* dst = pages + ((size_t)page * P + pos % P) * L;
+      float ss = 0.f;
+      for (int i = lane * 8; i < R; i += WAVE * 8) {
+        float v[8];
+        unpack8(load_frag(src + i), v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss = fmaf(v[e], v[e], ss);
+      }
+      const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)R + eps);
+      for (int i = lane * 8; i < R; i += WAVE * 8) {
+        float v[8];
+        unpack8(load_frag(src + i), v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = v[e] * inv * norm_w[i + e];
+        *reinterpret_cast<Frag*>(dst + i) = pack8(v);
+      }
+      if (lane * 8 < half) rotate8(src + R, dst + R, cs, lane * 8, half);
+      return;
+    }
+    first -= WAVE;
+    step -= WAVE;
+  }
+  const int per_head = half / 8;
+  for (int i = first; i < H * per_head; i += step) {
+    const int h = i / per_head, j = i % per_head * 8;
+    rotate8(row + (size_t)h * (dn + dr) + dn, q + (size_t)r * ldq + (size_t)h * L + R, cs, j, half);
+  }
+}
+
 }  // namespace
+
+APC_EXPORT int apc_latent_rows_bf16_takes(int ld, int dn, int dr, int c_off, int R, int ldq) {
+  return (ld % 8 == 0 && dn % 8 == 0 && dr > 0 && dr % 16 == 0 && dr <= 1024 && R % 8 == 0 && ldq % 8 == 0 &&
+          (c_off < 0 || c_off % 8 == 0)) ? 1 : 0;
+}
+
+APC_EXPORT int apc_latent_rows_bf16(const void* proj, int ld, int H, int dn, int dr, int c_off, int R,
+                                    const float* norm_w, float eps, const float* cos_sin, const int* positions,
+                                    const int* row_seg, const int* block_table, int max_blocks, void* pages, int P,
+                                    void* q, int ldq, int n_rows, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (!apc_latent_rows_bf16_takes(ld, dn, dr, c_off, R, ldq)) return APC_ERR_UNSUPPORTED;
+  if (H <= 0 || dn <= 0 || R <= 0 || P <= 0 || max_blocks <= 0 || ldq < H * (R + dr) || ld < H * (dn + dr) || !cos_sin ||
+      (c_off >= 0 && (ld < c_off + R + dr || !norm_w || !pages)) || ((uintptr_t)proj & 15u) || ((uintptr_t)q & 15u) ||
+      ((uintptr_t)pages & 15u) || ((uintptr_t)cos_sin & 15u))
+    return APC_ERR_BAD_ARG;
+  hipLaunchKernelGGL(latent_rows_bf16_kernel, dim3(n_rows), dim3(256), 0, stream, (const bf16_t*)proj, ld, H, dn, dr,
+                     c_off, R, norm_w, eps, cos_sin, positions, row_seg, block_table, max_blocks, (bf16_t*)pages, P,
+                     (bf16_t*)q, ldq);
+  APC_LAUNCH_CHECK();
+  return 0;
+}
 
 APC_EXPORT int apc_heads_gemm_bf16(const void* A, int lda, int a_head, const void* W, void* C, int ldc, int c_head, int M,
                                    int H, int N, int K, hipStream_t stream) {

@@ -152,22 +152,34 @@ __global__ __launch_bounds__(256) void tanh_norm_add_kernel(float* __restrict__ 
   if (h) store_f(h, h_dtype, (size_t)r * ldh + i, fmaf(squash<EXACT>(n.alpha * v), n.w[i], n.b[i]));
 }
 
-// The same for float32 x and y, 4 elements a thread on 16-byte accesses.
-template <bool EXACT>
+// The same for float32 x and y, VPT times 4 elements a thread on 16-byte accesses, all loads of x and y ahead of the
+// first store.
+template <bool EXACT, int VPT>
 __global__ __launch_bounds__(256) void tanh_norm_add_f4_kernel(float* __restrict__ x, int ldx, const float* __restrict__ y,
                                                                int ldy, TanhNorm post, TanhNorm n, void* __restrict__ h,
                                                                int h_dtype, int ldh, int dim) {
-  const int r = blockIdx.x, i = (blockIdx.y * 256 + threadIdx.x) * 4;
-  if (i >= dim) return;
-  float4* xp = reinterpret_cast<float4*>(x + (size_t)r * ldx + i);
-  const float4 xv = *xp, yv = *reinterpret_cast<const float4*>(y + (size_t)r * ldy + i);
-  const float4 pw = *reinterpret_cast<const float4*>(post.w + i), pb = *reinterpret_cast<const float4*>(post.b + i);
-  float4 v;
-  v.x = xv.x + fmaf(squash<EXACT>(post.alpha * yv.x), pw.x, pb.x);
-  v.y = xv.y + fmaf(squash<EXACT>(post.alpha * yv.y), pw.y, pb.y);
-  v.z = xv.z + fmaf(squash<EXACT>(post.alpha * yv.z), pw.z, pb.z);
-  v.w = xv.w + fmaf(squash<EXACT>(post.alpha * yv.w), pw.w, pb.w);
-  if (h) {
+  const int r = blockIdx.x, i0 = (blockIdx.y * VPT * 256 + threadIdx.x) * 4;
+  float4 xv[VPT], yv[VPT];
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = i0 + k * 1024;
+    if (i < dim) {
+      xv[k] = *reinterpret_cast<const float4*>(x + (size_t)r * ldx + i);
+      yv[k] = *reinterpret_cast<const float4*>(y + (size_t)r * ldy + i);
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = i0 + k * 1024;
+    if (i >= dim) return;
+    const float4 pw = *reinterpret_cast<const float4*>(post.w + i), pb = *reinterpret_cast<const float4*>(post.b + i);
+    float4 v;
+    v.x = xv[k].x + fmaf(squash<EXACT>(post.alpha * yv[k].x), pw.x, pb.x);
+    v.y = xv[k].y + fmaf(squash<EXACT>(post.alpha * yv[k].y), pw.y, pb.y);
+    v.z = xv[k].z + fmaf(squash<EXACT>(post.alpha * yv[k].z), pw.z, pb.z);
+    v.w = xv[k].w + fmaf(squash<EXACT>(post.alpha * yv[k].w), pw.w, pb.w);
+    *reinterpret_cast<float4*>(x + (size_t)r * ldx + i) = v;
+    if (!h) continue;
     const float4 w = *reinterpret_cast<const float4*>(n.w + i), b = *reinterpret_cast<const float4*>(n.b + i);
     float4 o;
     o.x = fmaf(squash<EXACT>(n.alpha * v.x), w.x, b.x);
@@ -184,7 +196,6 @@ __global__ __launch_bounds__(256) void tanh_norm_add_f4_kernel(float* __restrict
       *reinterpret_cast<uint2*>((bf16_t*)h + at) = pk;
     }
   }
-  *xp = v;
 }
 
 }  // namespace
@@ -245,14 +256,17 @@ APC_EXPORT int apc_tanh_norm_add(float* x, int ldx, const void* y, int y_dtype, 
   auto a16 = [](const void* p) { return ((uintptr_t)p & 15u) == 0; };
   if (y_dtype == APC_F32 && dim % 4 == 0 && ldx % 4 == 0 && ldy % 4 == 0 && a16(x) && a16(y) && a16(pw) && a16(pb) &&
       (!h || (ldh % 4 == 0 && a16(h) && a16(w) && a16(b)))) {
-    const dim3 grid(n_rows, ceil_div(dim, 1024));
+    const int vpt = n_rows >= 256 && dim > 1024 ? 2 : 1;       // (a step of few rows wants its blocks)
+    const dim3 grid(n_rows, ceil_div(dim, 1024 * vpt));
     if (grid.y > 65535) return APC_ERR_UNSUPPORTED;
-    if (exact)
-      hipLaunchKernelGGL(tanh_norm_add_f4_kernel<true>, grid, dim3(256), 0, stream, x, ldx, (const float*)y, ldy, post, n,
-                         h, h_dtype, ldh, dim);
-    else
-      hipLaunchKernelGGL(tanh_norm_add_f4_kernel<false>, grid, dim3(256), 0, stream, x, ldx, (const float*)y, ldy, post, n,
-                         h, h_dtype, ldh, dim);
+#define TANH_ADD(EXACT_, VPT_)                                                                                         \
+  hipLaunchKernelGGL((tanh_norm_add_f4_kernel<EXACT_, VPT_>), grid, dim3(256), 0, stream, x, ldx, (const float*)y, ldy, \
+                     post, n, h, h_dtype, ldh, dim)
+    if (exact && vpt == 2) TANH_ADD(true, 2);
+    else if (exact) TANH_ADD(true, 1);
+    else if (vpt == 2) TANH_ADD(false, 2);
+    else TANH_ADD(false, 1);
+#undef TANH_ADD
   } else {
     const dim3 grid(n_rows, ceil_div(dim, 256));
     if (grid.y > 65535) return APC_ERR_UNSUPPORTED;

@@ -22,18 +22,20 @@ namespace {
 constexpr int MAX_PER_LANE_R = 16;   // up to 1,024 router outputs
 constexpr int MAX_TOP = 32;
 
+// PL: router outputs a lane holds (the loops are unrolled over it)
+template <int PL>
 __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict__ z, int ldz,
                                                         const float* __restrict__ correction, int N, int K,
                                                         int renormalize, int score, int groups, int keep,
                                                         float w_scale, int* __restrict__ ids,
                                                         float* __restrict__ weights) {
-  __shared__ float cs[MAX_PER_LANE_R * WAVE];      // groups > 1: the choice scores, and whether a run is kept
-  __shared__ int kept[MAX_PER_LANE_R * WAVE];
+  __shared__ float cs[PL * WAVE];      // groups > 1: the choice scores, and whether a run is kept
+  __shared__ int kept[PL * WAVE];
   const int t = blockIdx.x, lane = threadIdx.x;
-  float s[MAX_PER_LANE_R], c[MAX_PER_LANE_R];
+  float s[PL], c[PL];
   float mx = -INFINITY;
 #pragma unroll
-  for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+  for (int e = 0; e < PL; ++e) {
     const int i = lane + e * WAVE;
     s[e] = i < N ? z[(size_t)t * ldz + i] : -INFINITY;
     mx = fmaxf(mx, s[e]);
@@ -41,7 +43,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
   mx = wave_max(mx);
   float sum = 0.f;
 #pragma unroll
-  for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+  for (int e = 0; e < PL; ++e) {
     const int i = lane + e * WAVE;
     if (score == 1) s[e] = i < N ? 1.0f / (1.0f + expf(-s[e])) : 0.f;
     else s[e] = i < N ? expf(s[e] - mx) : 0.f;
@@ -49,7 +51,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
   }
   sum = score == 1 ? 1.f : wave_sum(sum);
 #pragma unroll
-  for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+  for (int e = 0; e < PL; ++e) {
     const int i = lane + e * WAVE;
     s[e] = s[e] / sum;
     c[e] = i < N ? s[e] + (correction ? correction[i] : 0.f) : -INFINITY;
@@ -57,14 +59,14 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
   if (groups > keep) {
     const int n = N / groups;
 #pragma unroll
-    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+    for (int e = 0; e < PL; ++e) {
       const int i = lane + e * WAVE;
       if (i < N) cs[i] = c[e];
     }
     __syncthreads();
-    float gs[MAX_PER_LANE_R];
+    float gs[PL];
 #pragma unroll
-    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+    for (int e = 0; e < PL; ++e) {
       const int g = lane + e * WAVE;
       gs[e] = -INFINITY;
       if (g >= groups) continue;
@@ -81,7 +83,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
       float best = -INFINITY;
       int best_g = 0x7fffffff;
 #pragma unroll
-      for (int e = 0; e < MAX_PER_LANE_R; ++e)
+      for (int e = 0; e < PL; ++e)
         if (gs[e] > best) { best = gs[e]; best_g = lane + e * WAVE; }
 #pragma unroll
       for (int o = WAVE / 2; o > 0; o >>= 1) {
@@ -90,12 +92,12 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
         if (ob > best || (ob == best && og < best_g)) { best = ob; best_g = og; }
       }
 #pragma unroll
-      for (int e = 0; e < MAX_PER_LANE_R; ++e)
+      for (int e = 0; e < PL; ++e)
         if (lane + e * WAVE == best_g) { gs[e] = -INFINITY; kept[best_g] = 1; }
     }
     __syncthreads();
 #pragma unroll
-    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+    for (int e = 0; e < PL; ++e) {
       const int i = lane + e * WAVE;
       if (i < N && !kept[i / n]) c[e] = -INFINITY;
     }
@@ -107,7 +109,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
     float best = -INFINITY;
     int best_i = 0x7fffffff;
 #pragma unroll
-    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+    for (int e = 0; e < PL; ++e) {
       const int i = lane + e * WAVE;
       if (c[e] > best) { best = c[e]; best_i = i; }      // a lane's own candidates come in rising order of index
     }
@@ -119,7 +121,7 @@ __global__ __launch_bounds__(64) void route_topk_kernel(const float* __restrict_
     }
     float w = 0.f;
 #pragma unroll
-    for (int e = 0; e < MAX_PER_LANE_R; ++e) {
+    for (int e = 0; e < PL; ++e) {
       const int i = lane + e * WAVE;
       if (i == best_i) { w = s[e]; c[e] = -INFINITY; }
     }
@@ -225,8 +227,13 @@ APC_EXPORT int apc_route_topk(const float* z, int ldz, const float* correction, 
   if (groups < 1 || keep < 1 || keep > groups || N <= 0 || N % groups || K > keep * (N / groups)) return APC_ERR_BAD_ARG;
   if (N <= 0 || K <= 0 || K > N || ldz < N || !ids || !weights || score < 0 || score > 1) return APC_ERR_BAD_ARG;
   if (N > MAX_PER_LANE_R * WAVE || K > MAX_TOP) return APC_ERR_UNSUPPORTED;
-  hipLaunchKernelGGL(route_topk_kernel, dim3(n_rows), dim3(64), 0, stream, z, ldz, correction, N, K, renormalize, score,
-                     groups, keep, w_scale, ids, weights);
+#define TOPK_LAUNCH(PL_)                                                                                              \
+  hipLaunchKernelGGL(route_topk_kernel<PL_>, dim3(n_rows), dim3(64), 0, stream, z, ldz, correction, N, K, renormalize, \
+                     score, groups, keep, w_scale, ids, weights)
+  if (N <= WAVE) TOPK_LAUNCH(1);
+  else if (N <= 4 * WAVE) TOPK_LAUNCH(4);
+  else TOPK_LAUNCH(MAX_PER_LANE_R);
+#undef TOPK_LAUNCH
   APC_LAUNCH_CHECK();
   return 0;
 }

@@ -253,20 +253,47 @@ __global__ __launch_bounds__(256) void routed_gather_kernel(const bf16_t* __rest
   }
 }
 
+// grid: rows x blocks of 1,024 columns; 4 columns a thread, the pairs' loads of up to 4 choices in flight together
+// (VEC: 16-byte loads, D and the strides multiples of 4)
+template <bool VEC>
 __global__ __launch_bounds__(256) void routed_combine_kernel(const float* __restrict__ ys, const int* __restrict__ place,
                                                              const float* __restrict__ weights, int K,
                                                              const bf16_t* __restrict__ h, int ldh,
                                                              float* __restrict__ y, int ldy, int D, int in_weights) {
-  const int t = blockIdx.x;
-  for (int d = threadIdx.x; d < D; d += 256) {
-    float total = 0.f;
-    for (int k = 0; k < K; ++k) {
-      const int at = place[(size_t)t * K + k];
-      const float v = at >= 0 ? ys[(size_t)at * D + d] : bf16_to_float(h[(size_t)t * ldh + d]);
-      total = (in_weights && at >= 0) ? total + v : fmaf(weights[(size_t)t * K + k], v, total);
+  const int t = blockIdx.x, d0 = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (d0 >= D) return;
+  const int n = VEC ? 4 : min(4, D - d0);
+  float total[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < K; k0 += 4) {
+    float v[4][4], w[4];
+    int at[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const bool on = k0 + k < K;
+      at[k] = on ? place[(size_t)t * K + k0 + k] : -1;
+      w[k] = on ? weights[(size_t)t * K + k0 + k] : 0.f;
     }
-    y[(size_t)t * ldy + d] = total;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (k0 + k >= K) break;
+      if (VEC && at[k] >= 0) {
+        const float4 f = *reinterpret_cast<const float4*>(ys + (size_t)at[k] * D + d0);
+        v[k][0] = f.x; v[k][1] = f.y; v[k][2] = f.z; v[k][3] = f.w;
+      } else {
+        for (int e = 0; e < n; ++e)
+          v[k][e] = at[k] >= 0 ? ys[(size_t)at[k] * D + d0 + e] : bf16_to_float(h[(size_t)t * ldh + d0 + e]);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (k0 + k >= K) break;
+      for (int e = 0; e < n; ++e)
+        total[e] = (in_weights && at[k] >= 0) ? total[e] + v[k][e] : fmaf(w[k], v[k][e], total[e]);
+    }
   }
+  if (VEC) *reinterpret_cast<float4*>(y + (size_t)t * ldy + d0) = float4{total[0], total[1], total[2], total[3]};
+  else
+    for (int e = 0; e < n; ++e) y[(size_t)t * ldy + d0 + e] = total[e];
 }
 
 }  // namespace
@@ -341,8 +368,13 @@ APC_EXPORT int apc_routed_experts_bf16(const void* h, int ldh, const void* w_gat
                               /* float32 out */ 1, 0, 1.0f, 0.0f, stream);
     if (e) return e;
   }
-  hipLaunchKernelGGL(routed_combine_kernel, dim3(n_rows), dim3(256), 0, stream, ys, place, weights, K,
-                     (const bf16_t*)h, ldh, y, ldy, D, in_weights);
+  const dim3 gc(n_rows, ceil_div(D, 1024));
+  if (D % 4 == 0 && ldy % 4 == 0 && ((uintptr_t)y & 15u) == 0)
+    hipLaunchKernelGGL(routed_combine_kernel<true>, gc, dim3(256), 0, stream, ys, place, weights, K, (const bf16_t*)h, ldh,
+                       y, ldy, D, in_weights);
+  else
+    hipLaunchKernelGGL(routed_combine_kernel<false>, gc, dim3(256), 0, stream, ys, place, weights, K, (const bf16_t*)h, ldh,
+                       y, ldy, D, in_weights);
   APC_LAUNCH_CHECK();
   return 0;
 }

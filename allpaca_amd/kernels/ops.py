@@ -1037,6 +1037,11 @@ def latent_rows(proj: torch.Tensor, n_heads: int, head_dim: int, rot_dim: int, c
         _need(dr % 2 == 0 and cos_sin is not None and cos_sin.dtype == torch.float32 and cos_sin.is_contiguous()
               and cos_sin.dim() == 3 and tuple(cos_sin.shape[1:]) == (2, dr // 2),
               "cos/sin table must be float32 [positions, 2, rot/2]")
+    if _tuned_ok(proj, pages, q_out):
+        from . import tuned
+        if tuned.latent_rows_bf16(proj, ld, H, dn, dr, -1 if c_off is None else int(c_off), R, norm_w, eps, cos_sin, step,
+                                  block_table, pages, page_tokens, q_out, ldq):
+            return
     L = _lib.load("plain")
     _lib.check(L.apc_latent_rows(
         proj.data_ptr(), _code(proj), ld, H, dn, dr, -1 if c_off is None else int(c_off), R, _f32(norm_w, R, "norm weight"),

@@ -715,8 +715,23 @@ def heads_linear_bf16(a: torch.Tensor, a_head: int, w: PackedHeads, out: torch.T
                                      T, w.H, w.N, w.K, _ops._stream()), "heads_gemm_bf16")
 
 
+def latent_rows_bf16(proj, ld, H, dn, dr, c_off, R, norm_w, eps, cos_sin, step, block_table, pages, page_tokens, q_out,
+                     ldq) -> bool:
+    """The same on 16-byte accesses; False (nothing done) for sizes the kernel does not take."""
+    L = _lib.load("tuned")
+    T = proj.shape[0]
+    if not L.apc_latent_rows_bf16_takes(ld, dn, dr, c_off, R, ldq) or not _aligned(proj, pages, q_out, cos_sin):
+        return False
+    _lib.check(L.apc_latent_rows_bf16(
+        proj.data_ptr(), ld, H, dn, dr, c_off, R, _ops._f32(norm_w, R, "norm weight"), float(eps), cos_sin.data_ptr(),
+        _ops._i32(step.positions, T, "positions"), _ops._i32(step.row_seg, T, "row_seg"), block_table.data_ptr(),
+        block_table.shape[1], pages.data_ptr(), page_tokens, q_out.data_ptr(), ldq, T, _ops._stream()), "latent_rows_bf16")
+    return True
+
+
 LATENT_BLOCKS = 256          # blocks that the keys of few rows are cut for (a block a compute unit at a latent of 512)
-LATENT_SPLITS_MAX = 32
+LATENT_SPLITS_MAX = 128      # (the adding kernel takes up to 256; 128 was the fastest for one row over 32,768 keys)
+LATENT_DECODE_TILES = 2      # key tiles that a range of a decoded row's keys must keep
 LATENT_RANGE_TILES = 8       # key tiles (of 64) that a range of a prompt tile's keys must keep
 
 
@@ -757,6 +772,6 @@ def latent_attention_bf16(q, out, n_heads: int, rank: int, rot_dim: int, pages, 
     if step.n_decode_rows:
         n = step.n_decode_rows
         blocks = n * -(-H // (64 if H > 32 else 32))
-        splits = max(1, min(LATENT_BLOCKS // blocks, -(-step.max_decode_context // 64), LATENT_SPLITS_MAX))
+        splits = max(1, min(LATENT_BLOCKS // blocks, -(-step.max_decode_context // (64 * LATENT_DECODE_TILES)), LATENT_SPLITS_MAX))
         run(step.decode_rows, None, n, 1, splits, "latent_attention_bf16 (decoded rows)")
     return True

@@ -56,6 +56,7 @@ def check_latent_attention(H, R, dr, P_, segs, dtype, seed, scale=0.8, plant=(),
     if splits is not None:
         monkeypatch.setattr(tuned, "LATENT_BLOCKS", splits)
         monkeypatch.setattr(tuned, "LATENT_RANGE_TILES", 1)
+        monkeypatch.setattr(tuned, "LATENT_DECODE_TILES", 1)
     ops.latent_attention(dev(q.reshape(T, -1), tdt), out, H, R, dr, cache, P_, step.block_tables[0], step, scale)
     got = out.float().cpu().numpy().reshape(T, H, R)
     for i, ((p0, n), c) in enumerate(zip(segs, cs)):
