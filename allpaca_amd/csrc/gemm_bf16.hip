@@ -9,7 +9,7 @@
 // as 2 x 2 v_mfma_f32_32x32x16_bf16 accumulators.  Global loads run two K steps ahead of the MFMAs, and
 // loads and LDS stores are spread between the MFMAs of a step: LDS bandwidth (reads of operands plus stores of
 // the next step) and the load path are each about as busy as the matrix cores, so none of them may wait for another.
-// Epilogues: store bfloat16 / float32, add into a float32 residual, the squared relu in bfloat16 (grouped rows only), or SwiGLU: then the W tile is
+// Epilogues: store bfloat16 / float32, add into a float32 residual, an activation on the sums (bfloat16 out), or SwiGLU: then the W tile is
 // 64 gate rows and the matching 64 up rows, each wave computes gate and up of the same 64 x 32 outputs,
 // and the block writes a 128 x 64 tile of silu(gate) * up.
 // With 17..128 rows and a long K, K is cut into slices for different blocks and a second kernel adds the slices in
@@ -28,7 +28,7 @@ constexpr int BN = 128, BK = 64;
 constexpr int BM_ROWS = 128;
 constexpr int LDS_ROW = BK + 8;  // bfloat16 elements per LDS row (144 bytes)
 
-enum { G_STORE_BF16 = 0, G_STORE_F32 = 1, G_ACC_F32 = 2, G_SWIGLU = 3, G_PARTIAL = 4, G_RELU2 = 5 };
+enum { G_STORE_BF16 = 0, G_STORE_F32 = 1, G_ACC_F32 = 2, G_SWIGLU = 3, G_PARTIAL = 4, G_ACT = 5 };
 
 template <int BM>
 struct GemmRegs {
@@ -48,7 +48,8 @@ struct TiledPre {
 // side): `tiles` holds (matrix, first row, rows) of every row tile, `*n_tiles` of them, and matrix e starts
 // `w_stride` elements behind matrix e - 1.  The grid is (column tiles, most row tiles there can be); a block beyond
 // the tiles that exist leaves at once.  tiles == nullptr: one matrix for all rows.  act, alpha, limit: the activation of
-// the gated unit in mode G_SWIGLU (see gated_unit_act; 0: silu(g) * u).
+// the gated unit in mode G_SWIGLU (see gated_unit_act; 0: silu(g) * u); act: the activation in mode G_ACT (see
+// activation_f).
 struct GroupedRows {
   const int* tiles;
   const int* n_tiles;
@@ -95,7 +96,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
     const int e = grp.tiles[3 * ti], p0 = grp.tiles[3 * ti + 1];
     M = grp.tiles[3 * ti + 2];                       // the tile's rows are all the rows this block knows of
     A += (size_t)p0 * lda;
-    C = (char*)C + (size_t)p0 * ldc * (MODE == G_STORE_BF16 || MODE == G_SWIGLU || MODE == G_RELU2 ? 2 : 4);
+    C = (char*)C + (size_t)p0 * ldc * (MODE == G_STORE_BF16 || MODE == G_SWIGLU || MODE == G_ACT ? 2 : 4);
     W += (size_t)e * grp.w_stride;
     if (MODE == G_SWIGLU) W2 += (size_t)e * grp.w_stride;
   } else {
@@ -313,7 +314,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
           if (n >= N) continue;
           const size_t o = (size_t)m * ldc + n;
           if (MODE == G_STORE_BF16) ((bf16_t*)C)[o] = float_to_bf16(acc[a][b][r]);
-          else if (MODE == G_RELU2) ((bf16_t*)C)[o] = float_to_bf16(fmaxf(acc[a][b][r], 0.f) * fmaxf(acc[a][b][r], 0.f));
+          else if (MODE == G_ACT) ((bf16_t*)C)[o] = float_to_bf16(activation_f(acc[a][b][r], grp.act));
           else if (MODE == G_STORE_F32) ((float*)C)[o] = acc[a][b][r];
           else if (MODE == G_ACC_F32) ((float*)C)[o] += acc[a][b][r];
           else ((float*)C)[((size_t)blockIdx.z * M + m) * N + n] = acc[a][b][r];
@@ -327,9 +328,11 @@ static bool aligned16(const void* p) { return ((uintptr_t)p & 15u) == 0; }
 
 template <int MODE, bool PRE = false>
 static int launch_gemm(const bf16_t* A, int lda, const bf16_t* W, const bf16_t* W2, void* C, int ldc, int M, int N,
-                       int K, hipStream_t stream, TiledPre pre = TiledPre{}) {
+                       int K, hipStream_t stream, TiledPre pre = TiledPre{}, int act = 0) {
   constexpr int NB = MODE == G_SWIGLU ? BN / 2 : BN;
-  if constexpr (!PRE) {
+  if constexpr (MODE == G_ACT) {
+    if (gemm_direct_takes(G_STORE_BF16, A, lda, C, ldc, M, N, K)) return launch_gemm_direct_act(act, A, lda, W, C, ldc, M, N, K, stream);
+  } else if constexpr (!PRE) {
     // many rows, K a multiple of 128: the kernel that keeps the weights out of LDS (same sums, bit for bit)
     if (gemm_direct_takes(MODE, A, lda, C, ldc, M, N, K)) return launch_gemm_direct(MODE, A, lda, W, W2, C, ldc, M, N, K, stream);
   } else if constexpr (MODE == G_SWIGLU || MODE == G_STORE_BF16) {
@@ -364,7 +367,7 @@ static int launch_gemm(const bf16_t* A, int lda, const bf16_t* W, const bf16_t* 
   if (blocks > 0x7fffffffL) return APC_ERR_BAD_ARG;
 #define TILED_LAUNCH(EVEN_, BM_, DEPTH_)                                                                              \
   hipLaunchKernelGGL((gemm_bf16_kernel<MODE, EVEN_, BM_, PRE, DEPTH_>), dim3((unsigned)blocks), dim3(256), 0, stream, A, \
-                     lda, W, W2, ceil_div(K, 32), C, ldc, M, N, K, 1, pre)
+                     lda, W, W2, ceil_div(K, 32), C, ldc, M, N, K, 1, pre, GroupedRows{nullptr, nullptr, 0, act})
 #define TILED_BY_K(BM_, DEPTH_)                     \
   if (K % BK == 0) TILED_LAUNCH(true, BM_, DEPTH_); \
   else TILED_LAUNCH(false, BM_, DEPTH_)
@@ -390,6 +393,7 @@ struct FinishNorm {
   bf16_t* raw;
   int ld_raw;
   float* emit_ss;
+  int act = 0;      // mode G_ACT: the activation
 };
 
 // Sums the float32 sums that G_PARTIAL blocks left ([which][slice][M][N], slices in order) and finishes:
@@ -415,6 +419,7 @@ __global__ __launch_bounds__(256) void gemm_finish_kernel(const float* __restric
   float sq = 0.f;
   if (on) {
     if (mode == G_STORE_BF16) ((bf16_t*)C)[o] = float_to_bf16(g);
+    else if (mode == G_ACT) ((bf16_t*)C)[o] = float_to_bf16(activation_f(g, norm.act));
     else if (mode == G_STORE_F32) ((float*)C)[o] = g;
     else if (mode == G_ACC_F32) {
       const float x = ((float*)C)[o] + g;
@@ -471,7 +476,7 @@ static int launch_partials(const void* A, int lda, const void* W, const void* Wu
 // or added into the residual.  N and ldc multiples of 4, 16-byte aligned rows.  (One output a thread takes 34 us for
 // 2,048 x 4,096 outputs in two slices, this 13.)
 __global__ __launch_bounds__(256) void gemm_finish4_kernel(const float* __restrict__ partials, int k_split, int M, int N,
-                                                           int mode, void* __restrict__ C, int ldc) {
+                                                           int mode, void* __restrict__ C, int ldc, int act) {
   const int n4 = N / 4;
   const size_t total = (size_t)M * n4, plane = (size_t)M * N;
   for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
@@ -480,7 +485,9 @@ __global__ __launch_bounds__(256) void gemm_finish4_kernel(const float* __restri
     floatx4 g = *reinterpret_cast<const floatx4*>(src);
     for (int s = 1; s < k_split; ++s) g += *reinterpret_cast<const floatx4*>(src + s * plane);
     const size_t o = (size_t)m * ldc + n;
-    if (mode == G_STORE_BF16) {
+    if (mode == G_ACT)
+      for (int k = 0; k < 4; ++k) g[k] = activation_f(g[k], act);
+    if (mode == G_STORE_BF16 || mode == G_ACT) {
       uint2 pk;
       pk.x = pack_bf16x2(g[0], g[1]);
       pk.y = pack_bf16x2(g[2], g[3]);
@@ -499,13 +506,20 @@ static int launch_splitk(const void* A, int lda, const void* W, const void* Wu, 
                          hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
   if (ldc < N) return APC_ERR_BAD_ARG;
-  if (mode < 0 || mode > G_SWIGLU || (mode == G_SWIGLU) != (Wu != nullptr)) return APC_ERR_BAD_ARG;
+  if (mode_is_act(mode)) {
+    if (pre) return APC_ERR_BAD_ARG;
+    norm.act = mode - MODE_ACT;
+    mode = G_ACT;
+  } else if (mode < 0 || mode > G_SWIGLU) {
+    return APC_ERR_BAD_ARG;
+  }
+  if ((mode == G_SWIGLU) != (Wu != nullptr)) return APC_ERR_BAD_ARG;
   const int e = launch_partials(A, lda, W, Wu, M, N, K, k_split, workspace, stream);
   if (e) return e;
   if (!pre && !emit && mode != G_SWIGLU && N % 4 == 0 && ldc % 4 == 0 && aligned16(C) && (long)M * N >= (1L << 20)) {
     const long want = ((long)M * (N / 4) + 255) / 256;
     hipLaunchKernelGGL(gemm_finish4_kernel, dim3((unsigned)(want < 8192 ? want : 8192)), dim3(256), 0, stream, workspace,
-                       k_split, M, N, mode, C, ldc);
+                       k_split, M, N, mode, C, ldc, norm.act);
     APC_LAUNCH_CHECK();
     return 0;
   }
@@ -581,7 +595,7 @@ __global__ __launch_bounds__(256) void gemm_finish_qkv_rope_kernel(const float* 
 
 // Product for 17..128 rows: K is cut into `k_split` slices that different blocks multiply, so that matrices with
 // few output columns still give the chip enough blocks; `workspace` holds (Wu ? 2 : 1) * k_split * M * N floats.
-// mode as below, or 3 for SwiGLU (W = gate, Wu = up).
+// mode as below, or 3 for SwiGLU (W = gate, Wu = up), or 17 .. 19 (see apc_gemm_bf16).
 // How many slices of K the product of many rows (gemm_direct_bf16.hip) wants for this shape: 1, or 2 when narrow
 // tiles would be needed to fill the chip otherwise.  The caller brings the workspace for apc_gemm_splitk_bf16.
 APC_EXPORT int apc_gemm_direct_k_split(int M, int N, int K) { return gemm_direct_k_split(M, N, K); }
@@ -627,7 +641,8 @@ APC_EXPORT int apc_gemm_splitk_pre_bf16(const void* A, int lda, const float* ss,
   return launch_splitk(A, lda, W, Wu, C, ldc, M, N, K, mode, k_split, workspace, 1, 0, norm, stream);
 }
 
-// W: tiled layout of an [N, K] matrix.  mode: 0 store bfloat16, 1 store float32, 2 add into float32
+// W: tiled layout of an [N, K] matrix.  mode: 0 store bfloat16, 1 store float32, 2 add into float32, 17 .. 19: an
+// activation (see activation_f; 16 + its code) on the sums, then store bfloat16
 APC_EXPORT int apc_gemm_bf16(const void* A, int lda, const void* W, void* C, int ldc, int M, int N, int K, int mode,
                              hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
@@ -635,6 +650,7 @@ APC_EXPORT int apc_gemm_bf16(const void* A, int lda, const void* W, void* C, int
   if (K % 8 || lda % 8 || !aligned16(A) || !aligned16(W)) return APC_ERR_UNSUPPORTED;
   const bf16_t* a = (const bf16_t*)A;
   const bf16_t* w = (const bf16_t*)W;
+  if (mode_is_act(mode)) return launch_gemm<G_ACT>(a, lda, w, nullptr, C, ldc, M, N, K, stream, TiledPre{}, mode - MODE_ACT);
   switch (mode) {
     case G_STORE_BF16: return launch_gemm<G_STORE_BF16>(a, lda, w, nullptr, C, ldc, M, N, K, stream);
     case G_STORE_F32: return launch_gemm<G_STORE_F32>(a, lda, w, nullptr, C, ldc, M, N, K, stream);
@@ -644,13 +660,15 @@ APC_EXPORT int apc_gemm_bf16(const void* A, int lda, const void* W, void* C, int
 }
 
 // Rows in runs of one matrix each (see GroupedRows): mode G_SWIGLU (W, W2: gate and up; bfloat16 out; act, alpha, limit:
-// the gated unit's activation), G_RELU2 (the square of max(sum, 0), bfloat16 out) or G_STORE_F32.  tile_rows: 64 or 128, the rows `tiles` was cut for.
+// the gated unit's activation), G_ACT (act: the
+// activation on the sums, bfloat16 out) or G_STORE_F32.  tile_rows: 64 or 128, the rows `tiles` was cut for.
 APC_EXPORT int apc_gemm_grouped_bf16(const void* A, int lda, const void* W, const void* W2, size_t w_stride, void* C,
                                      int ldc, const int* tiles, const int* n_tiles, int max_tiles, int tile_rows,
                                      int N, int K, int mode, int act, float alpha, float limit, hipStream_t stream) {
   if (max_tiles <= 0) return 0;
   if (N <= 0 || K <= 0 || K % 8 || lda % 8 || !tiles || !n_tiles || (tile_rows != 64 && tile_rows != 128) ||
-      (mode != G_SWIGLU && mode != G_STORE_F32 && mode != G_RELU2) || (mode == G_SWIGLU && !W2) || max_tiles > 65535 || act < 0 || act > 1)
+      (mode != G_SWIGLU && mode != G_STORE_F32 && mode != G_ACT) || (mode == G_SWIGLU && (!W2 || act > 1)) || max_tiles > 65535 || act < 0 ||
+      act > 3)
     return APC_ERR_BAD_ARG;
   if (!aligned16(A) || !aligned16(W) || (W2 && !aligned16(W2))) return APC_ERR_UNSUPPORTED;
   const GroupedRows grp{tiles, n_tiles, w_stride, act, alpha, limit};
@@ -671,7 +689,7 @@ APC_EXPORT int apc_gemm_grouped_bf16(const void* A, int lda, const void* W, cons
     }                                                                        \
   } while (0)
   if (mode == G_SWIGLU) GROUPED_BY(G_SWIGLU);
-  else if (mode == G_RELU2) GROUPED_BY(G_RELU2);
+  else if (mode == G_ACT) GROUPED_BY(G_ACT);
   else GROUPED_BY(G_STORE_F32);
 #undef GROUPED_BY
 #undef GROUPED_LAUNCH

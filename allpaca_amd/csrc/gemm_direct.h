@@ -12,6 +12,9 @@ bool gemm_direct_takes(int mode, const void* A, int lda, const void* C, int ldc,
 // W, W2 in the tiled layout.  APC_ERR_UNSUPPORTED for a shape that gemm_direct_takes refuses.
 int launch_gemm_direct(int mode, const bf16_t* A, int lda, const bf16_t* W, const bf16_t* W2, void* C, int ldc, int M,
                        int N, int K, hipStream_t stream);
+// Mode 0 with an activation (see activation_f) on the sums; for shapes that gemm_direct_takes in mode 0.
+int launch_gemm_direct_act(int act, const bf16_t* A, int lda, const bf16_t* W, void* C, int ldc, int M, int N, int K,
+                           hipStream_t stream);
 // Products on rows that a product into the residual left for the RMS norm (A = the rows times the norm's weight, ss =
 // [M][ss_parts] sums of x^2): the sums are scaled by 1 / sqrt(sum(ss[m]) / K + eps), before the activation where there
 // is one.  mode 0 (store bfloat16) or 3 (SwiGLU).  SwiGLU from GEMM_DIRECT_PRE_MIN_ROWS rows on: the 28,672 weight

@@ -31,7 +31,7 @@ namespace {
 // D_..._PRE: A is a row that a product into the residual left for the RMS norm, and the sums are scaled by the row's
 // 1 / sqrt(mean of x^2 + eps).  D_ACC_EMIT: add into the residual and leave that row for the norm that reads it next.
 enum { D_STORE_BF16 = 0, D_STORE_F32 = 1, D_ACC_F32 = 2, D_SWIGLU = 3, D_SWIGLU_PRE = 4, D_ACC_EMIT = 5,
-       D_STORE_BF16_PRE = 6 };
+       D_STORE_BF16_PRE = 6, D_STORE_ACT = 7 };
 __host__ __device__ constexpr bool is_swiglu(int mode) { return mode == D_SWIGLU || mode == D_SWIGLU_PRE; }
 __host__ __device__ constexpr bool is_pre(int mode) { return mode == D_SWIGLU_PRE || mode == D_STORE_BF16_PRE; }
 
@@ -46,6 +46,7 @@ struct DirectPre {
   bf16_t* raw;
   int ldr;
   int part0;
+  int act;           // D_STORE_ACT: the activation on the sums
 };
 
 constexpr int R = 4;           // ring slots of W fragments: loads run R - 1 steps of 32 columns ahead
@@ -285,6 +286,7 @@ __device__ __forceinline__ void direct_tile(int bid, const bf16_t* __restrict__ 
 #pragma unroll
           for (int r = 0; r < 4; ++r)
             v[r] = MODE == D_STORE_BF16       ? acc[a][f][r]
+                   : MODE == D_STORE_ACT      ? activation_f(acc[a][f][r], pre.act)
                    : MODE == D_STORE_BF16_PRE ? acc[a][f][r] * row_scale[a]
                    : MODE == D_SWIGLU         ? silu_f(acc[a][f][r]) * acc[a][NOUT + f][r]
                                               : silu_f(acc[a][f][r] * row_scale[a]) * (acc[a][NOUT + f][r] * row_scale[a]);
@@ -454,7 +456,7 @@ int launch_gemm_direct_slices(const bf16_t* A, int lda, const bf16_t* W, float* 
 
 namespace {
 bool direct_takes(int mode, int min_rows, const void* A, int lda, const void* C, int ldc, int M, int N, int K) {
-  if (mode < 0 || mode > D_STORE_BF16_PRE || M < min_rows || K < 128 || K % 128 || N % 4 || ldc % 4) return false;
+  if (mode < 0 || mode > D_STORE_ACT || M < min_rows || K < 128 || K % 128 || N % 4 || ldc % 4) return false;
   if (((uintptr_t)A & 15u) || ((uintptr_t)C & 15u) || lda % 8) return false;
   // the lanes' byte offsets into the block's rows of A and the wave's bands of W are 32-bit
   if ((long)128 * lda * 2 >= 0x7fffffffL || (long)8 * ceil_div(K, 32) * 1024 >= 0x7fffffffL) return false;
@@ -469,6 +471,7 @@ int launch_columns(int nf, int mode, const bf16_t* A, int lda, const bf16_t* W, 
     case D_ACC_F32: return launch_mode<D_ACC_F32>(nf, A, lda, W, W2, C, ldc, M, N, K, stream, pre);
     case D_SWIGLU: return launch_mode<D_SWIGLU>(nf, A, lda, W, W2, C, ldc, M, N, K, stream, pre);
     case D_SWIGLU_PRE: return launch_mode<D_SWIGLU_PRE>(nf, A, lda, W, W2, C, ldc, M, N, K, stream, pre);
+    case D_STORE_ACT: return launch_mode<D_STORE_ACT>(nf, A, lda, W, W2, C, ldc, M, N, K, stream, pre);
     case D_ACC_EMIT: return launch_mode<D_ACC_EMIT>(nf, A, lda, W, W2, C, ldc, M, N, K, stream, pre);
     default: return launch_mode<D_STORE_BF16_PRE>(nf, A, lda, W, W2, C, ldc, M, N, K, stream, pre);
   }
@@ -516,7 +519,7 @@ int launch_direct(int mode, const bf16_t* A, int lda, const bf16_t* W, const bf1
   const int e = launch_columns(plan.nf1, mode, A, lda, W, W2, C, ldc, M, plan.cols1, K, stream, pre);
   if (e) return e;
   const size_t w_skip = (size_t)(plan.cols1 / 16) * ceil_div(K, 32) * 512;  // whole bands of the tiled layout
-  const size_t elem = (mode == D_STORE_BF16 || mode == D_STORE_BF16_PRE || swiglu) ? 2 : 4;
+  const size_t elem = (mode == D_STORE_BF16 || mode == D_STORE_BF16_PRE || mode == D_STORE_ACT || swiglu) ? 2 : 4;
   if (mode == D_ACC_EMIT) {
     pre.g += plan.cols1;
     pre.raw += plan.cols1;
@@ -535,6 +538,14 @@ int launch_gemm_direct(int mode, const bf16_t* A, int lda, const bf16_t* W, cons
                        int N, int K, hipStream_t stream) {
   if (!gemm_direct_takes(mode, A, lda, C, ldc, M, N, K) || (mode == D_SWIGLU) != (W2 != nullptr)) return APC_ERR_UNSUPPORTED;
   return launch_direct(mode, A, lda, W, W2, C, ldc, M, N, K, stream, DirectPre{});
+}
+
+int launch_gemm_direct_act(int act, const bf16_t* A, int lda, const bf16_t* W, void* C, int ldc, int M, int N, int K,
+                           hipStream_t stream) {
+  if (!gemm_direct_takes(D_STORE_BF16, A, lda, C, ldc, M, N, K)) return APC_ERR_UNSUPPORTED;
+  DirectPre pre{};
+  pre.act = act;
+  return launch_direct(D_STORE_ACT, A, lda, W, nullptr, C, ldc, M, N, K, stream, pre);
 }
 
 bool gemm_direct_pre_takes(int mode, const void* A, int lda, const void* C, int ldc, int M, int N, int K, int ss_parts) {

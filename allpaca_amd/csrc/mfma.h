@@ -55,6 +55,20 @@ __device__ __forceinline__ floatx16 mfma32(const Frag& a, const Frag& b, floatx1
 }
 
 __device__ __forceinline__ float silu_f(float g) { return g / (1.0f + __expf(-g)); }
+// An activation by code: 1 silu, 2 the square of max(z, 0), 3 gelu in its tanh form (tanh by one exponential, off by
+// about 1e-7), else z itself.
+__device__ __forceinline__ float activation_f(float z, int kind) {
+  if (kind == 1) return silu_f(z);
+  if (kind == 2) { const float r = fmaxf(z, 0.f); return r * r; }
+  if (kind == 3) {
+    const float e = __expf(-2.0f * 0.7978845608028654f * (z + 0.044715f * z * z * z));     // (1 + tanh t) / 2 = 1 / (1 + e)
+    return z / (1.0f + e);
+  }
+  return z;
+}
+// modes of the products from this one on: an activation (MODE_ACT + its code) on the sums, bfloat16 out
+constexpr int MODE_ACT = 16, MODE_ACT_LAST = MODE_ACT + 3;
+__host__ __device__ constexpr bool mode_is_act(int mode) { return mode > MODE_ACT && mode <= MODE_ACT_LAST; }
 // a gated unit's activation.  kind 0: silu(g) * u; kind 1, the clamped unit: g' * sigmoid(alpha g') * (u' + 1) with
 // g' = min(g, limit) and u' = clamp(u, -limit, limit)
 __device__ __forceinline__ float gated_unit_act(float g, float u, int kind, float alpha, float limit) {

@@ -359,7 +359,7 @@ APC_EXPORT int apc_routed_experts_bf16(const void* h, int ldh, const void* w_gat
     const size_t gate_elems = (size_t)ceil_div(F, 16) * ceil_div(D, 32) * TILE_ELEMS;
     const size_t down_elems = (size_t)ceil_div(D, 16) * ceil_div(F, 32) * TILE_ELEMS;
     int e = kind == 2 ? apc_gemm_grouped_bf16(hs, D, w_gate_up, nullptr, gate_elems, act, F, tiles, n_tiles, max_tiles,
-                                              tile_rows, F, D, /* squared relu */ 5, 0, 1.0f, 0.0f, stream)
+                                              tile_rows, F, D, /* squared relu */ 5, 2, 1.0f, 0.0f, stream)
                       : apc_gemm_grouped_bf16(hs, D, w_gate_up, (const bf16_t*)w_gate_up + gate_elems, 2 * gate_elems,
                                               act, F, tiles, n_tiles, max_tiles, tile_rows, F, D, /* gated unit */ 3,
                                               kind, alpha, limit, stream);

@@ -29,7 +29,7 @@
 constexpr int SK_U = 4;              // tiles (32 k each) per band per step
 constexpr int TILE_ELEMS = 16 * 32;  // elements of a tile
 
-enum { SK_STORE_BF16 = 0, SK_STORE_F32 = 1, SK_ACC_F32 = 2, SK_SWIGLU = 3, SK_QKV_ROPE = 4 };
+enum { SK_STORE_BF16 = 0, SK_STORE_F32 = 1, SK_ACC_F32 = 2, SK_SWIGLU = 3, SK_QKV_ROPE = 4, SK_ACT = 5 };
 
 template <int MT, int NB, int U>
 struct SkRegs {
@@ -51,6 +51,7 @@ struct SkNorm {
   const float* g;
   bf16_t* raw;
   int ld_raw;
+  int act = 0;   // SK_ACT: the activation on the sums (see activation_f), bfloat16 out
 };
 
 // SK_QKV_ROPE: the product that gives q, k and v of a row also turns q and k by the row's position and writes k
@@ -298,8 +299,12 @@ __global__ __launch_bounds__(WPB * 64, sk_blocks(MODE, WPB)) void skinny_gemm_ke
     }
     float sq = 0.f;  // EMIT: x^2 over this lane's columns
     if (fin_vec) {
-      if (MODE == SK_STORE_BF16 || MODE == SK_SWIGLU) {
+      if (MODE == SK_STORE_BF16 || MODE == SK_SWIGLU || MODE == SK_ACT) {
         floatx4 y = sum[0];
+        if (MODE == SK_ACT) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) y[r] = activation_f(sum[0][r], norm.act);
+        }
         if (MODE == SK_SWIGLU) {
 #pragma unroll
           for (int r = 0; r < 4; ++r) y[r] = silu_f(sum[0][r]) * sum[NSUM - 1][r];
@@ -329,6 +334,7 @@ __global__ __launch_bounds__(WPB * 64, sk_blocks(MODE, WPB)) void skinny_gemm_ke
         if (n >= N) continue;
         const size_t o = (size_t)m * ldc + n;
         if (MODE == SK_STORE_BF16) ((bf16_t*)C)[o] = float_to_bf16(sum[0][r]);
+        else if (MODE == SK_ACT) ((bf16_t*)C)[o] = float_to_bf16(activation_f(sum[0][r], norm.act));
         else if (MODE == SK_STORE_F32) ((float*)C)[o] = sum[0][r];
         else if (MODE == SK_ACC_F32) {
           const float x = ((float*)C)[o] + sum[0][r];
@@ -371,7 +377,7 @@ static int launch_skinny(const bf16_t* A, int lda, const bf16_t* W, const bf16_t
   if ((MODE == SK_SWIGLU || MODE == SK_QKV_ROPE) && wpb > 8) wpb = 8;
   if (PRE && norm.ld_ss > 4 * 4 * wpb * SS_LOADS) return APC_ERR_UNSUPPORTED;
   // whole 16-byte (float32) or 8-byte (bfloat16) accesses to C and to the emitted row where everything is aligned
-  const int elem = (MODE == SK_STORE_BF16 || MODE == SK_SWIGLU) ? 2 : 4;
+  const int elem = (MODE == SK_STORE_BF16 || MODE == SK_SWIGLU || MODE == SK_ACT) ? 2 : 4;
   int vec_c = ldc % 4 == 0 && ((uintptr_t)C % (4 * elem)) == 0;
   if (EMIT) vec_c = vec_c && norm.ld_raw % 4 == 0 && ((uintptr_t)norm.raw % 8) == 0 && aligned16(norm.g);
 #define SK_LAUNCH(NB_, WPB_)                                                                                  \
@@ -400,7 +406,8 @@ static bool operands_ok(const void* A, int lda, const void* W, int M, int K) {
   return M <= 16 && K % 8 == 0 && lda % 8 == 0 && aligned16(A) && aligned16(W);
 }
 
-// W: tiled layout of an [N, K] matrix.  mode: 0 store bfloat16, 1 store float32, 2 add into float32
+// W: tiled layout of an [N, K] matrix.  mode: 0 store bfloat16, 1 store float32, 2 add into float32, 17 .. 19: an
+// activation (see activation_f; 16 + its code) on the sums, then store bfloat16
 APC_EXPORT int apc_skinny_gemm_bf16(const void* A, int lda, const void* W, void* C, int ldc, int M, int N, int K,
                                     int mode, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
@@ -408,7 +415,11 @@ APC_EXPORT int apc_skinny_gemm_bf16(const void* A, int lda, const void* W, void*
   if (!operands_ok(A, lda, W, M, K)) return APC_ERR_UNSUPPORTED;
   const bf16_t* a = (const bf16_t*)A;
   const bf16_t* w = (const bf16_t*)W;
-  const SkNorm none{};
+  SkNorm none{};
+  if (mode_is_act(mode)) {
+    none.act = mode - MODE_ACT;
+    return launch_skinny<SK_ACT, false, false>(a, lda, w, nullptr, C, ldc, M, N, K, none, stream);
+  }
   switch (mode) {
     case SK_STORE_BF16: return launch_skinny<SK_STORE_BF16, false, false>(a, lda, w, nullptr, C, ldc, M, N, K, none, stream);
     case SK_STORE_F32: return launch_skinny<SK_STORE_F32, false, false>(a, lda, w, nullptr, C, ldc, M, N, K, none, stream);

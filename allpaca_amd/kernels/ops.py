@@ -940,9 +940,13 @@ def weighted_pair(u: torch.Tensor, a: float, v: torch.Tensor, b: float, out: tor
 
 def linear_act(a: torch.Tensor, w, out: torch.Tensor, activation: str) -> None:
     """out = act(a . w^T): the product's sums are 32-bit, the activation is applied to them before they are stored in
-    `out`'s element type."""
+    `out`'s element type (in the product itself where it runs on the MFMA kernels)."""
     _need(activation in ACTIVATIONS, f"linear_act: activation {activation!r} is not one of {sorted(ACTIVATIONS)}")
     T, n = out.shape
+    if isinstance(w, PackedWeight) and out.dtype == torch.bfloat16:
+        from . import tuned
+        tuned.gemm_bf16(a, w, out, activation=ACTIVATIONS[activation])
+        return
     sums = torch.empty((T, n), dtype=torch.float32, device=a.device)
     linear(a, w, sums)
     act_rows(sums, out, activation)

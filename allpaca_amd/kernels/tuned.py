@@ -85,8 +85,12 @@ def _act_ok(a: torch.Tensor) -> bool:
     return (a.dtype == torch.bfloat16 and a.shape[1] % 8 == 0 and _ops._rows(a, "a") % 8 == 0 and _aligned(a))
 
 
-def gemm_bf16(a: torch.Tensor, w: PackedWeight, out: torch.Tensor, accumulate: bool = False) -> None:
-    """out = a . w^T (bfloat16 or float32 out), or out += a . w^T (float32 out); w in the tiled layout."""
+MODE_ACT = 16     # the products' modes from here on: an activation (MODE_ACT + its code) on the sums, bfloat16 out
+
+
+def gemm_bf16(a: torch.Tensor, w: PackedWeight, out: torch.Tensor, accumulate: bool = False, activation: int = 0) -> None:
+    """out = a . w^T (bfloat16 or float32 out), or out += a . w^T (float32 out); w in the tiled layout.  `activation`
+    (a code of `ops.ACTIVATIONS`): out = act(a . w^T), applied to the float32 sums, bfloat16 out."""
     _ops._gpu(a, w.data, out)
     M, K = a.shape
     N = w.N
@@ -96,13 +100,14 @@ def gemm_bf16(a: torch.Tensor, w: PackedWeight, out: torch.Tensor, accumulate: b
         raise ValueError(f"gemm: out must be [{M}, {N}], got {tuple(out.shape)}")
     _ops._need(not accumulate or out.dtype == torch.float32, "gemm: accumulation needs a float32 destination")
     _ops._need(out.dtype in (torch.bfloat16, torch.float32), "gemm: out must be bfloat16 or float32")
+    _ops._need(not activation or (not accumulate and out.dtype == torch.bfloat16), "gemm: an activation stores bfloat16")
     _ops._need(w.data.is_contiguous() and w.data.shape[0] * 16 >= N and w.data.shape[1] * 32 >= K,
                "gemm: the tiled weight does not cover [N, K]")
     if not _act_ok(a):
         raise ValueError("gemm_bf16: activations must be bfloat16 rows of a width and stride that are multiples "
                          "of 8, 16-byte aligned")
     lda, ldc = _ops._rows(a, "a"), _ops._rows(out, "out")
-    mode = 2 if accumulate else (0 if out.dtype == torch.bfloat16 else 1)
+    mode = MODE_ACT + activation if activation else 2 if accumulate else (0 if out.dtype == torch.bfloat16 else 1)
     L = _lib.load("tuned")
     if M > SKINNY_MAX_ROWS:
         # more than 1,024 rows: the product of many rows says itself whether it wants K in two slices
