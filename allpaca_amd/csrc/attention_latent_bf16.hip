@@ -82,8 +82,9 @@ __device__ __forceinline__ void scores_done(floatx4 (&s)[PT][2]) {
 // nothing moves across: LDS reads stay as far ahead of what takes them as they are written
 __device__ __forceinline__ void in_order() { __builtin_amdgcn_sched_barrier(0); }
 
-// RT: blocks of 32 value elements, NB: blocks of 32 elements of a row, PT: 32-pair groups a block of threads takes
-template <int RT, int NB, int PT>
+// RT: blocks of 32 value elements, NB: blocks of 32 elements of a row (EVEN: a row fills them), PT: 32-pair groups a block
+// of threads takes
+template <int RT, int NB, int PT, bool EVEN>
 __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, int H, int R, int L, const bf16_t* __restrict__ pages,
     int pshift, const int* __restrict__ block_table, int max_blocks, const int* __restrict__ positions,
@@ -92,8 +93,8 @@ __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
   static_assert(PT == 1 || PT == 2, "a wave's scores are PT * 16 keys x 32 pairs");
   constexpr int NP = PT * 32, NG = 4 / PT;      // pairs of a block; waves that share a pair's keys
   constexpr int NV = (RT + 3) / 4;              // value blocks a wave
-  __shared__ __attribute__((aligned(1024))) bf16_t buf0[NB * KT * 32];
-  __shared__ __attribute__((aligned(1024))) bf16_t buf1[NB * KT * 32];
+  constexpr int BUF = NB * KT * 32;             // elements of a tile's buffer
+  __shared__ __attribute__((aligned(1024))) bf16_t bufs[2 * BUF];
   __shared__ __attribute__((aligned(16))) bf16_t ps[NP * PROW];
   __shared__ float mx[NG * NP];
   const int lane = threadIdx.x % WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
@@ -114,28 +115,6 @@ __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
 
   const int kb = PT == 1 ? wave * 16 : (wave % 2) * 32, pb = PT == 1 ? 0 : (wave / 2) * 32;
   const int group = PT == 1 ? wave : wave % 2;
-  // this lane's pairs of the scores: pb + li and pb + 16 + li
-  u32x4 qf[2][NB];
-  int posq[2];
-#pragma unroll
-  for (int p = 0; p < 2; ++p) {
-    const int pair = min(pair0 + pb + p * 16 + li, n_pairs - 1);
-    posq[p] = pos0 + pair / H;
-    const bf16_t* src = q + ((size_t)row0 * H + pair) * L;
-#pragma unroll
-    for (int b = 0; b < NB; ++b) {
-      const int e = b * 32 + lc * 8;
-      Frag f = load_frag(src + min(e, L - 8));
-#pragma unroll
-      for (int k = 0; k < 4; ++k) f.w[k] = e < L ? f.w[k] : 0u;
-      qf[p][b] = __builtin_bit_cast(u32x4, f);
-    }
-  }
-#pragma unroll
-  for (int p = 0; p < 2; ++p)
-#pragma unroll
-    for (int b = 0; b < NB; ++b) asm volatile("" : "+a"(qf[p][b]));
-
   // direct loads: this wave brings keys 16 wave .. + 15 of a tile; a lane the piece (lane % 4) ^ (lane / 16) of every
   // block of key 16 wave + lane / 4.  Pieces behind the row's end bring the row's first one, whose products meet zeros.
   const int key_of_lane = wave * 16 + lane / 4, piece = (lane % 4) ^ lc;
@@ -149,9 +128,40 @@ __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
 #pragma unroll
     for (int b = 0; b < NB; ++b) {
       const int e = b * 32 + piece * 8;
-      load_to_lds(row + (e < L ? e : 0), at + b * (KT * 64));
+      load_to_lds(row + (EVEN || e < L ? e : 0), at + b * (KT * 64));
     }
   };
+  int next_page = 0;
+  if (j0 < j1) {                     // (the first tile is on its way while the queries come in)
+    fill(bufs, row_of(j0, page_of(j0)));
+    if (j0 + 1 < j1) next_page = page_of(j0 + 1);
+  }
+
+  // this lane's pairs of the scores: pb + li and pb + 16 + li
+  u32x4 qf[2][NB];
+  int posq[2];
+#pragma unroll
+  for (int p = 0; p < 2; ++p) {
+    const int pair = min(pair0 + pb + p * 16 + li, n_pairs - 1);
+    posq[p] = pos0 + pair / H;
+    const bf16_t* src = q + ((size_t)row0 * H + pair) * L;
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const int e = b * 32 + lc * 8;
+      Frag f = load_frag(src + (EVEN ? e : min(e, L - 8)));
+      if constexpr (!EVEN) {
+        uint32_t keep = e < L ? ~0u : 0u;
+        asm("" : "+v"(keep));                     // (a select would become a branch around every load)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) f.w[k] &= keep;
+      }
+      qf[p][b] = __builtin_bit_cast(u32x4, f);
+    }
+  }
+#pragma unroll
+  for (int p = 0; p < 2; ++p)
+#pragma unroll
+    for (int b = 0; b < NB; ++b) asm volatile("" : "+a"(qf[p][b]));
 
   floatx16 o[NV][PT];
 #pragma unroll
@@ -171,10 +181,11 @@ __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
   const int v_at0 = v_key * 32 + (v_col ^ (2 * hh)) * 8 + (lane % 2) * 4;
   const int v_at1 = (v_key + 4) * 32 + (v_col ^ (2 * hh + 1)) * 8 + (lane % 2) * 4;
 
-  int next_page = 0;
-  auto pass = [&](bf16_t* cur, bf16_t* nxt, int j) {
+  if (j0 < j1) loads_barrier();
+  for (int j = j0; j < j1; ++j) {
+    const bf16_t* cur = bufs + ((j - j0) & 1) * BUF;
     if (j + 1 < j1) {
-      fill(nxt, row_of(j + 1, next_page));
+      fill(bufs + ((j - j0 + 1) & 1) * BUF, row_of(j + 1, next_page));
       if (j + 2 < j1) next_page = page_of(j + 2);
     }
     // scores
@@ -298,16 +309,6 @@ __global__ __launch_bounds__(256, NB > 6 ? 1 : 2) void latent_attention_kernel(
       }
     }
     loads_barrier();
-  };
-
-  if (j0 < j1) {
-    fill(buf0, row_of(j0, page_of(j0)));
-    if (j0 + 1 < j1) next_page = page_of(j0 + 1);
-    loads_barrier();
-    for (int j = j0; j < j1; j += 2) {
-      pass(buf0, buf1, j);
-      if (j + 1 < j1) pass(buf1, buf0, j + 1);
-    }
   }
   // sums of the pairs' weights over all their keys
 #pragma unroll
@@ -440,14 +441,16 @@ APC_EXPORT int apc_latent_attention_bf16(const void* q, void* out, int H, int R,
   if ((long)blocks * n_items * n_splits > 0x7fffffffL || (long)pairs * n_items > 0x7fffffffL) return APC_ERR_UNSUPPORTED;
   const LatentItems items{row0, rows, n_items, blocks};
   const int pshift = __builtin_ctz(page_tokens);
-#define LATENT_LAUNCH(RT_, PT_)                                                                                         \
-  hipLaunchKernelGGL((latent_attention_kernel<RT_, RT_ + 2, PT_>), dim3(blocks * n_items * n_splits), dim3(256), 0,     \
+#define LATENT_LAUNCH(RT_, PT_, EVEN_)                                                                                         \
+  hipLaunchKernelGGL((latent_attention_kernel<RT_, RT_ + 2, PT_, EVEN_>), dim3(blocks * n_items * n_splits), dim3(256), 0,     \
                      stream, (const bf16_t*)q, (bf16_t*)out, H, R, L, (const bf16_t*)pages, pshift, block_table,        \
                      max_blocks, positions, row_seg, items, n_splits, scale * LOG2E, parts, ml)
-#define LATENT_BY(RT_)               \
-  do {                               \
-    if (two) LATENT_LAUNCH(RT_, 2);  \
-    else LATENT_LAUNCH(RT_, 1);      \
+#define LATENT_BY(RT_)                                       \
+  do {                                                       \
+    if (two && L == (RT_ + 2) * 32) LATENT_LAUNCH(RT_, 2, true); \
+    else if (two) LATENT_LAUNCH(RT_, 2, false);              \
+    else if (L == (RT_ + 2) * 32) LATENT_LAUNCH(RT_, 1, true);   \
+    else LATENT_LAUNCH(RT_, 1, false);                       \
   } while (0)
   if (rt == 2) LATENT_BY(2);
   else if (rt == 4) LATENT_BY(4);

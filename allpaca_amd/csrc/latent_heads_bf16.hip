@@ -138,7 +138,9 @@ __device__ __forceinline__ void rotate8(const bf16_t* src, bf16_t* dst, const fl
 
 // A block: one row.  The first wave norms the latent and rotates the shared key part into the row's place in its page
 // (8 elements a lane); the other waves rotate the queries' parts, 8 pairs a lane.  Sizes and strides are multiples of 8,
-// the rotated part of 16.  c_off < 0: queries only.
+// the rotated part of 16.  c_off < 0: queries only.  WAVE_ROW (steps of many rows): a wave does all of a row, a block
+// four rows.
+template <bool WAVE_ROW>
 __global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __restrict__ proj, int ld, int H, int dn,
                                                                int dr, int c_off, int R, const float* __restrict__ norm_w,
                                                                float eps, const float* __restrict__ cos_sin,
@@ -146,12 +148,14 @@ __global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __r
                                                                const int* __restrict__ row_seg,
                                                                const int* __restrict__ block_table, int max_blocks,
                                                                bf16_t* __restrict__ pages, int P, bf16_t* __restrict__ q,
-                                                               int ldq) {
-  const int r = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, half = dr / 2, L = R + dr;
+                                                               int ldq, int n_rows) {
+  const int r = WAVE_ROW ? blockIdx.x * 4 + threadIdx.x / WAVE : blockIdx.x;
+  if (r >= n_rows) return;
+  const int wave = WAVE_ROW ? 0 : threadIdx.x / WAVE, lane = threadIdx.x % WAVE, half = dr / 2, L = R + dr;
   const int pos = positions[r];
   const float* cs = cos_sin + (size_t)pos * dr;
   const bf16_t* row = proj + (size_t)r * ld;
-  int first = threadIdx.x, step = 256;
+  int first = WAVE_ROW ? lane : threadIdx.x, step = WAVE_ROW ? WAVE : 256;
   if (c_off >= 0) {
     if (wave == 0) {
       const bf16_t* src = row + c_off;
@@ -173,10 +177,12 @@ __global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __r
         *reinterpret_cast<Frag*>(dst + i) = pack8(v);
       }
       if (lane * 8 < half) rotate8(src + R, dst + R, cs, lane * 8, half);
-      return;
+      if (!WAVE_ROW) return;
     }
-    first -= WAVE;
-    step -= WAVE;
+    if (!WAVE_ROW) {
+      first -= WAVE;
+      step -= WAVE;
+    }
   }
   const int per_head = half / 8;
   for (int i = first; i < H * per_head; i += step) {
@@ -202,9 +208,13 @@ APC_EXPORT int apc_latent_rows_bf16(const void* proj, int ld, int H, int dn, int
       (c_off >= 0 && (ld < c_off + R + dr || !norm_w || !pages)) || ((uintptr_t)proj & 15u) || ((uintptr_t)q & 15u) ||
       ((uintptr_t)pages & 15u) || ((uintptr_t)cos_sin & 15u))
     return APC_ERR_BAD_ARG;
-  hipLaunchKernelGGL(latent_rows_bf16_kernel, dim3(n_rows), dim3(256), 0, stream, (const bf16_t*)proj, ld, H, dn, dr,
-                     c_off, R, norm_w, eps, cos_sin, positions, row_seg, block_table, max_blocks, (bf16_t*)pages, P,
-                     (bf16_t*)q, ldq);
+#define ROWS_LAUNCH(WAVE_ROW_, BLOCKS_)                                                                                 \
+  hipLaunchKernelGGL((latent_rows_bf16_kernel<WAVE_ROW_>), dim3(BLOCKS_), dim3(256), 0, stream, (const bf16_t*)proj, ld, \
+                     H, dn, dr, c_off, R, norm_w, eps, cos_sin, positions, row_seg, block_table, max_blocks,            \
+                     (bf16_t*)pages, P, (bf16_t*)q, ldq, n_rows)
+  if (n_rows >= 1024) ROWS_LAUNCH(true, ceil_div(n_rows, 4));
+  else ROWS_LAUNCH(false, n_rows);
+#undef ROWS_LAUNCH
   APC_LAUNCH_CHECK();
   return 0;
 }

@@ -152,41 +152,44 @@ __global__ __launch_bounds__(256) void tanh_norm_add_kernel(float* __restrict__ 
   if (h) store_f(h, h_dtype, (size_t)r * ldh + i, fmaf(squash<EXACT>(n.alpha * v), n.w[i], n.b[i]));
 }
 
-// The same for float32 x and y, VPT times 4 elements a thread on 16-byte accesses, all loads of x and y ahead of the
-// first store.
-template <bool EXACT, int VPT>
+// The same for float32 x and y, 4 elements of ROWS rows a thread on 16-byte accesses: weights and biases are read once for
+// the rows, and all loads of x and y go out ahead of the first store.
+template <bool EXACT, int ROWS>
 __global__ __launch_bounds__(256) void tanh_norm_add_f4_kernel(float* __restrict__ x, int ldx, const float* __restrict__ y,
                                                                int ldy, TanhNorm post, TanhNorm n, void* __restrict__ h,
-                                                               int h_dtype, int ldh, int dim) {
-  const int r = blockIdx.x, i0 = (blockIdx.y * VPT * 256 + threadIdx.x) * 4;
-  float4 xv[VPT], yv[VPT];
+                                                               int h_dtype, int ldh, int n_rows, int dim) {
+  const int r0 = blockIdx.x * ROWS, i = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (i >= dim) return;
+  const int rows = min(ROWS, n_rows - r0);
+  float4 xv[ROWS], yv[ROWS];
 #pragma unroll
-  for (int k = 0; k < VPT; ++k) {
-    const int i = i0 + k * 1024;
-    if (i < dim) {
-      xv[k] = *reinterpret_cast<const float4*>(x + (size_t)r * ldx + i);
-      yv[k] = *reinterpret_cast<const float4*>(y + (size_t)r * ldy + i);
-    }
+  for (int k = 0; k < ROWS; ++k) {
+    const size_t r = r0 + min(k, rows - 1);
+    xv[k] = *reinterpret_cast<const float4*>(x + r * ldx + i);
+    yv[k] = *reinterpret_cast<const float4*>(y + r * ldy + i);
+  }
+  const float4 pw = *reinterpret_cast<const float4*>(post.w + i), pb = *reinterpret_cast<const float4*>(post.b + i);
+  float4 w = float4{0.f, 0.f, 0.f, 0.f}, b = w;
+  if (h) {
+    w = *reinterpret_cast<const float4*>(n.w + i);
+    b = *reinterpret_cast<const float4*>(n.b + i);
   }
 #pragma unroll
-  for (int k = 0; k < VPT; ++k) {
-    const int i = i0 + k * 1024;
-    if (i >= dim) return;
-    const float4 pw = *reinterpret_cast<const float4*>(post.w + i), pb = *reinterpret_cast<const float4*>(post.b + i);
+  for (int k = 0; k < ROWS; ++k) {
+    if (k >= rows) return;
     float4 v;
     v.x = xv[k].x + fmaf(squash<EXACT>(post.alpha * yv[k].x), pw.x, pb.x);
     v.y = xv[k].y + fmaf(squash<EXACT>(post.alpha * yv[k].y), pw.y, pb.y);
     v.z = xv[k].z + fmaf(squash<EXACT>(post.alpha * yv[k].z), pw.z, pb.z);
     v.w = xv[k].w + fmaf(squash<EXACT>(post.alpha * yv[k].w), pw.w, pb.w);
-    *reinterpret_cast<float4*>(x + (size_t)r * ldx + i) = v;
+    *reinterpret_cast<float4*>(x + (size_t)(r0 + k) * ldx + i) = v;
     if (!h) continue;
-    const float4 w = *reinterpret_cast<const float4*>(n.w + i), b = *reinterpret_cast<const float4*>(n.b + i);
     float4 o;
     o.x = fmaf(squash<EXACT>(n.alpha * v.x), w.x, b.x);
     o.y = fmaf(squash<EXACT>(n.alpha * v.y), w.y, b.y);
     o.z = fmaf(squash<EXACT>(n.alpha * v.z), w.z, b.z);
     o.w = fmaf(squash<EXACT>(n.alpha * v.w), w.w, b.w);
-    const size_t at = (size_t)r * ldh + i;
+    const size_t at = (size_t)(r0 + k) * ldh + i;
     if (h_dtype == APC_F32) {
       *reinterpret_cast<float4*>((float*)h + at) = o;
     } else {
@@ -256,15 +259,15 @@ APC_EXPORT int apc_tanh_norm_add(float* x, int ldx, const void* y, int y_dtype, 
   auto a16 = [](const void* p) { return ((uintptr_t)p & 15u) == 0; };
   if (y_dtype == APC_F32 && dim % 4 == 0 && ldx % 4 == 0 && ldy % 4 == 0 && a16(x) && a16(y) && a16(pw) && a16(pb) &&
       (!h || (ldh % 4 == 0 && a16(h) && a16(w) && a16(b)))) {
-    const int vpt = n_rows >= 256 && dim > 1024 ? 2 : 1;       // (a step of few rows wants its blocks)
-    const dim3 grid(n_rows, ceil_div(dim, 1024 * vpt));
+    const int rows = n_rows >= 1024 ? 4 : 1;                  // (a step of few rows wants its blocks)
+    const dim3 grid(ceil_div(n_rows, rows), ceil_div(dim, 1024));
     if (grid.y > 65535) return APC_ERR_UNSUPPORTED;
-#define TANH_ADD(EXACT_, VPT_)                                                                                         \
-  hipLaunchKernelGGL((tanh_norm_add_f4_kernel<EXACT_, VPT_>), grid, dim3(256), 0, stream, x, ldx, (const float*)y, ldy, \
-                     post, n, h, h_dtype, ldh, dim)
-    if (exact && vpt == 2) TANH_ADD(true, 2);
+#define TANH_ADD(EXACT_, ROWS_)                                                                                         \
+  hipLaunchKernelGGL((tanh_norm_add_f4_kernel<EXACT_, ROWS_>), grid, dim3(256), 0, stream, x, ldx, (const float*)y, ldy, \
+                     post, n, h, h_dtype, ldh, n_rows, dim)
+    if (exact && rows == 4) TANH_ADD(true, 4);
     else if (exact) TANH_ADD(true, 1);
-    else if (vpt == 2) TANH_ADD(false, 2);
+    else if (rows == 4) TANH_ADD(false, 4);
     else TANH_ADD(false, 1);
 #undef TANH_ADD
   } else {

@@ -230,6 +230,67 @@ __global__ __launch_bounds__(NT) void gated_rmsnorm_kernel(const float* __restri
   }
 }
 
+// The same for rows whose width is a multiple of 4 and at most NT * 4 * VPT, on 16-byte loads: a thread keeps its elements
+// between the sum and the scaling, and all its loads are in flight together.  Which of the two kernels runs is fixed by
+// the width and the alignment of the rows alone.
+template <int NT, int VPT>
+__global__ __launch_bounds__(NT) void gated_rmsnorm_f4_kernel(const float* __restrict__ o, int ldo_in,
+                                                              const float* __restrict__ w, float eps,
+                                                              const void* __restrict__ gate, int gate_dtype, int ldg,
+                                                              void* __restrict__ out, int out_dtype, int ldo, int dim) {
+  __shared__ float red[NT / WAVE];
+  const int r = blockIdx.x, n4 = dim / 4;
+  float4 v[VPT], g[VPT];
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    const int i = threadIdx.x + j * NT;
+    v[j] = i < n4 ? reinterpret_cast<const float4*>(o + (size_t)r * ldo_in)[i] : float4{0.f, 0.f, 0.f, 0.f};
+    g[j] = float4{0.f, 0.f, 0.f, 0.f};
+    if (gate && i < n4) {
+      const size_t at = (size_t)r * ldg + (size_t)i * 4;
+      if (gate_dtype == APC_F32) {
+        g[j] = *reinterpret_cast<const float4*>((const float*)gate + at);
+      } else {
+        const uint2 u = *reinterpret_cast<const uint2*>((const bf16_t*)gate + at);
+        g[j] = float4{__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
+                      __uint_as_float(u.y & 0xffff0000u)};
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    ss = fmaf(v[j].x, v[j].x, ss);
+    ss = fmaf(v[j].y, v[j].y, ss);
+    ss = fmaf(v[j].z, v[j].z, ss);
+    ss = fmaf(v[j].w, v[j].w, ss);
+  }
+  ss = block_sum<NT>(ss, red);
+  const float inv = 1.0f / sqrtf(ss / (float)dim + eps);
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    const int i = threadIdx.x + j * NT;
+    if (i >= n4) continue;
+    const float4 wv = reinterpret_cast<const float4*>(w)[i];
+    float4 y = float4{(v[j].x * inv) * wv.x, (v[j].y * inv) * wv.y, (v[j].z * inv) * wv.z, (v[j].w * inv) * wv.w};
+    if (gate) {
+      y.x *= sigmoid_f(g[j].x);
+      y.y *= sigmoid_f(g[j].y);
+      y.z *= sigmoid_f(g[j].z);
+      y.w *= sigmoid_f(g[j].w);
+    }
+    const size_t at = (size_t)r * ldo + (size_t)i * 4;
+    if (out_dtype == APC_F32) {
+      *reinterpret_cast<float4*>((float*)out + at) = y;
+    } else {
+      uint2 pk;
+      pk.x = pack_bf16x2(y.x, y.y);
+      pk.y = pack_bf16x2(y.z, y.w);
+      *reinterpret_cast<uint2*>((bf16_t*)out + at) = pk;
+    }
+  }
+}
+
 // ---------------------------------------------------------------------------
 // Two softmax maps of a head over the same values, a [T][H][2][dv] float32:
 //   o = a1 - lam * a2;  out = o / sqrt(mean_dv(o^2) + eps) * post * sigmoid(gate[t][h])   (gate: one number a head)
@@ -327,6 +388,20 @@ APC_EXPORT int apc_gated_rmsnorm(const float* o, int ldo_in, const float* w, flo
     if (dim / g > 65535) return APC_ERR_UNSUPPORTED;
     hipLaunchKernelGGL(gated_groupnorm_kernel, dim3(n_rows, dim / g), dim3(64), 0, stream, o, ldo_in, w, eps, gate,
                        gate_dtype, ldg, gate_kind, out, out_dtype, ldo, g);
+    APC_LAUNCH_CHECK();
+    return 0;
+  }
+  auto aligned = [](const void* p, int dtype) { return ((uintptr_t)p & (dtype == APC_F32 ? 15u : 7u)) == 0; };
+  if (dim % 4 == 0 && dim <= 256 * 4 * 8 && ldo_in % 4 == 0 && ldo % 4 == 0 && aligned(o, APC_F32) && aligned(w, APC_F32) &&
+      aligned(out, out_dtype) && (!gate || (ldg % 4 == 0 && aligned(gate, gate_dtype)))) {
+#define GATED_LAUNCH(VPT_)                                                                                               \
+  hipLaunchKernelGGL((gated_rmsnorm_f4_kernel<256, VPT_>), dim3(n_rows), dim3(256), 0, stream, o, ldo_in, w, eps, gate, \
+                     gate_dtype, ldg, out, out_dtype, ldo, dim)
+    if (dim <= 1024) GATED_LAUNCH(1);
+    else if (dim <= 2048) GATED_LAUNCH(2);
+    else if (dim <= 4096) GATED_LAUNCH(4);
+    else GATED_LAUNCH(8);
+#undef GATED_LAUNCH
     APC_LAUNCH_CHECK();
     return 0;
   }
