@@ -20,6 +20,7 @@ _ELEM = {"float32": 4, "bfloat16": 2, "int32": 4}
 class GroupCost:
     page_bytes: int                  # one page over all layers of the group
     window: Optional[int]            # positions after which a request's pages of this group stop growing
+    keep_first: int = 0              # positions at the start that stay beside the window
 
 
 @dataclass(frozen=True)
@@ -37,7 +38,8 @@ class CacheEstimate:
             return cache_elem_bytes if name is None else _ELEM[name]
 
         paged, state = group_needs(needs)
-        groups = [GroupCost(len(entries) * math.prod(n.page_shape(page_tokens)) * elem(n), getattr(n, "window", None))
+        groups = [GroupCost(len(entries) * math.prod(n.page_shape(page_tokens)) * elem(n), getattr(n, "window", None),
+                            int(getattr(n, "keep_first", 0) or 0))
                   for n, entries in paged]
         slot = sum(len(entries) * math.prod(n.slot_shape()) * elem(n) for n, entries in state)
         return CacheEstimate(page_tokens, groups, slot)
@@ -51,9 +53,9 @@ class CacheEstimate:
         """Pages one request of `tokens` tokens holds in a group (a window's group stops growing; one page more
         than the window covers, since the window's ends fall inside pages)."""
         P = self.page_tokens
-        w = self.groups[group].window
+        w, keep = self.groups[group].window, -(-self.groups[group].keep_first // P)
         n = -(-tokens // P)
-        return n if w is None else min(n, -(-w // P) + 1)
+        return n if w is None else min(n, keep + -(-w // P) + 1)
 
     def bytes_for(self, tokens: int) -> int:
         """Cache bytes of one request that holds `tokens` tokens (pages are whole), without its state slot."""

@@ -188,8 +188,10 @@ class CacheManager:
             raise ValueError("a page pool needs at least one page")
         self._lib = L = _host()
         windows = [(-1 if getattr(n, "window", None) is None else int(n.window)) for n, _ in paged]
+        keeps = [int(getattr(n, "keep_first", 0) or 0) for n, _ in paged]
         G = len(paged)
         self._c = L.apc_cache_new(page_tokens, G, (ctypes.c_int * max(G, 1))(*windows),
+                                  (ctypes.c_int * max(G, 1))(*keeps),
                                   (ctypes.c_int * max(G, 1))(*[int(n) for n in num_pages]), max_requests)
         if not self._c:
             raise ValueError("the cache manager could not be set up with these sizes")

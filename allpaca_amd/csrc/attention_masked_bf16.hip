@@ -5,6 +5,9 @@
 //   n positions counted from position 0);  s = (q . k) * scale;  weights exp(s) / (sink + sum exp(s)), sink = 1 (a key
 //   of score 0 without a value) or 0;  query head h reads kv head h / (H / G).
 //
+// `keep` n with a window: the row sees the keys at positions below n as well, the first of the sequence, as tiles (or
+// passes) ahead of the window's.
+//
 // `key_parts` = M > 1: a cached key of dk elements is M keys of dk / M side by side, one for each of M softmax maps over
 // the same values; q holds H heads of dk / M, head j uses part j % M of the keys (M consecutive heads are the maps of
 // one head).  The kernels keep the whole key as the summed axis and give a head's query zeros outside its own part, so
@@ -47,13 +50,13 @@ __device__ __forceinline__ float row4_sum(float v) {
   v += __shfl_xor(v, 16, WAVE);
   return v + __shfl_xor(v, 32, WAVE);
 }
-// all but the positions lo <= p < hi of a value operand's 8 are cleared (what lies there may be anything, and
-// 0 x NaN is NaN)
-__device__ __forceinline__ void keep_positions(Frag& v, int lo, int hi) {
+// all but the positions p < kept or lo <= p < hi of a value operand's 8 are cleared (what lies there may be anything,
+// and 0 x NaN is NaN)
+__device__ __forceinline__ void keep_positions(Frag& v, int lo, int hi, int kept) {
 #pragma unroll
   for (int w = 0; w < 4; ++w) {
-    const uint32_t a = (2 * w >= lo && 2 * w < hi) ? 0x0000ffffu : 0u;
-    const uint32_t b = (2 * w + 1 >= lo && 2 * w + 1 < hi) ? 0xffff0000u : 0u;
+    const uint32_t a = ((2 * w >= lo || 2 * w < kept) && 2 * w < hi) ? 0x0000ffffu : 0u;
+    const uint32_t b = ((2 * w + 1 >= lo || 2 * w + 1 < kept) && 2 * w + 1 < hi) ? 0xffff0000u : 0u;
     v.w[w] &= a | b;
   }
 }
@@ -92,7 +95,7 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
     const bf16_t* __restrict__ q, int ldq, void* __restrict__ out, int ldo, int H, int G, int dk, int dv,
     const bf16_t* __restrict__ cache, int P, const int* __restrict__ block_table, int max_blocks,
     const int* __restrict__ positions, const int* __restrict__ row_seg, const int* __restrict__ tile_row0,
-    const int* __restrict__ tile_rows, int n_tiles, int mask, int mask_size, int sink, const float* __restrict__ sinks,
+    const int* __restrict__ tile_rows, int n_tiles, int mask, int mask_size, int keep, int sink, const float* __restrict__ sinks,
     const float* __restrict__ gate, int ldg, float scale, int key_parts, int out_f32, float softcap,
     const float* __restrict__ r1, const float* __restrict__ r2) {
   constexpr int KROW = DKP + (DKP % 128 == 0 ? 72 : DKP % 128 == 64 ? 8 : DKP % 128 == 32 ? 40 : 104);
@@ -182,11 +185,12 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
   int page_next = 0;
   auto lookup_tile = [&](int t0) { page_next = bt[min(t0 + grp * 8, last_group) / P]; };
   Frag kreg[KP], vreg[VP];
-  int v_lo = 0, v_hi = 8;
+  int v_lo = 0, v_hi = 8, v_kept = 0;
   auto load_tile = [&](int t0) {
     const int tg = min(t0 + grp * 8, last_group), slot0 = tg % P;
     v_lo = first - tg;
     v_hi = last - tg + 1;
+    v_kept = keep - tg;
     const bf16_t* kp = k_head + (size_t)page_next * page_stride + (size_t)slot0 * dk;
     const bf16_t* vp = v_head + (size_t)page_next * page_stride + slot0;
 #pragma unroll
@@ -201,22 +205,25 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
 #pragma unroll
     for (int j = 0; j < VP; ++j) {
       if (v_on[j]) {
-        if (v_lo > 0 || v_hi < 8) keep_positions(vreg[j], v_lo, v_hi);
+        if (v_lo > 0 || v_hi < 8) keep_positions(vreg[j], v_lo, v_hi, v_kept);
         *reinterpret_cast<Frag*>(Vs + v_ldst[j]) = vreg[j];
       }
     }
   };
 
-  const int t_begin = (first / KT) * KT;
+  // the tiles of the kept first keys, then those from the window's first key on
+  const int t_window = (first / KT) * KT;
+  auto tile_after = [&](int t0) { return t0 + KT >= keep && t0 + KT < t_window ? t_window : t0 + KT; };
+  const int t_begin = keep > 0 ? 0 : t_window;
   lookup_tile(t_begin);
   load_tile(t_begin);
-  lookup_tile(t_begin + KT);
+  lookup_tile(tile_after(t_begin));
   __syncthreads();
   store_tile();
   __syncthreads();
-  for (int t0 = t_begin; t0 <= last; t0 += KT) {
-    load_tile(t0 + KT);
-    lookup_tile(t0 + 2 * KT);
+  for (int t0 = t_begin; t0 <= last; t0 = tile_after(t0)) {
+    load_tile(tile_after(t0));
+    lookup_tile(tile_after(tile_after(t0)));
 
     floatx4 s[KT / 16];
 #pragma unroll
@@ -238,7 +245,7 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
         }
     }
     float mx = -INFINITY;
-    if (t0 >= wave_lo && t0 + KT - 1 <= wave_hi) {
+    if ((t0 >= wave_lo || t0 + KT <= keep) && t0 + KT - 1 <= wave_hi) {
 #pragma unroll
       for (int nt = 0; nt < KT / 16; ++nt)
 #pragma unroll
@@ -249,7 +256,7 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int t = t0 + nt * 16 + lc * 4 + r;
-          const float v = (t >= my_lo && t <= my_pos) ? s[nt][r] : -INFINITY;
+          const float v = ((t >= my_lo || t < keep) && t <= my_pos) ? s[nt][r] : -INFINITY;
           s[nt][r] = v;
           mx = fmaxf(mx, v);
         }
@@ -336,7 +343,7 @@ template <int KS, int ET>  // 32-element steps over a key; tiles of 16 value ele
 __global__ __launch_bounds__(DT) void attn_masked_decode_kernel(
     const bf16_t* __restrict__ q, int ldq, int H, int G, int dk, int dv, const bf16_t* __restrict__ cache, int P,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ positions,
-    const int* __restrict__ row_seg, const int* __restrict__ rows, int mask, int mask_size, float scale, int n_splits,
+    const int* __restrict__ row_seg, const int* __restrict__ rows, int mask, int mask_size, int keep, float scale, int n_splits,
     float* __restrict__ parts, int key_parts, float softcap, const float* __restrict__ r1,
     const float* __restrict__ r2) {
   __shared__ __attribute__((aligned(16))) float sc_all[NW][HGMAX * SROW];
@@ -377,19 +384,21 @@ __global__ __launch_bounds__(DT) void attn_masked_decode_kernel(
 
   // the row's own keys in n_splits ranges of whole passes: a step's rows differ in length, and the launch is made for
   // the longest the step may hold
-  const int row_passes = (pos + 1 - a0 + DT - 1) / DT;
-  const int kps = (row_passes + n_splits - 1) / n_splits * DT;
-  const int lo_t = a0 + split * kps;
-  const int hi_t = min(lo_t + kps, pos + 1);
-  for (int t0 = lo_t + wave * WAVE; t0 < hi_t; t0 += DT) {
-    if (t0 + WAVE <= first) continue;           // (only in front of the row's first key)
+  // (the first kept_passes of a row's passes are those of the kept first keys in front of a0)
+  const int kept_passes = (min(keep, a0) + DT - 1) / DT;
+  const int row_passes = kept_passes + (pos + 1 - a0 + DT - 1) / DT;
+  const int per_split = (row_passes + n_splits - 1) / n_splits;
+  const int pass_end = min((split + 1) * per_split, row_passes);
+  for (int pass = split * per_split; pass < pass_end; ++pass) {
+    const int t0 = (pass < kept_passes ? pass * DT : a0 + (pass - kept_passes) * DT) + wave * WAVE;
+    if (t0 > pos || (t0 + WAVE <= first && t0 >= keep)) continue;           // no key the row sees
     // ---- scores of keys t0 .. t0 + 63: 4 tiles of 16 keys
     {
       Frag kf[4][KS];
 #pragma unroll
       for (int tt = 0; tt < 4; ++tt) {
         const int t = t0 + tt * 16 + li;
-        const bool seen = t >= first && t <= pos;
+        const bool seen = (t >= first || t < keep) && t <= pos;
         const bf16_t* kp = head + (size_t)(seen ? bt[t / P] : 0) * page_stride + (size_t)(t % P) * dk;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
@@ -422,9 +431,9 @@ __global__ __launch_bounds__(DT) void attn_masked_decode_kernel(
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
         const int tp = t0 + kk * 32 + lc * 8;
-        if (e < dv && tp <= pos && tp + 8 > first) {
+        if (e < dv && tp <= pos && (tp + 8 > first || tp < keep)) {
           vf[i][kk] = load_frag_once(head + (size_t)bt[tp / P] * page_stride + (size_t)P * dk + (size_t)e * P + tp % P);
-          if (tp < first || tp + 8 > pos + 1) keep_positions(vf[i][kk], first - tp, pos - tp + 1);
+          if (tp < first || tp + 8 > pos + 1) keep_positions(vf[i][kk], first - tp, pos - tp + 1, keep - tp);
         } else {
           vf[i][kk] = zero_frag();
         }
@@ -433,7 +442,7 @@ __global__ __launch_bounds__(DT) void attn_masked_decode_kernel(
     wave_lds_order();
     // ---- softmax, a key a lane
     const int t = t0 + lane;
-    const bool valid = t >= first && t <= pos;
+    const bool valid = (t >= first || t < keep) && t <= pos;
     for (int j = 0; j < per; ++j) {
       const float s = valid ? sc[j * SROW + lane] : -INFINITY;
       const float m_old = ml[j][0], l_old = ml[j][1];
@@ -531,9 +540,9 @@ __global__ __launch_bounds__(64) void attn_masked_merge_kernel(const float* __re
 bool aligned16(const void* p) { return ((uintptr_t)p & 15u) == 0; }
 
 int check_sizes(const void* q, int ldq, const void* out, int ldo, const void* cache, int H, int G, int dk, int dv, int P,
-                int mask, int mask_size, float scale, int key_parts, int out_f32) {
+                int mask, int mask_size, int keep, float scale, int key_parts, int out_f32) {
   if (H <= 0 || G <= 0 || H % G || dk <= 0 || dv <= 0 || P <= 0 || mask < 0 || mask > 2 || (mask && mask_size <= 0) ||
-      key_parts < 1 || dk % key_parts || (H / G) % key_parts)
+      keep < 0 || (keep && mask != 1) || key_parts < 1 || dk % key_parts || (H / G) % key_parts)
     return APC_ERR_BAD_ARG;
   if (dk % (8 * key_parts) || dv % 4 || dk > DMAX || dv > DMAX || P % 8 || ldq % 8 || ldo % 4 || !aligned16(q) ||
       !aligned16(cache) || ((uintptr_t)out & (out_f32 ? 15u : 7u)) || !(scale > 0.f))
@@ -555,12 +564,13 @@ APC_EXPORT int apc_attention_masked_prefill_bf16(const void* q, int ldq, void* o
                                                  int dv, const void* cache, int page_tokens, const int* block_table,
                                                  int max_blocks, const int* positions, const int* row_seg,
                                                  const int* tile_row0, const int* tile_rows, int n_tiles, int mask,
-                                                 int mask_size, int sink, const float* sinks, const float* gate,
+                                                 int mask_size, int keep, int sink, const float* sinks, const float* gate,
                                                  int ldg, float scale, int key_parts, int out_f32, float softcap,
                                                  const float* r1, const float* r2, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   if ((sinks && !sink) || (gate && ldg < H) || softcap < 0.f || (!r1) != (!r2)) return APC_ERR_BAD_ARG;
-  int e = check_sizes(q, ldq, out, ldo, cache, H, G, dk, dv, page_tokens, mask, mask_size, scale, key_parts, out_f32);
+  int e = check_sizes(q, ldq, out, ldo, cache, H, G, dk, dv, page_tokens, mask, mask_size, keep, scale, key_parts,
+                      out_f32);
   if (e) return e;
   n_tiles *= 2;  // halves
   if (max_blocks <= 0 || (long)n_tiles * H > 0x7fffffffL) return APC_ERR_BAD_ARG;
@@ -568,7 +578,7 @@ APC_EXPORT int apc_attention_masked_prefill_bf16(const void* q, int ldq, void* o
 #define MP_LAUNCH(DK_, DV_)                                                                                         \
   hipLaunchKernelGGL((attn_masked_prefill_kernel<DK_, DV_>), grid, block, 0, stream, (const bf16_t*)q, ldq,          \
                      out, ldo, H, G, dk, dv, (const bf16_t*)cache, page_tokens, block_table, max_blocks,             \
-                     positions, row_seg, tile_row0, tile_rows, n_tiles, mask, mask_size, sink, sinks, gate, ldg,     \
+                     positions, row_seg, tile_row0, tile_rows, n_tiles, mask, mask_size, keep, sink, sinks, gate, ldg,     \
                      scale, key_parts, out_f32, softcap, r1, r2)
 #define MP_VALUES(DK_)                       \
   do {                                       \
@@ -589,14 +599,16 @@ APC_EXPORT int apc_attention_masked_prefill_bf16(const void* q, int ldq, void* o
 APC_EXPORT int apc_attention_masked_decode_bf16(const void* q, int ldq, void* out, int ldo, int n_rows, int H, int G,
                                                 int dk, int dv, const void* cache, int page_tokens,
                                                 const int* block_table, int max_blocks, const int* positions,
-                                                const int* row_seg, const int* rows, int mask, int mask_size, int sink,
+                                                const int* row_seg, const int* rows, int mask, int mask_size,
+                                                int keep, int sink,
                                                 const float* sinks, const float* gate, int ldg, float scale,
                                                 int n_splits, float* parts, int key_parts, int out_f32,
                                                 float softcap, const float* r1, const float* r2,
                                                 hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if ((sinks && !sink) || (gate && ldg < H) || softcap < 0.f || (!r1) != (!r2)) return APC_ERR_BAD_ARG;
-  int e = check_sizes(q, ldq, out, ldo, cache, H, G, dk, dv, page_tokens, mask, mask_size, scale, key_parts, out_f32);
+  int e = check_sizes(q, ldq, out, ldo, cache, H, G, dk, dv, page_tokens, mask, mask_size, keep, scale, key_parts,
+                      out_f32);
   if (e) return e;
   if (!apc_attention_masked_takes(H, G, dk, dv, page_tokens, key_parts)) return APC_ERR_UNSUPPORTED;
   if (n_splits <= 0 || n_splits > WAVE || !parts || max_blocks <= 0 ||
@@ -606,7 +618,7 @@ APC_EXPORT int apc_attention_masked_decode_bf16(const void* q, int ldq, void* ou
 #define MD_LAUNCH(KS_, ET_)                                                                                       \
   hipLaunchKernelGGL((attn_masked_decode_kernel<KS_, ET_>), grid, block, 0, stream, (const bf16_t*)q, ldq, H, G, dk, \
                      dv, (const bf16_t*)cache, page_tokens, block_table, max_blocks, positions, row_seg, rows, mask,  \
-                     mask_size, scale, n_splits, parts, key_parts, softcap, r1, r2)
+                     mask_size, keep, scale, n_splits, parts, key_parts, softcap, r1, r2)
 #define MD_VALUES(KS_)                     \
   do {                                     \
     if (dv <= 64) MD_LAUNCH(KS_, 4);       \

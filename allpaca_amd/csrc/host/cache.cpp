@@ -35,8 +35,9 @@ Pool::Pool(int pages) : n(pages), held((size_t)pages, 0) {
   for (int p = pages - 1; p >= 0; --p) free_.push_back(p);  // page 0 goes out first
 }
 
-Cache::Cache(int page_tokens_, const std::vector<int>& windows_, const std::vector<int>& pages, int max_requests_)
-    : page_tokens(page_tokens_), windows(windows_), slots(max_requests_), max_requests(max_requests_) {
+Cache::Cache(int page_tokens_, const std::vector<int>& windows_, const std::vector<int>& keeps_,
+             const std::vector<int>& pages, int max_requests_)
+    : page_tokens(page_tokens_), windows(windows_), keeps(keeps_), slots(max_requests_), max_requests(max_requests_) {
   for (int n : pages) pools.emplace_back(n);
 }
 
@@ -93,7 +94,7 @@ int Cache::commit(long long id, int n_new) {
   for (size_t g = 0; g < pools.size(); ++g) {
     auto& t = s->tables[g];
     const int passed = std::min(first_needed((int)g, s->length) / page_tokens, (int)t.size());
-    for (int i = 0; i < passed; ++i)
+    for (int i = kept_pages((int)g); i < passed; ++i)
       if (t[i] != APC_PAGE_FREED) {
         const int rc = pools[g].give_back(t[i]);
         if (rc) return rc;
@@ -234,13 +235,13 @@ APC_HOST_EXPORT int apc_pool_drain(void* pool, int* out, int cap) {
   return k;
 }
 
-APC_HOST_EXPORT void* apc_cache_new(int page_tokens, int n_groups, const int* windows, const int* pages,
+APC_HOST_EXPORT void* apc_cache_new(int page_tokens, int n_groups, const int* windows, const int* keeps, const int* pages,
                                     int max_requests) {
   if (page_tokens <= 0 || n_groups < 0 || n_groups > APC_MAX_GROUPS || max_requests <= 0) return nullptr;
   for (int g = 0; g < n_groups; ++g)
-    if (pages[g] <= 0) return nullptr;
-  return new Cache(page_tokens, std::vector<int>(windows, windows + n_groups), std::vector<int>(pages, pages + n_groups),
-                   max_requests);
+    if (pages[g] <= 0 || keeps[g] < 0) return nullptr;
+  return new Cache(page_tokens, std::vector<int>(windows, windows + n_groups), std::vector<int>(keeps, keeps + n_groups),
+                   std::vector<int>(pages, pages + n_groups), max_requests);
 }
 APC_HOST_EXPORT void apc_cache_free(void* c) { delete (Cache*)c; }
 APC_HOST_EXPORT void* apc_cache_pool(void* c, int group) {  // group -1: the state slots

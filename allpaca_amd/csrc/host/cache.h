@@ -46,14 +46,18 @@ struct Seq {
 struct Cache {
   int page_tokens;
   std::vector<int> windows;   // per paged group: -1 none
+  std::vector<int> keeps;     // per paged group: positions at the start that no window passes (0: none)
   std::vector<Pool> pools;
   Pool slots;
   int max_requests;
   std::unordered_map<long long, Seq> seqs;
   long long versions = 0;
   std::string why;
-  Cache(int page_tokens, const std::vector<int>& windows, const std::vector<int>& pages, int max_requests);
+  Cache(int page_tokens, const std::vector<int>& windows, const std::vector<int>& keeps, const std::vector<int>& pages,
+        int max_requests);
   int first_needed(int group, int next_pos) const;
+  // pages at the start of a request that hold a kept position: they stay until the request ends
+  int kept_pages(int group) const { return (keeps[group] + page_tokens - 1) / page_tokens; }
   Seq* find(long long id);
   int admit(long long id);    // the slot, or an error code
   void pages_needed(const Seq& s, int n_new, int* out) const;

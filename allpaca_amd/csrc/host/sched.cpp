@@ -218,7 +218,8 @@ APC_HOST_EXPORT int apc_sched_too_large(void* sp, int prompt, int max_tokens, in
   const int need = (prompt + max_tokens + P - 1) / P;
   for (size_t g = 0; g < C.pools.size(); ++g) {
     int worst = need;
-    if (C.windows[g] >= 0) worst = std::min(need, (C.windows[g] + P - 1) / P + 1 + (S.chunk + P - 1) / P);
+    if (C.windows[g] >= 0)
+      worst = std::min(need, C.kept_pages((int)g) + (C.windows[g] + P - 1) / P + 1 + (S.chunk + P - 1) / P);
     if (worst > C.pools[g].n) {
       if (group) *group = (int)g;
       return worst;

@@ -14,6 +14,23 @@ namespace {
 
 constexpr int TILE = 512;
 
+__device__ __forceinline__ void store4(float* dst, const floatx4& v, int left) {
+  if (left >= 4) *reinterpret_cast<float4*>(dst) = float4{v[0], v[1], v[2], v[3]};
+  else
+    for (int r = 0; r < left; ++r) dst[r] = v[r];
+}
+// times sigmoid of the logits that lie at the outputs' own places
+__device__ __forceinline__ void gate4(floatx4& v, const bf16_t* g, int left) {
+  if (left >= 4) {
+    const uint2 p = *reinterpret_cast<const uint2*>(g);
+    const float z[4] = {__uint_as_float(p.x << 16), __uint_as_float(p.x & 0xffff0000u), __uint_as_float(p.y << 16),
+                        __uint_as_float(p.y & 0xffff0000u)};
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] *= 1.0f / (1.0f + __expf(-z[r]));
+  } else {
+    for (int r = 0; r < left; ++r) v[r] *= 1.0f / (1.0f + __expf(-bf16_to_float(g[r])));
+  }
+}
 __device__ __forceinline__ void store4(bf16_t* dst, const floatx4& v, int left) {
   if (left >= 4) {
     uint2 pk;
@@ -25,9 +42,11 @@ __device__ __forceinline__ void store4(bf16_t* dst, const floatx4& v, int left) 
   }
 }
 
+template <typename Out>
 __global__ __launch_bounds__(256) void heads_gemm_few_kernel(const bf16_t* __restrict__ A, int lda, int a_head,
-                                                             const bf16_t* __restrict__ W, bf16_t* __restrict__ C,
-                                                             int ldc, int c_head, int M, int N, int K) {
+                                                             const bf16_t* __restrict__ W, Out* __restrict__ C,
+                                                             int ldc, int c_head, const bf16_t* __restrict__ gate,
+                                                             int ldg, int M, int N, int K) {
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, li = lane % 16, lc = lane / 16;
   const int h = blockIdx.y, bands = (N + 15) / 16, chunks = (K + 31) / 32;
   const int band = blockIdx.x * 4 + wave;
@@ -48,12 +67,16 @@ __global__ __launch_bounds__(256) void heads_gemm_few_kernel(const bf16_t* __res
     for (int x = 0; x < U; ++x) acc = mfma16(fw[x], fa[x], acc);
   }
   const int n = band * 16 + lc * 4;
-  if (li < M && n < N) store4(C + (size_t)li * ldc + (size_t)h * c_head + n, acc, N - n);
+  if (li >= M || n >= N) return;
+  if (gate) gate4(acc, gate + (size_t)li * ldg + (size_t)h * c_head + n, N - n);
+  store4(C + (size_t)li * ldc + (size_t)h * c_head + n, acc, N - n);
 }
 
+template <typename Out>
 __global__ __launch_bounds__(256) void heads_gemm_kernel(const bf16_t* __restrict__ A, int lda, int a_head,
-                                                         const bf16_t* __restrict__ W, bf16_t* __restrict__ C, int ldc,
-                                                         int c_head, int M, int N, int K) {
+                                                         const bf16_t* __restrict__ W, Out* __restrict__ C, int ldc,
+                                                         int c_head, const bf16_t* __restrict__ gate, int ldg, int M,
+                                                         int N, int K) {
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, li = lane % 16, lc = lane / 16;
   const int h = blockIdx.z, bands = (N + 15) / 16, chunks = (K + 31) / 32;
   const int m0 = blockIdx.y * 128 + (wave / 2) * 64, band0 = (blockIdx.x * 2 + wave % 2) * 4;
@@ -95,11 +118,13 @@ __global__ __launch_bounds__(256) void heads_gemm_kernel(const bf16_t* __restric
   for (int t = 0; t < 4; ++t) {
     const int m = m0 + t * 16 + li;
     if (m >= M) continue;
-    bf16_t* row = C + (size_t)m * ldc + (size_t)h * c_head;
+    Out* row = C + (size_t)m * ldc + (size_t)h * c_head;
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
       const int n = (band0 + b) * 16 + lc * 4;
-      if (n < N) store4(row + n, acc[b][t], N - n);
+      if (n >= N) continue;
+      if (gate) gate4(acc[b][t], gate + (size_t)m * ldg + (size_t)h * c_head + n, N - n);
+      store4(row + n, acc[b][t], N - n);
     }
   }
 }
@@ -142,7 +167,7 @@ __device__ __forceinline__ void rotate8(const bf16_t* src, bf16_t* dst, const fl
 // four rows.
 template <bool WAVE_ROW>
 __global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __restrict__ proj, int ld, int H, int dn,
-                                                               int dr, int c_off, int R, const float* __restrict__ norm_w,
+                                                               int dr, const bf16_t* __restrict__ kv, int ldkv, int c_off, int R, const float* __restrict__ norm_w,
                                                                float eps, const float* __restrict__ cos_sin,
                                                                const int* __restrict__ positions,
                                                                const int* __restrict__ row_seg,
@@ -158,7 +183,7 @@ __global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __r
   int first = WAVE_ROW ? lane : threadIdx.x, step = WAVE_ROW ? WAVE : 256;
   if (c_off >= 0) {
     if (wave == 0) {
-      const bf16_t* src = row + c_off;
+      const bf16_t* src = kv + (size_t)r * ldkv + c_off;
       const int page = block_table[(size_t)row_seg[r] * max_blocks + pos / P];
       bf16_t* dst = pages + ((size_t)page * P + pos % P) * L;
       float ss = 0.f;
@@ -193,24 +218,25 @@ __global__ __launch_bounds__(256) void latent_rows_bf16_kernel(const bf16_t* __r
 
 }  // namespace
 
-APC_EXPORT int apc_latent_rows_bf16_takes(int ld, int dn, int dr, int c_off, int R, int ldq) {
-  return (ld % 8 == 0 && dn % 8 == 0 && dr > 0 && dr % 16 == 0 && dr <= 1024 && R % 8 == 0 && ldq % 8 == 0 &&
+APC_EXPORT int apc_latent_rows_bf16_takes(int ld, int dn, int dr, int ldkv, int c_off, int R, int ldq) {
+  return (ld % 8 == 0 && ldkv % 8 == 0 && dn % 8 == 0 && dr > 0 && dr % 16 == 0 && dr <= 1024 && R % 8 == 0 && ldq % 8 == 0 &&
           (c_off < 0 || c_off % 8 == 0)) ? 1 : 0;
 }
 
-APC_EXPORT int apc_latent_rows_bf16(const void* proj, int ld, int H, int dn, int dr, int c_off, int R,
+APC_EXPORT int apc_latent_rows_bf16(const void* proj, int ld, int H, int dn, int dr, const void* kv, int ldkv, int c_off,
+                                    int R,
                                     const float* norm_w, float eps, const float* cos_sin, const int* positions,
                                     const int* row_seg, const int* block_table, int max_blocks, void* pages, int P,
                                     void* q, int ldq, int n_rows, hipStream_t stream) {
   if (n_rows <= 0) return 0;
-  if (!apc_latent_rows_bf16_takes(ld, dn, dr, c_off, R, ldq)) return APC_ERR_UNSUPPORTED;
+  if (!apc_latent_rows_bf16_takes(ld, dn, dr, ldkv, c_off, R, ldq)) return APC_ERR_UNSUPPORTED;
   if (H <= 0 || dn <= 0 || R <= 0 || P <= 0 || max_blocks <= 0 || ldq < H * (R + dr) || ld < H * (dn + dr) || !cos_sin ||
-      (c_off >= 0 && (ld < c_off + R + dr || !norm_w || !pages)) || ((uintptr_t)proj & 15u) || ((uintptr_t)q & 15u) ||
+      (c_off >= 0 && (!kv || ldkv < c_off + R + dr || !norm_w || !pages)) || ((uintptr_t)kv & 15u) || ((uintptr_t)proj & 15u) || ((uintptr_t)q & 15u) ||
       ((uintptr_t)pages & 15u) || ((uintptr_t)cos_sin & 15u))
     return APC_ERR_BAD_ARG;
 #define ROWS_LAUNCH(WAVE_ROW_, BLOCKS_)                                                                                 \
   hipLaunchKernelGGL((latent_rows_bf16_kernel<WAVE_ROW_>), dim3(BLOCKS_), dim3(256), 0, stream, (const bf16_t*)proj, ld, \
-                     H, dn, dr, c_off, R, norm_w, eps, cos_sin, positions, row_seg, block_table, max_blocks,            \
+                     H, dn, dr, (const bf16_t*)kv, ldkv, c_off, R, norm_w, eps, cos_sin, positions, row_seg, block_table, max_blocks,            \
                      (bf16_t*)pages, P, (bf16_t*)q, ldq, n_rows)
   if (n_rows >= 1024) ROWS_LAUNCH(true, ceil_div(n_rows, 4));
   else ROWS_LAUNCH(false, n_rows);
@@ -219,20 +245,32 @@ APC_EXPORT int apc_latent_rows_bf16(const void* proj, int ld, int H, int dn, int
   return 0;
 }
 
-APC_EXPORT int apc_heads_gemm_bf16(const void* A, int lda, int a_head, const void* W, void* C, int ldc, int c_head, int M,
-                                   int H, int N, int K, hipStream_t stream) {
+// C bfloat16, or float32 with c_f32; gate (bfloat16 logits at the outputs' own places, may be null)
+APC_EXPORT int apc_heads_gemm_bf16(const void* A, int lda, int a_head, const void* W, void* C, int ldc, int c_head,
+                                   int c_f32, const void* gate, int ldg, int M, int H, int N, int K,
+                                   hipStream_t stream) {
   if (M <= 0 || H <= 0 || N <= 0) return 0;
-  if (K <= 0 || a_head < K || c_head < N || lda < (H - 1) * a_head + K || ldc < (H - 1) * c_head + N) return APC_ERR_BAD_ARG;
+  if (K <= 0 || a_head < K || c_head < N || lda < (H - 1) * a_head + K || ldc < (H - 1) * c_head + N ||
+      (gate && ldg < (H - 1) * c_head + N))
+    return APC_ERR_BAD_ARG;
   if (K % 8 || a_head % 8 || lda % 8 || c_head % 4 || ldc % 4 || ((uintptr_t)A & 15u) || ((uintptr_t)W & 15u) ||
-      ((uintptr_t)C & 7u) || H > 65535 || ceil_div(M, 128) > 65535)
+      ((uintptr_t)C & (c_f32 ? 15u : 7u)) || (gate && (ldg % 4 || ((uintptr_t)gate & 7u))) || H > 65535 || ceil_div(M, 128) > 65535)
     return APC_ERR_UNSUPPORTED;
   const int bands = ceil_div(N, 16);
-  if (M <= 16)
-    hipLaunchKernelGGL(heads_gemm_few_kernel, dim3(ceil_div(bands, 4), H), dim3(256), 0, stream, (const bf16_t*)A, lda,
-                       a_head, (const bf16_t*)W, (bf16_t*)C, ldc, c_head, M, N, K);
-  else
-    hipLaunchKernelGGL(heads_gemm_kernel, dim3(ceil_div(bands, 8), ceil_div(M, 128), H), dim3(256), 0, stream,
-                       (const bf16_t*)A, lda, a_head, (const bf16_t*)W, (bf16_t*)C, ldc, c_head, M, N, K);
+#define HEADS_LAUNCH(Out_)                                                                                             \
+  do {                                                                                                                 \
+    if (M <= 16)                                                                                                       \
+      hipLaunchKernelGGL(heads_gemm_few_kernel<Out_>, dim3(ceil_div(bands, 4), H), dim3(256), 0, stream,               \
+                         (const bf16_t*)A, lda, a_head, (const bf16_t*)W, (Out_*)C, ldc, c_head, (const bf16_t*)gate,  \
+                         ldg, M, N, K);                                                                                \
+    else                                                                                                               \
+      hipLaunchKernelGGL(heads_gemm_kernel<Out_>, dim3(ceil_div(bands, 8), ceil_div(M, 128), H), dim3(256), 0, stream, \
+                         (const bf16_t*)A, lda, a_head, (const bf16_t*)W, (Out_*)C, ldc, c_head, (const bf16_t*)gate,  \
+                         ldg, M, N, K);                                                                                \
+  } while (0)
+  if (c_f32) HEADS_LAUNCH(float);
+  else HEADS_LAUNCH(bf16_t);
+#undef HEADS_LAUNCH
   APC_LAUNCH_CHECK();
   return 0;
 }

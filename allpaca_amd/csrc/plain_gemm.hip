@@ -13,8 +13,11 @@ constexpr int TM = 64, TN = 64, TK = 16;
 
 // mode 0: C = acc (C of c_dtype)   mode 1: C += acc (C float32)
 // blockIdx.z: one of several products of the same sizes, whose operands lie these many elements apart.
+// With `gate` (rows of ldg, read at the output's own place): C = acc * sigmoid(gate).
 struct HeadStrides {
   size_t a = 0, w = 0, c = 0;
+  const void* gate = nullptr;
+  int gate_dtype = APC_F32, ldg = 0;
 };
 __global__ __launch_bounds__(256) void gemm_plain_kernel(const void* __restrict__ A, int a_dtype, int lda,
                                                          const void* __restrict__ W, int w_dtype, int ldw,
@@ -70,6 +73,10 @@ __global__ __launch_bounds__(256) void gemm_plain_kernel(const void* __restrict_
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
       const size_t o = blockIdx.z * hs.c + (size_t)m * ldc + n;
+      if (hs.gate) {
+        const float z = load_f(hs.gate, hs.gate_dtype, blockIdx.z * hs.c + (size_t)m * hs.ldg + n);
+        acc[i][j] *= 1.0f / (1.0f + expf(-z));
+      }
       if (mode == 1) ((float*)C)[o] += acc[i][j];
       else store_f(C, c_dtype, o, acc[i][j]);
     }
@@ -89,15 +96,19 @@ APC_EXPORT int apc_gemm_plain(const void* A, int a_dtype, int lda, const void* W
   return 0;
 }
 
-// A matrix of its own for every head: C[m][h * c_head + n] = A[m][h * a_head ..] . W[h][n], W [H][N][K] contiguous.
+// A matrix of its own for every head: C[m][h * c_head + n] = A[m][h * a_head ..] . W[h][n], W [H][N][K] contiguous;
+// times sigmoid(gate[m][h * c_head + n]) with a gate.
 APC_EXPORT int apc_heads_gemm_plain(const void* A, int a_dtype, int lda, int a_head, const void* W, int w_dtype, void* C,
-                                    int c_dtype, int ldc, int c_head, int M, int H, int N, int K, hipStream_t stream) {
+                                    int c_dtype, int ldc, int c_head, const void* gate, int gate_dtype, int ldg, int M, int H,
+                                    int N, int K, hipStream_t stream) {
   if (M <= 0 || H <= 0 || N <= 0) return 0;
-  if (K <= 0 || a_head < K || c_head < N || lda < (H - 1) * a_head + K || ldc < (H - 1) * c_head + N) return APC_ERR_BAD_ARG;
+  if (K <= 0 || a_head < K || c_head < N || lda < (H - 1) * a_head + K || ldc < (H - 1) * c_head + N ||
+      (gate && ldg < (H - 1) * c_head + N))
+    return APC_ERR_BAD_ARG;
   const int gy = ceil_div(M, TM);
   if (gy > 65535 || H > 65535) return APC_ERR_BAD_ARG;
   hipLaunchKernelGGL(gemm_plain_kernel, dim3(ceil_div(N, TN), gy, H), dim3(256), 0, stream, A, a_dtype, lda, W, w_dtype, K,
-                     C, c_dtype, ldc, M, N, K, 0, HeadStrides{(size_t)a_head, (size_t)N * K, (size_t)c_head});
+                     C, c_dtype, ldc, M, N, K, 0, HeadStrides{(size_t)a_head, (size_t)N * K, (size_t)c_head, gate, gate_dtype, ldg});
   APC_LAUNCH_CHECK();
   return 0;
 }

@@ -14,7 +14,7 @@
 namespace {
 
 __global__ __launch_bounds__(256) void latent_rows_kernel(const void* __restrict__ proj, int dtype, int ld, int H, int dn,
-                                                          int dr, int c_off, int R, const float* __restrict__ norm_w,
+                                                          int dr, const void* __restrict__ kv, int ldkv, int c_off, int R, const float* __restrict__ norm_w,
                                                           float eps, const float* __restrict__ cos_sin,
                                                           const int* __restrict__ positions,
                                                           const int* __restrict__ row_seg,
@@ -25,7 +25,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const void* __restrict
   const int r = blockIdx.x, tid = threadIdx.x, half = dr / 2;
   const int pos = positions[r];
   const float* cs = cos_sin + (size_t)pos * dr;
-  const size_t base = (size_t)r * ld;
+  const size_t base = (size_t)r * ld, kv_base = (size_t)r * ldkv + c_off;
   for (int i = tid; i < H * half; i += 256) {
     const int h = i / half, j = i % half;
     const size_t src = base + (size_t)h * (dn + dr) + dn + j, dst = (size_t)r * ldq + (size_t)h * (R + dr) + R + j;
@@ -36,7 +36,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const void* __restrict
   if (!norm_w) return;
   float ss = 0.f;
   for (int i = tid; i < R; i += 256) {
-    const float v = load_f(proj, dtype, base + c_off + i);
+    const float v = load_f(kv, dtype, kv_base + i);
     ss = fmaf(v, v, ss);
   }
   ss = block_sum<256>(ss, red);
@@ -44,9 +44,9 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const void* __restrict
   const int page = block_table[(size_t)row_seg[r] * max_blocks + pos / P];
   const size_t out = ((size_t)page * P + pos % P) * (R + dr);
   for (int i = tid; i < R; i += 256)
-    store_f(pages, page_dtype, out + i, load_f(proj, dtype, base + c_off + i) * inv * norm_w[i]);
+    store_f(pages, page_dtype, out + i, load_f(kv, dtype, kv_base + i) * inv * norm_w[i]);
   for (int j = tid; j < half; j += 256) {
-    const float u = load_f(proj, dtype, base + c_off + R + j), v = load_f(proj, dtype, base + c_off + R + half + j);
+    const float u = load_f(kv, dtype, kv_base + R + j), v = load_f(kv, dtype, kv_base + R + half + j);
     const float c = cs[j], s = cs[half + j];
     store_f(pages, page_dtype, out + R + j, u * c - v * s);
     store_f(pages, page_dtype, out + R + half + j, v * c + u * s);
@@ -203,16 +203,17 @@ __global__ __launch_bounds__(256) void tanh_norm_add_f4_kernel(float* __restrict
 
 }  // namespace
 
-// c_off < 0: the row has queries only (nothing goes into the pages)
-APC_EXPORT int apc_latent_rows(const void* proj, int dtype, int ld, int H, int dn, int dr, int c_off, int R,
-                               const float* norm_w, float eps, const float* cos_sin, const int* positions,
+// kv [rows][ldkv]: the rows of the latents (which may be those of the queries), read from column c_off on; c_off < 0:
+// queries only (nothing goes into the pages)
+APC_EXPORT int apc_latent_rows(const void* proj, int dtype, int ld, int H, int dn, int dr, const void* kv,
+                               int ldkv, int c_off, int R, const float* norm_w, float eps, const float* cos_sin, const int* positions,
                                const int* row_seg, const int* block_table, int max_blocks, void* pages, int page_dtype,
                                int P, void* q, int q_dtype, int ldq, int n_rows, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (H <= 0 || dn <= 0 || dr < 0 || dr % 2 || R <= 0 || P <= 0 || max_blocks <= 0 || ldq < H * (R + dr) ||
-      ld < H * (dn + dr) || (c_off >= 0 && (ld < c_off + R + dr || !norm_w || !pages)) || (dr && !cos_sin))
+      ld < H * (dn + dr) || (c_off >= 0 && (!kv || ldkv < c_off + R + dr || !norm_w || !pages)) || (dr && !cos_sin))
     return APC_ERR_BAD_ARG;
-  hipLaunchKernelGGL(latent_rows_kernel, dim3(n_rows), dim3(256), 0, stream, proj, dtype, ld, H, dn, dr, c_off, R,
+  hipLaunchKernelGGL(latent_rows_kernel, dim3(n_rows), dim3(256), 0, stream, proj, dtype, ld, H, dn, dr, kv, ldkv, c_off, R,
                      c_off >= 0 ? norm_w : nullptr, eps, cos_sin, positions, row_seg, block_table, max_blocks, pages,
                      page_dtype, P, q, q_dtype, ldq);
   APC_LAUNCH_CHECK();

@@ -213,6 +213,7 @@ APC_EXPORT int apc_conv_state(const void* proj, int in_dtype, int ld, const floa
 // 64 anchored at key 0, online softmax in float32.
 //   the row at position pos sees keys t in [first, pos]:
 //     mask 0: first = 0;  mask 1 (window of n): first = max(0, pos - n + 1);  mask 2 (chunks of n): first = pos - pos % n
+//   and, with a window, the keys t < keep: the first ones of the sequence
 //   s_t = (q . K[t]) * scale;  p_t = exp(s_t) / (sink + sum exp(s_t)),  sink = 0, 1 (a key of score 0 without a value)
 //   or exp(sinks[h]) (`sinks`: a learned score per query head, not scaled)
 //   out = sum p_t V[t] (times sigmoid(gate[row][h]) with `gate`: logits [rows][>= H]);  query head h reads key/value
@@ -229,7 +230,7 @@ __global__ __launch_bounds__(64) void masked_attention_plain_kernel(
     const void* __restrict__ q, int q_dtype, int ldq, void* __restrict__ out, int out_dtype, int ldo, int H, int G,
     int dk, int dv, const void* __restrict__ cache, int cache_dtype, int P, const int* __restrict__ block_table,
     int max_blocks, const int* __restrict__ positions, const int* __restrict__ row_seg, int mask, int mask_size,
-    int sink, const float* __restrict__ sinks, const void* __restrict__ gate, int gate_dtype, int ldg, float scale,
+    int keep, int sink, const float* __restrict__ sinks, const void* __restrict__ gate, int gate_dtype, int ldg, float scale,
     int key_parts, float softcap, const float* __restrict__ bias_r1, const float* __restrict__ bias_r2) {
   __shared__ float qs[MAX_PER_LANE * WAVE];
   __shared__ float ps[WAVE];
@@ -252,9 +253,11 @@ __global__ __launch_bounds__(64) void masked_attention_plain_kernel(
   for (int e = 0; e < MAX_PER_LANE; ++e) o[e] = 0.f;
   float m = sink ? (sinks ? sinks[h] : 0.f) : -INFINITY, l = sink ? 1.f : 0.f;
 
-  for (int c = first / WAVE; c <= pos / WAVE; ++c) {
+  // groups in order: those of the kept first keys, then from the window's first key on
+  for (int c = keep > 0 ? 0 : first / WAVE; c <= pos / WAVE;
+       c = (c + 1) * WAVE >= keep && c + 1 < first / WAVE ? first / WAVE : c + 1) {
     const int t = c * WAVE + lane;
-    const bool valid = t >= first && t <= pos;
+    const bool valid = (t >= first || t < keep) && t <= pos;
     float s = -INFINITY;
     if (valid) {
       const size_t kb = (size_t)bt[t / P] * page_elems + head_off + (size_t)(t % P) * dk + part0;
@@ -275,10 +278,10 @@ __global__ __launch_bounds__(64) void masked_attention_plain_kernel(
     ps[lane] = p;
     __syncthreads();
     const int j_end = min(WAVE, pos - c * WAVE + 1);
-    const int j_begin = max(0, first - c * WAVE);
-    for (int j = j_begin; j < j_end; ++j) {
-      const float pj = ps[j];
+    for (int j = 0; j < j_end; ++j) {
       const int tj = c * WAVE + j;
+      if (tj < first && tj >= keep) continue;
+      const float pj = ps[j];
       const size_t vb = (size_t)bt[tj / P] * page_elems + head_off + (size_t)P * dk + (tj % P);
 #pragma unroll
       for (int e = 0; e < MAX_PER_LANE; ++e) {
@@ -299,19 +302,19 @@ __global__ __launch_bounds__(64) void masked_attention_plain_kernel(
 APC_EXPORT int apc_masked_attention_plain(const void* q, int q_dtype, int ldq, void* out, int out_dtype, int ldo,
                                           int n_rows, int H, int G, int dk, int dv, const void* cache, int cache_dtype,
                                           int page_tokens, const int* block_table, int max_blocks,
-                                          const int* positions, const int* row_seg, int mask, int mask_size, int sink,
+                                          const int* positions, const int* row_seg, int mask, int mask_size, int keep, int sink,
                                           const float* sinks, const void* gate, int gate_dtype, int ldg, float scale,
                                           int key_parts, float softcap, const float* bias_r1, const float* bias_r2,
                                           hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || dk <= 0 || dv <= 0 || page_tokens <= 0 || max_blocks <= 0 || mask < 0 || mask > 2 ||
-      (mask != 0 && mask_size <= 0) || key_parts < 1 || dk % key_parts || (H / G) % key_parts || (sinks && !sink) ||
+      (mask != 0 && mask_size <= 0) || keep < 0 || (keep && mask != 1) || key_parts < 1 || dk % key_parts || (H / G) % key_parts || (sinks && !sink) ||
       (gate && ldg < H) || softcap < 0.f || (!bias_r1) != (!bias_r2))
     return APC_ERR_BAD_ARG;
   if (dk > MAX_PER_LANE * WAVE || dv > MAX_PER_LANE * WAVE || H > 65535) return APC_ERR_UNSUPPORTED;
   hipLaunchKernelGGL(masked_attention_plain_kernel, dim3(n_rows, H), dim3(64), 0, stream, q, q_dtype, ldq, out,
                      out_dtype, ldo, H, G, dk, dv, cache, cache_dtype, page_tokens, block_table, max_blocks, positions,
-                     row_seg, mask, mask_size, sink, sinks, gate, gate_dtype, ldg, scale, key_parts, softcap, bias_r1,
+                     row_seg, mask, mask_size, keep, sink, sinks, gate, gate_dtype, ldg, scale, key_parts, softcap, bias_r1,
                      bias_r2);
   APC_LAUNCH_CHECK();
   return 0;

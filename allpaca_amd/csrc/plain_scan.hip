@@ -23,13 +23,13 @@ __device__ __forceinline__ float activate(float z, int kind) {
 
 // ---------------------------------------------------------------------------
 // Short causal convolution over time on every channel, the bias behind it, then an activation:
-//   y[t][c] = act(sum_j w[c][j] * u[t - (n-1) + j][c] + b[c]),  u = x[:, c] of the rows of the same segment
+//   y[t][c] = act(sum_j w[c][j] * u[t - (n-1) + j][c] + b[c]),  u = x[:, c] + in_bias[c] of the rows of the same segment
 // u of the n-1 positions ahead of a segment's first row comes from state[slot][n-1][C] (zero for a new request).
 // The state is moved on by `conv_state_kernel` of the attention's convolution afterwards (it keeps inputs, too).
 // ---------------------------------------------------------------------------
 __global__ void conv_channels_kernel(const void* __restrict__ x, int x_dtype, int ldx, int C,
-                                     const float* __restrict__ w, const float* __restrict__ bias, int taps,
-                                     const float* __restrict__ state, const int* __restrict__ row_seg,
+                                     const float* __restrict__ in_bias, const float* __restrict__ w,
+                                     const float* __restrict__ bias, int taps, const float* __restrict__ state, const int* __restrict__ row_seg,
                                      const int* __restrict__ seg_row0, const int* __restrict__ slots, int act,
                                      void* __restrict__ out, int out_dtype, int ldo) {
   const int r = blockIdx.x;
@@ -38,10 +38,11 @@ __global__ void conv_channels_kernel(const void* __restrict__ x, int x_dtype, in
   const int seg = row_seg[r];
   const int i_in_seg = r - seg_row0[seg];
   const float* st = taps > 1 ? state + (size_t)slots[seg] * (taps - 1) * C : nullptr;
+  const float ib = in_bias ? in_bias[c] : 0.f;
   float acc = 0.f;
   for (int j = 0; j < taps; ++j) {              // oldest first
     const int back = taps - 1 - j;
-    const float u = back <= i_in_seg ? load_f(x, x_dtype, (size_t)(r - back) * ldx + c)
+    const float u = back <= i_in_seg ? load_f(x, x_dtype, (size_t)(r - back) * ldx + c) + ib
                                      : st[(size_t)(taps - 1 - (back - i_in_seg)) * C + c];
     acc = fmaf(w[(size_t)c * taps + j], u, acc);
   }
@@ -55,17 +56,18 @@ __global__ void conv_channels_kernel(const void* __restrict__ x, int x_dtype, in
 // The same sums in the same order as the kernel above.
 template <int TAPS, int ROWS>
 __global__ __launch_bounds__(256) void conv_channels_bf16x8_kernel(
-    const bf16_t* __restrict__ x, int ldx, int n_rows, int C, const float* __restrict__ w,
-    const float* __restrict__ bias, const float* __restrict__ state, const int* __restrict__ row_seg,
+    const bf16_t* __restrict__ x, int ldx, int n_rows, int C, const float* __restrict__ in_bias,
+    const float* __restrict__ w, const float* __restrict__ bias, const float* __restrict__ state, const int* __restrict__ row_seg,
     const int* __restrict__ seg_row0, const int* __restrict__ slots, int act, bf16_t* __restrict__ out, int ldo) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
   if (c >= C) return;
-  float wt[8][TAPS], b[8];
+  float wt[8][TAPS], b[8], ib[8];
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) wt[e][j] = w[(size_t)(c + e) * TAPS + j];
     b[e] = bias ? bias[c + e] : 0.f;
+    ib[e] = in_bias ? in_bias[c + e] : 0.f;
   }
   float u[TAPS][8];                               // the inputs of the row and of its TAPS - 1 predecessors, oldest first
   int seg_before = -1;
@@ -81,8 +83,8 @@ __global__ __launch_bounds__(256) void conv_channels_bf16x8_kernel(
         const uint32_t p[4] = {v.x, v.y, v.z, v.w};
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
-          u[j][2 * k] = __uint_as_float(p[k] << 16);
-          u[j][2 * k + 1] = __uint_as_float(p[k] & 0xffff0000u);
+          u[j][2 * k] = __uint_as_float(p[k] << 16) + ib[2 * k];
+          u[j][2 * k + 1] = __uint_as_float(p[k] & 0xffff0000u) + ib[2 * k + 1];
         }
       } else {
         const float* sp = state + ((size_t)slots[seg] * (TAPS - 1) + (TAPS - 1 - (back - i_in_seg))) * C + c;
@@ -217,8 +219,8 @@ __global__ void weighted_pair_kernel(float* __restrict__ x, int ldx, const float
 
 }  // namespace
 
-APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows, int C, const float* w,
-                                 const float* bias, int taps, const float* state, const int* row_seg,
+APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows, int C, const float* in_bias,
+                                 const float* w, const float* bias, int taps, const float* state, const int* row_seg,
                                  const int* seg_row0, const int* slots, int act, void* out, int out_dtype, int ldo,
                                  hipStream_t stream) {
   if (n_rows <= 0) return 0;
@@ -233,10 +235,10 @@ APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows
   do {                                                                                                               \
     if (rows_a_block == 8)                                                                                           \
       hipLaunchKernelGGL((conv_channels_bf16x8_kernel<TAPS_, 8>), grid, dim3(256), 0, stream, (const bf16_t*)x, ldx,  \
-                         n_rows, C, w, bias, state, row_seg, seg_row0, slots, act, (bf16_t*)out, ldo);               \
+                         n_rows, C, in_bias, w, bias, state, row_seg, seg_row0, slots, act, (bf16_t*)out, ldo);      \
     else                                                                                                             \
       hipLaunchKernelGGL((conv_channels_bf16x8_kernel<TAPS_, 1>), grid, dim3(256), 0, stream, (const bf16_t*)x, ldx,  \
-                         n_rows, C, w, bias, state, row_seg, seg_row0, slots, act, (bf16_t*)out, ldo);               \
+                         n_rows, C, in_bias, w, bias, state, row_seg, seg_row0, slots, act, (bf16_t*)out, ldo);      \
   } while (0)
     if (taps == 1) CC_LAUNCH(1);
     else if (taps == 2) CC_LAUNCH(2);
@@ -246,8 +248,8 @@ APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows
     APC_LAUNCH_CHECK();
     return 0;
   }
-  hipLaunchKernelGGL(conv_channels_kernel, dim3(n_rows, ceil_div(C, 256)), dim3(256), 0, stream, x, x_dtype, ldx, C, w,
-                     bias, taps, state, row_seg, seg_row0, slots, act, out, out_dtype, ldo);
+  hipLaunchKernelGGL(conv_channels_kernel, dim3(n_rows, ceil_div(C, 256)), dim3(256), 0, stream, x, x_dtype, ldx, C,
+                     in_bias, w, bias, taps, state, row_seg, seg_row0, slots, act, out, out_dtype, ldo);
   APC_LAUNCH_CHECK();
   return 0;
 }

@@ -77,7 +77,7 @@ _lib.SIGNATURES["host"].update({
     "apc_pool_new": [I], "apc_pool_free": [P], "apc_pool_alloc": [P], "apc_pool_give_back": [P, I],
     "apc_pool_free_count": [P], "apc_pool_pages": [P], "apc_pool_allocations": [P],
     "apc_pool_held": [P, POINTER(c_int), I], "apc_pool_log_frees": [P, I], "apc_pool_drain": [P, POINTER(c_int), I],
-    "apc_cache_new": [I, I, POINTER(c_int), POINTER(c_int), I], "apc_cache_free": [P], "apc_cache_pool": [P, I],
+    "apc_cache_new": [I, I, POINTER(c_int), POINTER(c_int), POINTER(c_int), I], "apc_cache_free": [P], "apc_cache_pool": [P, I],
     "apc_cache_admit": [P, c_longlong], "apc_cache_release": [P, c_longlong],
     "apc_cache_reserve": [P, c_longlong, I], "apc_cache_commit": [P, c_longlong, I],
     "apc_cache_truncate": [P, c_longlong, I], "apc_cache_length": [P, c_longlong], "apc_cache_slot": [P, c_longlong],

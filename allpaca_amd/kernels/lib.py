@@ -36,7 +36,7 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_paged_attention_plain": [P, I, I, I, P, I, I, I, I, I, I, P, I, I, P, I, P, P, I, F, P],
         "apc_conv_heads": [P, I, I, I, I, I, I, I, I, I, I, I, P, P, I, P, I, P, P, P, P, P, I, F, I, P, P, I, F, I, P, I, I, P, I, P, I, I, P],
         "apc_conv_state": [P, I, I, P, I, P, I, I, P, P, P, P],
-        "apc_masked_attention_plain": [P, I, I, P, I, I, I, I, I, I, I, P, I, I, P, I, P, P, I, I, I, P, P, I, I, F, I, F, P, P, P],
+        "apc_masked_attention_plain": [P, I, I, P, I, I, I, I, I, I, I, P, I, I, P, I, P, P, I, I, I, I, P, P, I, I, F, I, F, P, P, P],
         "apc_rotary_pages": [P, I, I, I, I, I, I, P, I, I, P, I, I, I, I, P, I, I, I, I, I, I, P, I, I, I, I, I, I, P, P, P,
                              P, I, P, I, I, I, P, P, F, P],
         "apc_streams_step": [P, I, I, I, P, I, I, P, P, P, P, F, P, I, I, P, P],
@@ -50,10 +50,10 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_diff_combine": [P, I, F, F, F, P, I, I, P, I, I, I, I, I, P],
         "apc_route_topk": [P, I, P, I, I, I, I, I, I, I, F, P, P, P],
         "apc_routed_glu": [P, I, I, P, I, I, I, I, P, I, P, I, I, I, F, F, P, P],
-        "apc_conv_channels": [P, I, I, I, I, P, P, I, P, P, P, P, I, P, I, I, P],
+        "apc_conv_channels": [P, I, I, I, I, P, P, P, I, P, P, P, P, I, P, I, I, P],
         "apc_selective_scan": [P, I, I, P, I, P, P, P, I, P, P, I, I, P, I, I, I, P, P, P, P, I, I, P],
-        "apc_heads_gemm_plain": [P, I, I, I, P, I, P, I, I, I, I, I, I, I, P],
-        "apc_latent_rows": [P, I, I, I, I, I, I, I, P, F, P, P, P, P, I, P, I, I, P, I, I, I, P],
+        "apc_heads_gemm_plain": [P, I, I, I, P, I, P, I, I, I, P, I, I, I, I, I, I, P],
+        "apc_latent_rows": [P, I, I, I, I, I, P, I, I, I, P, F, P, P, P, P, I, P, I, I, P, I, I, I, P],
         "apc_latent_attention_plain": [P, I, I, P, I, I, I, I, I, I, P, I, I, P, I, P, P, F, P],
         "apc_tanh_norm": [P, I, I, P, F, P, P, P, I, I, I, I, I, P],
         "apc_tanh_norm_add": [P, I, P, I, I, F, P, P, F, P, P, P, I, I, I, I, I, P],
@@ -61,6 +61,8 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_bias_rows": [P, I, P, I, I, P],
         "apc_weighted_pair": [P, I, P, I, F, P, I, F, I, I, P],
         "apc_routed_down": [P, I, P, I, I, I, I, P, P, I, P, I, I, P, I, I, I, P],
+        "apc_delta_rule": [P, I, I, I, I, I, I, I, I, I, P, I, I, I, I, P, P, F, P, I, P, P, P, P, I, P],
+        "apc_gated_recurrence": [P, I, I, P, I, P, I, P, P, I, I, P, F, P, I, I, P, P, P, P, I, I, P],
         "apc_argmax_rows": [P, I, I, I, P, P, P],
         "apc_argmax_rows_no_alloc": [P, I, I, I, P, P],
         "apc_sample_rows": [P, I, I, I, P, P, P, P, P, P, Z, I, P],
@@ -96,14 +98,14 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_selective_scan_bf16": [P, I, P, I, P, P, P, I, P, P, I, P, I, I, I, P, P, P, I, P, P, P, P, P, I, P],
         "apc_linear_rotate_bf16": [P, I, I, I, I, I, I, P, P, F, I, P],
         "apc_linear_attention_bf16": [P, I, I, I, I, I, I, I, I, P, P, I, P, P, P, I, P, P, P, P, I, P],
-        "apc_heads_gemm_bf16": [P, I, I, P, P, I, I, I, I, I, I, P],
-        "apc_latent_rows_bf16_takes": [I, I, I, I, I, I],
-        "apc_latent_rows_bf16": [P, I, I, I, I, I, I, P, F, P, P, P, P, I, P, I, P, I, I, P],
+        "apc_heads_gemm_bf16": [P, I, I, P, P, I, I, I, P, I, I, I, I, I, P],
+        "apc_latent_rows_bf16_takes": [I, I, I, I, I, I, I],
+        "apc_latent_rows_bf16": [P, I, I, I, I, P, I, I, I, P, F, P, P, P, P, I, P, I, P, I, I, P],
         "apc_latent_attention_takes": [I, I, I, I],
         "apc_latent_attention_bf16": [P, P, I, I, I, P, I, P, I, P, P, P, P, I, I, I, P, P, F, P],
         "apc_attention_masked_takes": [I, I, I, I, I, I],
-        "apc_attention_masked_prefill_bf16": [P, I, P, I, I, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, P, P, I, F, I, I, F, P, P, P],
-        "apc_attention_masked_decode_bf16": [P, I, P, I, I, I, I, I, I, P, I, P, I, P, P, P, I, I, I, P, P, I, F, I, P, I, I, F, P, P, P],
+        "apc_attention_masked_prefill_bf16": [P, I, P, I, I, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, P, P, I, F, I, I, F, P, P, P],
+        "apc_attention_masked_decode_bf16": [P, I, P, I, I, I, I, I, I, P, I, P, I, P, P, P, I, I, I, I, P, P, I, F, I, P, I, I, F, P, P, P],
         "apc_rotary_pages_bf16_takes": [I] * 16,
         "apc_rotary_pages_bf16": [P, I, I, I, I, I, P, I, P, I, I, I, P, I, I, I, I, I, I, P, I, I, I, I, I, P, P, P, P, I,
                                   P, I, I, P, P, F, P],

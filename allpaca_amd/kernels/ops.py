@@ -465,11 +465,12 @@ def masked_attention_plain(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_k
                            positions: torch.Tensor, row_seg: torch.Tensor, mask: str, mask_size: int, sink: bool,
                            scale: float, key_parts: int = 1, sinks: Optional[torch.Tensor] = None,
                            gate: Optional[torch.Tensor] = None, softcap: float = 0.0,
-                           distance_bias: Optional[tuple] = None) -> None:
+                           distance_bias: Optional[tuple] = None, keep_first: int = 0) -> None:
     _gpu(q, out, cache, block_table, positions, row_seg, sinks, gate)
     r1, r2 = distance_bias if distance_bias is not None else (None, None)
     _gpu(r1, r2)
     _need(float(softcap) >= 0.0, "attention: the soft cap must not be negative")
+    _need(int(keep_first) >= 0 and (not keep_first or mask == "window"), "attention: kept first tokens go with a window")
     ldq, ldo = _rows(q, "attention q"), _rows(out, "attention out")
     T = q.shape[0]
     _check_key_parts(n_heads, n_kv_heads, key_dim, key_parts)
@@ -483,8 +484,8 @@ def masked_attention_plain(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_k
     _lib.check(L.apc_masked_attention_plain(
         q.data_ptr(), _code(q), ldq, out.data_ptr(), _code(out), ldo, T, n_heads, n_kv_heads, key_dim, value_dim,
         cache.data_ptr(), _code(cache), page_tokens, block_table.data_ptr(), block_table.shape[1],
-        _i32(positions, T, "positions"), _i32(row_seg, T, "row_seg"), MASKS[mask], int(mask_size), 1 if sink else 0,
-        _f32(sinks, n_heads, "sinks"), gate.data_ptr() if gate is not None else 0,
+        _i32(positions, T, "positions"), _i32(row_seg, T, "row_seg"), MASKS[mask], int(mask_size), int(keep_first),
+        1 if sink else 0, _f32(sinks, n_heads, "sinks"), gate.data_ptr() if gate is not None else 0,
         _code(gate) if gate is not None else 0, _rows(gate, "head gate") if gate is not None else 0,
         float(scale), int(key_parts), float(softcap), _f32(r1, n_heads, "distance bias r1"),
         _f32(r2, n_heads, "distance bias r2"), _stream()), "masked_attention_plain")
@@ -506,8 +507,9 @@ def masked_attention(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_kv_head
                      cache: torch.Tensor, page_tokens: int, block_table: torch.Tensor, step, mask: str = "causal",
                      mask_size: int = 0, sink: bool = False, scale: float = 1.0, key_parts: int = 1,
                      sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, softcap: float = 0.0,
-                     distance_bias: Optional[tuple] = None) -> None:
-    """`key_parts` = M > 1: a cached key of `key_dim` elements is M keys of key_dim / M side by side, one for each of M
+                     distance_bias: Optional[tuple] = None, keep_first: int = 0) -> None:
+    """`mask` "causal": a row sees all earlier keys and its own; "window": the last `mask_size` of them, and with
+    `keep_first` n also the sequence's first n; "chunk": those of its own chunk of `mask_size` positions.  `key_parts` = M > 1: a cached key of `key_dim` elements is M keys of key_dim / M side by side, one for each of M
     softmax maps over the same values; q holds `n_heads` heads of key_dim / M, head j uses part j % M (M consecutive
     heads are the maps of one head), and `out` holds n_heads heads of value_dim (float32 or the run's type).
     `sinks` float32 [heads]: the sink's score per head (0 without).  `gate` [rows, >= heads] logits: head h of a row
@@ -517,11 +519,11 @@ def masked_attention(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_kv_head
         from . import tuned
         if tuned.masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache, page_tokens,
                                        block_table, step, mask, mask_size, sink, scale, key_parts, sinks, gate,
-                                       softcap, distance_bias):
+                                       softcap, distance_bias, keep_first):
             return
     masked_attention_plain(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache, page_tokens, block_table,
                            step.positions, step.row_seg, mask, mask_size, sink, scale, key_parts, sinks, gate,
-                           softcap, distance_bias)
+                           softcap, distance_bias, keep_first)
 
 
 def rotary_pages(q: torch.Tensor, q_off: int, n_heads: int, q_dim: int, q_rot0: int, q_out: torch.Tensor,
@@ -845,12 +847,13 @@ ACTIVATIONS = {"none": 0, "silu": 1, "relu2": 2, "gelu_tanh": 3}
 
 def conv_channels(x: torch.Tensor, channels: int, conv_w: torch.Tensor, bias: Optional[torch.Tensor],
                   state: Optional[torch.Tensor], step, slots: Optional[torch.Tensor], activation: str,
-                  out: torch.Tensor) -> None:
-    """A short causal convolution over time on the first `channels` columns of x, the bias behind it, then the
-    activation: out[t][c] = act(sum_j conv_w[c][j] * x[t - (taps - 1) + j][c] + bias[c]) inside a segment; the inputs
+                  out: torch.Tensor, in_bias: Optional[torch.Tensor] = None) -> None:
+    """A short causal convolution over time on the first `channels` columns of x (plus `in_bias`: these sums are the
+    convolution's inputs), the bias behind it, then the activation:
+    out[t][c] = act(sum_j conv_w[c][j] * (x[t - (taps - 1) + j][c] + in_bias[c]) + bias[c]) inside a segment; the inputs
     of the positions ahead of a segment come from `state` float32 [slots + 1, taps - 1, channels], which is moved on to
     the segment's last inputs."""
-    _gpu(x, conv_w, bias, state, slots, out)
+    _gpu(x, conv_w, bias, state, slots, out, in_bias)
     ldx, ldo = _rows(x, "conv input"), _rows(out, "conv out")
     T, C = x.shape[0], int(channels)
     _need(activation in ACTIVATIONS, f"conv_channels: activation {activation!r} is not one of {sorted(ACTIVATIONS)}")
@@ -864,13 +867,14 @@ def conv_channels(x: torch.Tensor, channels: int, conv_w: torch.Tensor, bias: Op
               and state.dtype == torch.float32 and tuple(state.shape[1:]) == (taps - 1, C),
               f"conv_channels: state must be float32 [slots, {taps - 1}, {C}]")
     L = _lib.load("plain")
-    _lib.check(L.apc_conv_channels(x.data_ptr(), _code(x), ldx, T, C, conv_w.data_ptr(), _f32(bias, C, "bias"), taps,
+    ib = _f32(in_bias, C, "input bias")
+    _lib.check(L.apc_conv_channels(x.data_ptr(), _code(x), ldx, T, C, ib, conv_w.data_ptr(), _f32(bias, C, "bias"), taps,
                                    state.data_ptr() if taps > 1 else 0, _i32(step.row_seg, T, "row_seg"),
                                    _i32(step.seg_row0, S, "seg_row0"), _i32(slots, S, "slots") if taps > 1 else 0,
                                    ACTIVATIONS[activation], out.data_ptr(), _code(out), ldo, _stream()),
                "conv_channels")
     if taps > 1:
-        _lib.check(L.apc_conv_state(x.data_ptr(), _code(x), ldx, 0, taps, state.data_ptr(), C, S,
+        _lib.check(L.apc_conv_state(x.data_ptr(), _code(x), ldx, ib, taps, state.data_ptr(), C, S,
                                     _i32(step.seg_row0, S, "seg_row0"), _i32(step.seg_rows, S, "seg_rows"),
                                     _i32(slots, S, "slots"), _stream()), "conv_state")
 
@@ -998,12 +1002,14 @@ def prepare_heads(w: torch.Tensor, run_dtype: torch.dtype, a_head: int, out_head
     return w.contiguous()
 
 
-def heads_linear(a: torch.Tensor, a_head: int, w, out: torch.Tensor, out_head: int) -> None:
+def heads_linear(a: torch.Tensor, a_head: int, w, out: torch.Tensor, out_head: int,
+                 gate: Optional[torch.Tensor] = None) -> None:
     """out[t, h * out_head + n] = sum_k a[t, h * a_head + k] w[h, n, k] for every head h; w [heads, n, k] or its tiled
-    form (`prepare_heads`)."""
+    form (`prepare_heads`).  `gate` (logits of out's shape): times sigmoid(gate[t, h * out_head + n])."""
+    _need(gate is None or (gate.shape == out.shape and gate.is_cuda), "heads_linear: the gate has out's shape")
     if not isinstance(w, torch.Tensor):
         from . import tuned
-        tuned.heads_linear_bf16(a, a_head, w, out, out_head)
+        tuned.heads_linear_bf16(a, a_head, w, out, out_head, gate)
         return
     _gpu(a, w, out)
     lda, ldo = _rows(a, "heads_linear a"), _rows(out, "heads_linear out")
@@ -1013,7 +1019,10 @@ def heads_linear(a: torch.Tensor, a_head: int, w, out: torch.Tensor, out_head: i
           and (H - 1) * out_head + N <= out.shape[1], "heads_linear: head ranges exceed the rows")
     L = _lib.load("plain")
     _lib.check(L.apc_heads_gemm_plain(a.data_ptr(), _code(a), lda, int(a_head), w.data_ptr(), _code(w), out.data_ptr(),
-                                      _code(out), ldo, int(out_head), T, H, N, K, _stream()), "heads_gemm_plain")
+                                      _code(out), ldo, int(out_head), gate.data_ptr() if gate is not None else 0,
+                                      _code(gate) if gate is not None else 0,
+                                      _rows(gate, "gate") if gate is not None else 0, T, H, N, K, _stream()),
+               "heads_gemm_plain")
 
 
 def _latent_pages(pages: torch.Tensor, row: int, page_tokens: int, block_table: torch.Tensor) -> None:
@@ -1025,17 +1034,20 @@ def _latent_pages(pages: torch.Tensor, row: int, page_tokens: int, block_table: 
 
 def latent_rows(proj: torch.Tensor, n_heads: int, head_dim: int, rot_dim: int, c_off: Optional[int], rank: int,
                 norm_w: Optional[torch.Tensor], eps: float, cos_sin: Optional[torch.Tensor], step,
-                block_table: torch.Tensor, pages: torch.Tensor, page_tokens: int, q_out: torch.Tensor) -> None:
+                block_table: torch.Tensor, pages: torch.Tensor, page_tokens: int, q_out: torch.Tensor,
+                kv: Optional[torch.Tensor] = None) -> None:
     """Query head h of a row: proj[:, h * (head_dim + rot_dim) ...], whose last rot_dim elements are rotated by the row's
     position (pairs i, i + rot_dim/2; cos_sin float32 [positions, 2, rot_dim/2]) and go to the end of head h of q_out
-    [rows, heads * (rank + rot_dim)].  With `c_off`: proj[:, c_off : c_off + rank] divided by its root mean square and
-    multiplied with norm_w, and the rot_dim elements behind it, rotated, go into the row's slot of its page
-    [slot][rank + rot_dim]."""
-    _gpu(proj, norm_w, cos_sin, block_table, pages, q_out)
+    [rows, heads * (rank + rot_dim)].  With `c_off`: kv[:, c_off : c_off + rank] (`kv`: rows of their own, absent: proj)
+    divided by its root mean square and multiplied with norm_w, and the rot_dim elements behind it, rotated, go into the
+    row's slot of its page [slot][rank + rot_dim]."""
+    kv = proj if kv is None else kv
+    _gpu(proj, norm_w, cos_sin, block_table, pages, q_out, kv)
     T, H, dn, dr, R = proj.shape[0], int(n_heads), int(head_dim), int(rot_dim), int(rank)
-    ld, ldq = _rows(proj, "projected rows"), _rows(q_out, "latent queries")
+    ld, ldq, ldkv = _rows(proj, "projected rows"), _rows(q_out, "latent queries"), _rows(kv, "latent rows")
     _need(proj.shape[1] >= H * (dn + dr) and q_out.shape == (T, H * (R + dr)), "latent_rows: q heads exceed the row")
-    _need(c_off is None or (norm_w is not None and c_off + R + dr <= proj.shape[1]), "latent_rows: the latent exceeds the row")
+    _need(c_off is None or (norm_w is not None and c_off + R + dr <= kv.shape[1] and kv.shape[0] == T
+                             and kv.dtype == proj.dtype), "latent_rows: the latent exceeds the row")
     _latent_pages(pages, R + dr, page_tokens, block_table)
     if dr:
         _need(dr % 2 == 0 and cos_sin is not None and cos_sin.dtype == torch.float32 and cos_sin.is_contiguous()
@@ -1043,12 +1055,12 @@ def latent_rows(proj: torch.Tensor, n_heads: int, head_dim: int, rot_dim: int, c
               "cos/sin table must be float32 [positions, 2, rot/2]")
     if _tuned_ok(proj, pages, q_out):
         from . import tuned
-        if tuned.latent_rows_bf16(proj, ld, H, dn, dr, -1 if c_off is None else int(c_off), R, norm_w, eps, cos_sin, step,
+        if tuned.latent_rows_bf16(proj, ld, H, dn, dr, kv, ldkv, -1 if c_off is None else int(c_off), R, norm_w, eps, cos_sin, step,
                                   block_table, pages, page_tokens, q_out, ldq):
             return
     L = _lib.load("plain")
     _lib.check(L.apc_latent_rows(
-        proj.data_ptr(), _code(proj), ld, H, dn, dr, -1 if c_off is None else int(c_off), R, _f32(norm_w, R, "norm weight"),
+        proj.data_ptr(), _code(proj), ld, H, dn, dr, kv.data_ptr(), ldkv, -1 if c_off is None else int(c_off), R, _f32(norm_w, R, "norm weight"),
         float(eps), cos_sin.data_ptr() if dr else 0, _i32(step.positions, T, "positions"), _i32(step.row_seg, T, "row_seg"),
         block_table.data_ptr(), block_table.shape[1], pages.data_ptr(), _code(pages), page_tokens, q_out.data_ptr(),
         _code(q_out), ldq, T, _stream()), "latent_rows")
@@ -1081,3 +1093,57 @@ def latent_attention(q: torch.Tensor, out: torch.Tensor, n_heads: int, rank: int
             return
     latent_attention_plain(q, out, n_heads, rank, rot_dim, pages, page_tokens, block_table, step.positions, step.row_seg,
                            scale)
+
+
+# --------------------------------------------------------------------------- gated delta rule, gated linear recurrence
+def delta_rule(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, n_heads: int, n_kv_heads: int, key_dim: int,
+               value_dim: int, ba: torch.Tensor, a_off: int, b_off: int, A: torch.Tensor, dt_bias: torch.Tensor,
+               state: torch.Tensor, step, slots: torch.Tensor, out: torch.Tensor) -> None:
+    """Per head, over the rows of every segment in order, S [key_dim, value_dim] float32 a request:
+      S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  out = S^T q
+    rows[:, q_off ...] and [:, k_off ...] hold `n_kv_heads` heads of key_dim, which are divided by sqrt(sum of squares +
+    1e-6), q also times key_dim^(-1/2); head h uses q/k head h // (n_heads / n_kv_heads); v heads at v_off.
+    beta = sigmoid(ba[:, b_off + h]), g = exp(-A[h] softplus(ba[:, a_off + h] + dt_bias[h])) (A, dt_bias float32 [heads]).
+    state float32 [slots + 1, heads, key_dim, value_dim]; out float32 [rows, heads * value_dim]."""
+    _gpu(rows, ba, A, dt_bias, state, slots, out)
+    ld, ldba, ldo = _rows(rows, "rows"), _rows(ba, "step sizes and decays"), _rows(out, "delta rule out")
+    T = rows.shape[0]
+    H, G, dk, dv = int(n_heads), int(n_kv_heads), int(key_dim), int(value_dim)
+    _need(H % G == 0 and q_off + G * dk <= rows.shape[1] and k_off + G * dk <= rows.shape[1]
+          and v_off + H * dv <= rows.shape[1], "delta rule: head ranges exceed the row")
+    _need(ba.shape[0] == T and a_off + H <= ba.shape[1] and b_off + H <= ba.shape[1], "delta rule: a and b exceed their row")
+    _need(out.dtype == torch.float32 and out.shape == (T, H * dv), "delta rule: out float32 [rows, heads * value_dim]")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, dk, dv),
+          f"delta rule: state must be float32 [slots, {H}, {dk}, {dv}]")
+    S = step.n_segs
+    L = _lib.load("plain")
+    _lib.check(L.apc_delta_rule(rows.data_ptr(), _code(rows), ld, q_off, k_off, v_off, H, G, dk, dv, ba.data_ptr(),
+                                _code(ba), ldba, a_off, b_off, _f32(A, H, "A"), _f32(dt_bias, H, "dt bias"),
+                                float(dk) ** -0.5, state.data_ptr(), S, _i32(step.seg_row0, S, "seg_row0"),
+                                _i32(step.seg_rows, S, "seg_rows"), _i32(slots, S, "slots"), out.data_ptr(), ldo,
+                                _stream()), "delta_rule")
+
+
+def gated_recurrence(u: torch.Tensor, z: torch.Tensor, z_bias: torch.Tensor, blocks: int, rate: torch.Tensor,
+                     y: torch.Tensor, y_bias: Optional[torch.Tensor], state: torch.Tensor, step, slots: torch.Tensor,
+                     out: torch.Tensor, out_scale: float = 1.0) -> None:
+    """Per channel, over the rows of every segment in order, S float32 a request:
+      r = sigmoid(z_r), i = sigmoid(z_i), log a = rate r;  S <- exp(log a) S + sqrt(1 - a^2) i u
+      out = S * gelu(y + y_bias) * out_scale
+    u, y, out [rows, channels] (any element type).  z float32 [rows, 2 channels] (+ z_bias [2 channels]): the channels are
+    `blocks` equal parts of w; part b's r logits stand at columns b * 2w ..., its i logits w further on.  rate, y_bias
+    float32 [channels]; state float32 [slots + 1, channels]."""
+    _gpu(u, z, z_bias, rate, y, y_bias, state, slots, out)
+    T, C = out.shape
+    _need(u.shape == (T, C) and y.shape == (T, C) and z.shape == (T, 2 * C) and z.dtype == torch.float32,
+          "gated recurrence: u and y [rows, channels], z float32 [rows, 2 channels]")
+    _need(int(blocks) > 0 and C % int(blocks) == 0, "gated recurrence: the parts must be equal")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (C,),
+          f"gated recurrence: state must be float32 [slots, {C}]")
+    S = step.n_segs
+    L = _lib.load("plain")
+    _lib.check(L.apc_gated_recurrence(
+        u.data_ptr(), _code(u), _rows(u, "u"), z.data_ptr(), _rows(z, "gate logits"), _f32(z_bias, 2 * C, "gate biases"),
+        int(blocks), _f32(rate, C, "rate"), y.data_ptr(), _code(y), _rows(y, "y"), _f32(y_bias, C, "y bias"),
+        float(out_scale), state.data_ptr(), C, S, _i32(step.seg_row0, S, "seg_row0"), _i32(step.seg_rows, S, "seg_rows"),
+        _i32(slots, S, "slots"), out.data_ptr(), _code(out), _rows(out, "out"), _stream()), "gated_recurrence")

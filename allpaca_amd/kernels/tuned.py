@@ -467,7 +467,7 @@ MASKED_DECODE_SPLITS = 64     # at most: the adding kernel takes 64 parts
 
 def masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache, page_tokens, block_table, step,
                           mask: str, mask_size: int, sink: bool, scale: float, key_parts: int = 1, sinks=None,
-                          gate=None, softcap: float = 0.0, distance_bias=None) -> bool:
+                          gate=None, softcap: float = 0.0, distance_bias=None, keep_first: int = 0) -> bool:
     """Attention with a chunked or sliding mask and an optional sink on the MFMA kernels: segments of several rows on
     the tiled kernel, single rows on the kernel that cuts a row's keys into ranges.  False (nothing done) for sizes
     they do not take; the caller then runs the plain kernel."""
@@ -496,24 +496,27 @@ def masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache
                "block table must be contiguous int32 [segments, blocks]")
     _ops._need(step.positions.numel() >= T and step.row_seg.numel() >= T, "step rows differ from q rows")
     code, stream = _ops.MASKS[mask], _ops._stream()
+    keep = int(keep_first)
+    _ops._need(keep >= 0 and (not keep or mask == "window"), "attention: kept first tokens go with a window")
     if step.n_tiles:
         _lib.check(L.apc_attention_masked_prefill_bf16(
             q.data_ptr(), ldq, out.data_ptr(), ldo, n_heads, n_kv_heads, key_dim, value_dim, cache.data_ptr(),
             page_tokens, block_table.data_ptr(), block_table.shape[1], step.positions.data_ptr(),
             step.row_seg.data_ptr(), step.tile_row0.data_ptr(), step.tile_rows.data_ptr(), step.n_tiles, code,
-            int(mask_size), 1 if sink else 0, sinks_p, gate_p, ldg, float(scale), int(key_parts), 1 if f32 else 0,
-            float(softcap), r1_p, r2_p, stream), "attention_masked_prefill_bf16")
+            int(mask_size), keep, 1 if sink else 0, sinks_p, gate_p, ldg, float(scale), int(key_parts),
+            1 if f32 else 0, float(softcap), r1_p, r2_p, stream), "attention_masked_prefill_bf16")
     if step.n_decode_rows:
         n = step.n_decode_rows
         keys = min(step.max_decode_context, mask_size) if code else step.max_decode_context
-        passes = -(-(keys + 255) // 256)        # a row's first pass starts at a multiple of 256 at or below its first key
+        # a row's first pass starts at a multiple of 256 at or below its first key; kept first keys are passes of their own
+        passes = -(-(keys + 255) // 256) + -(-min(keep, step.max_decode_context) // 256)
         splits = max(1, min(passes, MASKED_DECODE_SPLITS, MASKED_DECODE_BLOCKS // max(1, n * n_kv_heads)))
         parts = torch.empty(n * n_heads * splits * (value_dim + 2), dtype=torch.float32, device=q.device)
         _lib.check(L.apc_attention_masked_decode_bf16(
             q.data_ptr(), ldq, out.data_ptr(), ldo, n, n_heads, n_kv_heads, key_dim, value_dim, cache.data_ptr(),
             page_tokens, block_table.data_ptr(), block_table.shape[1], step.positions.data_ptr(),
             step.row_seg.data_ptr(), step.decode_rows.data_ptr() if step.decode_rows is not None else 0, code,
-            int(mask_size), 1 if sink else 0, sinks_p, gate_p, ldg, float(scale), splits, parts.data_ptr(),
+            int(mask_size), keep, 1 if sink else 0, sinks_p, gate_p, ldg, float(scale), splits, parts.data_ptr(),
             int(key_parts), 1 if f32 else 0, float(softcap), r1_p, r2_p, stream), "attention_masked_decode_bf16")
     return True
 
@@ -706,29 +709,34 @@ def pack_heads(w: torch.Tensor, a_head: int, out_head: int):
     return PackedHeads(torch.stack([pack_mfma(w[h].contiguous()).data for h in range(H)]).contiguous(), H, N, K)
 
 
-def heads_linear_bf16(a: torch.Tensor, a_head: int, w: PackedHeads, out: torch.Tensor, out_head: int) -> None:
+def heads_linear_bf16(a: torch.Tensor, a_head: int, w: PackedHeads, out: torch.Tensor, out_head: int, gate=None) -> None:
     _ops._gpu(a, w.data, out)
     lda, ldo = _ops._rows(a, "heads_linear a"), _ops._rows(out, "heads_linear out")
     T = a.shape[0]
-    _ops._need(a.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and out.shape[0] == T
+    f32 = out.dtype == torch.float32
+    _ops._need(a.dtype == torch.bfloat16 and (f32 or out.dtype == torch.bfloat16) and out.shape[0] == T
                and (w.H - 1) * a_head + w.K <= a.shape[1] and (w.H - 1) * out_head + w.N <= out.shape[1],
                "heads_linear: bfloat16 rows that hold the heads' ranges")
-    _ops._need(lda % 8 == 0 and ldo % 4 == 0 and _aligned(a) and out.data_ptr() % 8 == 0,
+    ldg = _ops._rows(gate, "gate") if gate is not None else 0
+    _ops._need(gate is None or (gate.dtype == torch.bfloat16 and ldg % 4 == 0 and gate.data_ptr() % 8 == 0),
+               "heads_linear_bf16: the gate's logits are bfloat16 rows of a stride that is a multiple of 4")
+    _ops._need(lda % 8 == 0 and ldo % 4 == 0 and _aligned(a) and out.data_ptr() % (16 if f32 else 8) == 0,
                "heads_linear_bf16: rows of a stride that is a multiple of 8 (out: 4), aligned")
     L = _lib.load("tuned")
     _lib.check(L.apc_heads_gemm_bf16(a.data_ptr(), lda, int(a_head), w.data.data_ptr(), out.data_ptr(), ldo, int(out_head),
-                                     T, w.H, w.N, w.K, _ops._stream()), "heads_gemm_bf16")
+                                     1 if f32 else 0, gate.data_ptr() if gate is not None else 0, ldg, T, w.H, w.N, w.K,
+                                     _ops._stream()), "heads_gemm_bf16")
 
 
-def latent_rows_bf16(proj, ld, H, dn, dr, c_off, R, norm_w, eps, cos_sin, step, block_table, pages, page_tokens, q_out,
-                     ldq) -> bool:
+def latent_rows_bf16(proj, ld, H, dn, dr, kv, ldkv, c_off, R, norm_w, eps, cos_sin, step, block_table, pages,
+                     page_tokens, q_out, ldq) -> bool:
     """The same on 16-byte accesses; False (nothing done) for sizes the kernel does not take."""
     L = _lib.load("tuned")
     T = proj.shape[0]
-    if not L.apc_latent_rows_bf16_takes(ld, dn, dr, c_off, R, ldq) or not _aligned(proj, pages, q_out, cos_sin):
+    if not L.apc_latent_rows_bf16_takes(ld, dn, dr, ldkv, c_off, R, ldq) or not _aligned(proj, kv, pages, q_out, cos_sin):
         return False
     _lib.check(L.apc_latent_rows_bf16(
-        proj.data_ptr(), ld, H, dn, dr, c_off, R, _ops._f32(norm_w, R, "norm weight"), float(eps), cos_sin.data_ptr(),
+        proj.data_ptr(), ld, H, dn, dr, kv.data_ptr(), ldkv, c_off, R, _ops._f32(norm_w, R, "norm weight"), float(eps), cos_sin.data_ptr(),
         _ops._i32(step.positions, T, "positions"), _ops._i32(step.row_seg, T, "row_seg"), block_table.data_ptr(),
         block_table.shape[1], pages.data_ptr(), page_tokens, q_out.data_ptr(), ldq, T, _ops._stream()), "latent_rows_bf16")
     return True

@@ -43,6 +43,7 @@ HEADS: Registry = Registry("output head")
 # one tensor of slots).
 #   kind = "pages":  page_shape(page_tokens) -> the shape of one page of one layer; `window` (None: every position is
 #                    kept; n: pages that the last n positions no longer reach are given back during the request);
+#                    `keep_first` (absent: 0): pages that hold one of the first n positions stay beside the window;
 #                    dtype: None (the run's cache element type) or a name ("float32", "bfloat16", "int32")
 #   kind = "slot":   slot_shape() -> the shape of one request's state in one layer, zeroed at admission; dtype as above
 @dataclass(frozen=True)
@@ -61,12 +62,14 @@ class PagedKV:
 
 @dataclass(frozen=True)
 class PagedKeysValues:
-    """Keys of `key_dim` and values of `value_dim` elements a head, of every position (or of the last `window`), in
-    pages of one row per kv head: first the page's keys [slot][key_dim], then its values [value_dim][slot]."""
+    """Keys of `key_dim` and values of `value_dim` elements a head, of every position (or of the last `window`, and with
+    it of the first `keep_first`), in pages of one row per kv head: first the page's keys [slot][key_dim], then its
+    values [value_dim][slot]."""
     kv_heads: int
     key_dim: int
     value_dim: int
     window: Optional[int] = None
+    keep_first: int = 0
     kind = "pages"
     dtype = None
 

@@ -9,7 +9,8 @@
   out = Wo (sum p v)
 Options: `qk_norm` (every q and k head is divided by its root mean square over the head and multiplied with the
 tensors "<q>.norm" / "<k>.norm" [key_dim], shared by all heads, before the rotation; values that are the keys stay as
-projected), `softcap` c (s <- c * tanh(s / c)), `rope_scaling` (a frequency rule of `parts/rope.py`).
+projected), `keep_first` n (with a window: the first n tokens of the sequence stay visible beside it, at their true
+positions), `softcap` c (s <- c * tanh(s / c)), `rope_scaling` (a frequency rule of `parts/rope.py`).
 
 `latent_attention`: queries, keys and values go through low-rank latents.
   a = [Wdq; Wdkv; Wg] h                                   (one product; 32-bit rows)
@@ -45,7 +46,7 @@ class SinkAttention(Mixer):
                  rotary_dim: int = 0, rope_theta: float = 10000.0, mask: str = "causal", mask_size: int = 0,
                  learned_sink: bool = True, values_are_keys: bool = False, names: Optional[Mapping[str, str]] = None,
                  qk_norm: bool = False, norm_eps: float = 1e-6, softcap: float = 0.0,
-                 rope_scaling: Optional[Mapping] = None):
+                 rope_scaling: Optional[Mapping] = None, keep_first: int = 0):
         if num_heads % num_kv_heads:
             raise ValueError(f"attention: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         _check_mask(mask, mask_size)
@@ -57,7 +58,9 @@ class SinkAttention(Mixer):
         if self.rot % 2 or not (0 <= self.rot <= self.dk):
             raise ValueError(f"attention: rotary_dim {rotary_dim} must be even and at most key_dim {key_dim}")
         self.scale, self.theta = float(scale), float(rope_theta)
-        self.mask, self.mask_size = mask, int(mask_size)
+        self.mask, self.mask_size, self.keep_first = mask, int(mask_size), int(keep_first)
+        if self.keep_first < 0 or (self.keep_first and mask != "window"):
+            raise ValueError(f"attention: keep_first {keep_first} goes with a window and must not be negative")
         self.learned_sink, self.values_are_keys = bool(learned_sink), bool(values_are_keys)
         self.qk_norm, self.eps, self.softcap = bool(qk_norm), float(norm_eps), float(softcap)
         if self.softcap < 0:
@@ -82,7 +85,9 @@ class SinkAttention(Mixer):
         return out
 
     def cache_need(self):
-        return PagedKeysValues(self.G, self.dk, self.dv, self.mask_size if self.mask == "window" else None)
+        if self.mask == "window":
+            return PagedKeysValues(self.G, self.dk, self.dv, self.mask_size, self.keep_first)
+        return PagedKeysValues(self.G, self.dk, self.dv)
 
     def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
         self.rt = rt
@@ -114,7 +119,7 @@ class SinkAttention(Mixer):
         attn = torch.empty((T, self.H * self.dv), dtype=dt, device=dev)
         ops.masked_attention(q, attn, self.H, self.G, self.dk, self.dv, pages.kv, pages.page_tokens, pages.block_table,
                              step, self.mask, self.mask_size, self.learned_sink, self.scale, sinks=self.sinks,
-                             softcap=self.softcap)
+                             softcap=self.softcap, keep_first=self.keep_first)
         out = torch.empty((T, self.D), dtype=torch.float32, device=dev)
         ops.linear(attn, self.w_o, out)
         return out
