@@ -97,7 +97,7 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
     const int* __restrict__ positions, const int* __restrict__ row_seg, const int* __restrict__ tile_row0,
     const int* __restrict__ tile_rows, int n_tiles, int mask, int mask_size, int keep, int sink, const float* __restrict__ sinks,
     const float* __restrict__ gate, int ldg, float scale, int key_parts, int out_f32, float softcap,
-    const float* __restrict__ r1, const float* __restrict__ r2) {
+    const float* __restrict__ r1, const float* __restrict__ r2, float out_scale) {
   constexpr int KROW = DKP + (DKP % 128 == 0 ? 72 : DKP % 128 == 64 ? 8 : DKP % 128 == 32 ? 40 : 104);
   __shared__ __attribute__((aligned(16))) bf16_t Ks[KT * KROW];
   __shared__ __attribute__((aligned(16))) bf16_t Vs[DVP * (KT + KPAD)];
@@ -301,7 +301,7 @@ __global__ __launch_bounds__(256) void attn_masked_prefill_kernel(
     __syncthreads();
   }
   if (my_row < nrows) {
-    float inv = 1.0f / l_run;
+    float inv = out_scale / l_run;
     if (gate) inv *= 1.0f / (1.0f + __expf(-gate[(size_t)(row0 + my_row) * ldg + h]));
     const size_t at = (size_t)(row0 + my_row) * ldo + (size_t)h * dv;
     bf16_t* orow = (bf16_t*)out + at;
@@ -502,7 +502,7 @@ __global__ __launch_bounds__(DT) void attn_masked_decode_kernel(
   }
 }
 
-// out[row][head] = sum_s e^(m_s - M) o_s / (sink e^(z - M) + sum_s e^(m_s - M) l_s),  M = max(m_s, z with a sink), z the
+// out[row][head] = out_scale * sum_s e^(m_s - M) o_s / (sink e^(z - M) + sum_s e^(m_s - M) l_s),  M = max(m_s, z with a sink), z the
 // sink's score (0, or sinks[head]); times sigmoid(gate[row][head]) with a gate;
 // at most 64 parts: lane s holds part s's maximum and sum.  The parts' elements are asked for 16 parts at a time, with
 // no condition on the way (a part beyond the last one is read as the last one, with weight 0).
@@ -510,7 +510,8 @@ __global__ __launch_bounds__(64) void attn_masked_merge_kernel(const float* __re
                                                                int dv, const int* __restrict__ rows, int sink,
                                                                const float* __restrict__ sinks,
                                                                const float* __restrict__ gate, int ldg,
-                                                               void* __restrict__ out, int ldo, int out_f32) {
+                                                               void* __restrict__ out, int ldo, int out_f32,
+                                                               float out_scale) {
   const int ri = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int r = rows ? rows[ri] : ri;
   const float* p = parts + ((size_t)ri * H + h) * n_parts * (dv + 2);
@@ -521,7 +522,7 @@ __global__ __launch_bounds__(64) void attn_masked_merge_kernel(const float* __re
   if (sink) M = fmaxf(M, z);
   const float w = m == -INFINITY ? 0.f : __expf(m - M);
   const float L = wave_sum(w * l) + (sink ? __expf(z - M) : 0.f);
-  float inv = 1.0f / L;
+  float inv = out_scale / L;
   if (gate) inv *= 1.0f / (1.0f + __expf(-gate[(size_t)r * ldg + h]));
   for (int e0 = 0; e0 < dv; e0 += WAVE) {
     const int e = min(e0 + lane, dv - 1);
@@ -566,7 +567,8 @@ APC_EXPORT int apc_attention_masked_prefill_bf16(const void* q, int ldq, void* o
                                                  const int* tile_row0, const int* tile_rows, int n_tiles, int mask,
                                                  int mask_size, int keep, int sink, const float* sinks, const float* gate,
                                                  int ldg, float scale, int key_parts, int out_f32, float softcap,
-                                                 const float* r1, const float* r2, hipStream_t stream) {
+                                                 const float* r1, const float* r2, float out_scale,
+                                                 hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   if ((sinks && !sink) || (gate && ldg < H) || softcap < 0.f || (!r1) != (!r2)) return APC_ERR_BAD_ARG;
   int e = check_sizes(q, ldq, out, ldo, cache, H, G, dk, dv, page_tokens, mask, mask_size, keep, scale, key_parts,
@@ -579,7 +581,7 @@ APC_EXPORT int apc_attention_masked_prefill_bf16(const void* q, int ldq, void* o
   hipLaunchKernelGGL((attn_masked_prefill_kernel<DK_, DV_>), grid, block, 0, stream, (const bf16_t*)q, ldq,          \
                      out, ldo, H, G, dk, dv, (const bf16_t*)cache, page_tokens, block_table, max_blocks,             \
                      positions, row_seg, tile_row0, tile_rows, n_tiles, mask, mask_size, keep, sink, sinks, gate, ldg,     \
-                     scale, key_parts, out_f32, softcap, r1, r2)
+                     scale, key_parts, out_f32, softcap, r1, r2, out_scale)
 #define MP_VALUES(DK_)                       \
   do {                                       \
     if (dv <= 64) MP_LAUNCH(DK_, 64);        \
@@ -603,7 +605,7 @@ APC_EXPORT int apc_attention_masked_decode_bf16(const void* q, int ldq, void* ou
                                                 int keep, int sink,
                                                 const float* sinks, const float* gate, int ldg, float scale,
                                                 int n_splits, float* parts, int key_parts, int out_f32,
-                                                float softcap, const float* r1, const float* r2,
+                                                float softcap, const float* r1, const float* r2, float out_scale,
                                                 hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if ((sinks && !sink) || (gate && ldg < H) || softcap < 0.f || (!r1) != (!r2)) return APC_ERR_BAD_ARG;
@@ -632,7 +634,7 @@ APC_EXPORT int apc_attention_masked_decode_bf16(const void* q, int ldq, void* ou
 #undef MD_LAUNCH
   APC_LAUNCH_CHECK();
   hipLaunchKernelGGL(attn_masked_merge_kernel, dim3(n_rows, H), dim3(64), 0, stream, parts, n_splits, H, dv, rows, sink,
-                     sinks, gate, ldg, out, ldo, out_f32);
+                     sinks, gate, ldg, out, ldo, out_f32, out_scale);
   APC_LAUNCH_CHECK();
   return 0;
 }

@@ -216,7 +216,7 @@ APC_EXPORT int apc_conv_state(const void* proj, int in_dtype, int ld, const floa
 //   and, with a window, the keys t < keep: the first ones of the sequence
 //   s_t = (q . K[t]) * scale;  p_t = exp(s_t) / (sink + sum exp(s_t)),  sink = 0, 1 (a key of score 0 without a value)
 //   or exp(sinks[h]) (`sinks`: a learned score per query head, not scaled)
-//   out = sum p_t V[t] (times sigmoid(gate[row][h]) with `gate`: logits [rows][>= H]);  query head h reads key/value
+//   out = out_scale * sum p_t V[t] (times sigmoid(gate[row][h]) with `gate`: logits [rows][>= H]);  query head h reads key/value
 //   head h / (H / G).
 // With `key_parts` = M > 1 a key of dk elements is M keys of dk / M side by side, one for each of M maps over the same
 // values: q holds H heads of dk / M elements, head j computes its scores with part j % M of the keys of kv head
@@ -231,7 +231,8 @@ __global__ __launch_bounds__(64) void masked_attention_plain_kernel(
     int dk, int dv, const void* __restrict__ cache, int cache_dtype, int P, const int* __restrict__ block_table,
     int max_blocks, const int* __restrict__ positions, const int* __restrict__ row_seg, int mask, int mask_size,
     int keep, int sink, const float* __restrict__ sinks, const void* __restrict__ gate, int gate_dtype, int ldg, float scale,
-    int key_parts, float softcap, const float* __restrict__ bias_r1, const float* __restrict__ bias_r2) {
+    int key_parts, float softcap, const float* __restrict__ bias_r1, const float* __restrict__ bias_r2,
+    float out_scale) {
   __shared__ float qs[MAX_PER_LANE * WAVE];
   __shared__ float ps[WAVE];
   const int r = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -290,7 +291,7 @@ __global__ __launch_bounds__(64) void masked_attention_plain_kernel(
       }
     }
   }
-  float inv = 1.0f / l;
+  float inv = out_scale / l;
   if (gate) inv *= 1.0f / (1.0f + expf(-load_f(gate, gate_dtype, (size_t)r * ldg + h)));
 #pragma unroll
   for (int e = 0; e < MAX_PER_LANE; ++e) {
@@ -305,7 +306,7 @@ APC_EXPORT int apc_masked_attention_plain(const void* q, int q_dtype, int ldq, v
                                           const int* positions, const int* row_seg, int mask, int mask_size, int keep, int sink,
                                           const float* sinks, const void* gate, int gate_dtype, int ldg, float scale,
                                           int key_parts, float softcap, const float* bias_r1, const float* bias_r2,
-                                          hipStream_t stream) {
+                                          float out_scale, hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || dk <= 0 || dv <= 0 || page_tokens <= 0 || max_blocks <= 0 || mask < 0 || mask > 2 ||
       (mask != 0 && mask_size <= 0) || keep < 0 || (keep && mask != 1) || key_parts < 1 || dk % key_parts || (H / G) % key_parts || (sinks && !sink) ||
@@ -315,7 +316,7 @@ APC_EXPORT int apc_masked_attention_plain(const void* q, int q_dtype, int ldq, v
   hipLaunchKernelGGL(masked_attention_plain_kernel, dim3(n_rows, H), dim3(64), 0, stream, q, q_dtype, ldq, out,
                      out_dtype, ldo, H, G, dk, dv, cache, cache_dtype, page_tokens, block_table, max_blocks, positions,
                      row_seg, mask, mask_size, keep, sink, sinks, gate, gate_dtype, ldg, scale, key_parts, softcap, bias_r1,
-                     bias_r2);
+                     bias_r2, out_scale);
   APC_LAUNCH_CHECK();
   return 0;
 }

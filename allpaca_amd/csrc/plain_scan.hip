@@ -25,19 +25,20 @@ __device__ __forceinline__ float activate(float z, int kind) {
 // Short causal convolution over time on every channel, the bias behind it, then an activation:
 //   y[t][c] = act(sum_j w[c][j] * u[t - (n-1) + j][c] + b[c]),  u = x[:, c] + in_bias[c] of the rows of the same segment
 // u of the n-1 positions ahead of a segment's first row comes from state[slot][n-1][C] (zero for a new request).
-// The state is moved on by `conv_state_kernel` of the attention's convolution afterwards (it keeps inputs, too).
+// The state is moved on by `conv_state_kernel` of the attention's convolution afterwards (it keeps inputs, too), or, with
+// `fold` (every segment is a single row), by the thread that has read it.
 // ---------------------------------------------------------------------------
 __global__ void conv_channels_kernel(const void* __restrict__ x, int x_dtype, int ldx, int C,
                                      const float* __restrict__ in_bias, const float* __restrict__ w,
-                                     const float* __restrict__ bias, int taps, const float* __restrict__ state, const int* __restrict__ row_seg,
+                                     const float* __restrict__ bias, int taps, float* __restrict__ state, const int* __restrict__ row_seg,
                                      const int* __restrict__ seg_row0, const int* __restrict__ slots, int act,
-                                     void* __restrict__ out, int out_dtype, int ldo) {
+                                     int fold, void* __restrict__ out, int out_dtype, int ldo) {
   const int r = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int seg = row_seg[r];
   const int i_in_seg = r - seg_row0[seg];
-  const float* st = taps > 1 ? state + (size_t)slots[seg] * (taps - 1) * C : nullptr;
+  float* st = taps > 1 ? state + (size_t)slots[seg] * (taps - 1) * C : nullptr;
   const float ib = in_bias ? in_bias[c] : 0.f;
   float acc = 0.f;
   for (int j = 0; j < taps; ++j) {              // oldest first
@@ -45,6 +46,7 @@ __global__ void conv_channels_kernel(const void* __restrict__ x, int x_dtype, in
     const float u = back <= i_in_seg ? load_f(x, x_dtype, (size_t)(r - back) * ldx + c) + ib
                                      : st[(size_t)(taps - 1 - (back - i_in_seg)) * C + c];
     acc = fmaf(w[(size_t)c * taps + j], u, acc);
+    if (fold && j > 0) st[(size_t)(j - 1) * C + c] = u;      // (row j - 1 of the state was read one turn earlier)
   }
   if (bias) acc += bias[c];
   store_f(out, out_dtype, (size_t)r * ldo + c, activate(acc, act));
@@ -57,8 +59,8 @@ __global__ void conv_channels_kernel(const void* __restrict__ x, int x_dtype, in
 template <int TAPS, int ROWS>
 __global__ __launch_bounds__(256) void conv_channels_bf16x8_kernel(
     const bf16_t* __restrict__ x, int ldx, int n_rows, int C, const float* __restrict__ in_bias,
-    const float* __restrict__ w, const float* __restrict__ bias, const float* __restrict__ state, const int* __restrict__ row_seg,
-    const int* __restrict__ seg_row0, const int* __restrict__ slots, int act, bf16_t* __restrict__ out, int ldo) {
+    const float* __restrict__ w, const float* __restrict__ bias, float* __restrict__ state, const int* __restrict__ row_seg,
+    const int* __restrict__ seg_row0, const int* __restrict__ slots, int act, int fold, bf16_t* __restrict__ out, int ldo) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
   if (c >= C) return;
   float wt[8][TAPS], b[8], ib[8];
@@ -104,6 +106,14 @@ __global__ __launch_bounds__(256) void conv_channels_bf16x8_kernel(
       for (int j = 0; j < TAPS; ++j) load_input(j);
     }
     seg_before = seg;
+    if (TAPS > 1 && fold) {
+#pragma unroll
+      for (int j = 1; j < TAPS; ++j) {
+        float* sp = state + ((size_t)slots[seg] * (TAPS - 1) + j - 1) * C + c;
+        *reinterpret_cast<float4*>(sp) = float4{u[j][0], u[j][1], u[j][2], u[j][3]};
+        *reinterpret_cast<float4*>(sp + 4) = float4{u[j][4], u[j][5], u[j][6], u[j][7]};
+      }
+    }
     uint32_t o[4];
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
@@ -220,8 +230,8 @@ __global__ void weighted_pair_kernel(float* __restrict__ x, int ldx, const float
 }  // namespace
 
 APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows, int C, const float* in_bias,
-                                 const float* w, const float* bias, int taps, const float* state, const int* row_seg,
-                                 const int* seg_row0, const int* slots, int act, void* out, int out_dtype, int ldo,
+                                 const float* w, const float* bias, int taps, float* state, const int* row_seg,
+                                 const int* seg_row0, const int* slots, int act, int fold, void* out, int out_dtype, int ldo,
                                  hipStream_t stream) {
   if (n_rows <= 0) return 0;
   if (C <= 0 || ldx < C || ldo < C || taps < 1 || !w || act < 0 || act > 3 || !row_seg || !seg_row0) return APC_ERR_BAD_ARG;
@@ -235,10 +245,10 @@ APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows
   do {                                                                                                               \
     if (rows_a_block == 8)                                                                                           \
       hipLaunchKernelGGL((conv_channels_bf16x8_kernel<TAPS_, 8>), grid, dim3(256), 0, stream, (const bf16_t*)x, ldx,  \
-                         n_rows, C, in_bias, w, bias, state, row_seg, seg_row0, slots, act, (bf16_t*)out, ldo);      \
+                         n_rows, C, in_bias, w, bias, state, row_seg, seg_row0, slots, act, fold, (bf16_t*)out, ldo); \
     else                                                                                                             \
       hipLaunchKernelGGL((conv_channels_bf16x8_kernel<TAPS_, 1>), grid, dim3(256), 0, stream, (const bf16_t*)x, ldx,  \
-                         n_rows, C, in_bias, w, bias, state, row_seg, seg_row0, slots, act, (bf16_t*)out, ldo);      \
+                         n_rows, C, in_bias, w, bias, state, row_seg, seg_row0, slots, act, fold, (bf16_t*)out, ldo); \
   } while (0)
     if (taps == 1) CC_LAUNCH(1);
     else if (taps == 2) CC_LAUNCH(2);
@@ -249,7 +259,7 @@ APC_EXPORT int apc_conv_channels(const void* x, int x_dtype, int ldx, int n_rows
     return 0;
   }
   hipLaunchKernelGGL(conv_channels_kernel, dim3(n_rows, ceil_div(C, 256)), dim3(256), 0, stream, x, x_dtype, ldx, C,
-                     in_bias, w, bias, taps, state, row_seg, seg_row0, slots, act, out, out_dtype, ldo);
+                     in_bias, w, bias, taps, state, row_seg, seg_row0, slots, act, fold, out, out_dtype, ldo);
   APC_LAUNCH_CHECK();
   return 0;
 }

@@ -36,7 +36,7 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_paged_attention_plain": [P, I, I, I, P, I, I, I, I, I, I, P, I, I, P, I, P, P, I, F, P],
         "apc_conv_heads": [P, I, I, I, I, I, I, I, I, I, I, I, P, P, I, P, I, P, P, P, P, P, I, F, I, P, P, I, F, I, P, I, I, P, I, P, I, I, P],
         "apc_conv_state": [P, I, I, P, I, P, I, I, P, P, P, P],
-        "apc_masked_attention_plain": [P, I, I, P, I, I, I, I, I, I, I, P, I, I, P, I, P, P, I, I, I, I, P, P, I, I, F, I, F, P, P, P],
+        "apc_masked_attention_plain": [P, I, I, P, I, I, I, I, I, I, I, P, I, I, P, I, P, P, I, I, I, I, P, P, I, I, F, I, F, P, P, F, P],
         "apc_rotary_pages": [P, I, I, I, I, I, I, P, I, I, P, I, I, I, I, P, I, I, I, I, I, I, P, I, I, I, I, I, I, P, P, P,
                              P, I, P, I, I, I, P, P, F, P],
         "apc_streams_step": [P, I, I, I, P, I, I, P, P, P, P, F, P, I, I, P, P],
@@ -50,7 +50,7 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_diff_combine": [P, I, F, F, F, P, I, I, P, I, I, I, I, I, P],
         "apc_route_topk": [P, I, P, I, I, I, I, I, I, I, F, P, P, P],
         "apc_routed_glu": [P, I, I, P, I, I, I, I, P, I, P, I, I, I, F, F, P, P],
-        "apc_conv_channels": [P, I, I, I, I, P, P, P, I, P, P, P, P, I, P, I, I, P],
+        "apc_conv_channels": [P, I, I, I, I, P, P, P, I, P, P, P, P, I, I, P, I, I, P],
         "apc_selective_scan": [P, I, I, P, I, P, P, P, I, P, P, I, I, P, I, I, I, P, P, P, P, I, I, P],
         "apc_heads_gemm_plain": [P, I, I, I, P, I, P, I, I, I, P, I, I, I, I, I, I, P],
         "apc_latent_rows": [P, I, I, I, I, I, P, I, I, I, P, F, P, P, P, P, I, P, I, I, P, I, I, I, P],
@@ -103,9 +103,15 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_latent_rows_bf16": [P, I, I, I, I, P, I, I, I, P, F, P, P, P, P, I, P, I, P, I, I, P],
         "apc_latent_attention_takes": [I, I, I, I],
         "apc_latent_attention_bf16": [P, P, I, I, I, P, I, P, I, P, P, P, P, I, I, I, P, P, F, P],
+        "apc_delta_rule_bf16_takes": [I, I, I, I, I, I, I],
+        "apc_delta_rule_fact_size": [I],
+        "apc_delta_rule_coef_size": [I],
+        "apc_delta_rule_bf16": [P, I, I, I, I, I, I, I, I, P, I, I, I, P, P, F, P, I, P, P, P, I, P, P, P, P, P, P, I, P],
+        "apc_gated_recurrence_bf16_takes": [I, I, I, I, I, I],
+        "apc_gated_recurrence_bf16": [P, I, P, I, P, I, P, P, I, P, F, P, I, I, P, P, P, I, P, P, P, P, P, I, P],
         "apc_attention_masked_takes": [I, I, I, I, I, I],
-        "apc_attention_masked_prefill_bf16": [P, I, P, I, I, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, P, P, I, F, I, I, F, P, P, P],
-        "apc_attention_masked_decode_bf16": [P, I, P, I, I, I, I, I, I, P, I, P, I, P, P, P, I, I, I, I, P, P, I, F, I, P, I, I, F, P, P, P],
+        "apc_attention_masked_prefill_bf16": [P, I, P, I, I, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, P, P, I, F, I, I, F, P, P, F, P],
+        "apc_attention_masked_decode_bf16": [P, I, P, I, I, I, I, I, I, P, I, P, I, P, P, P, I, I, I, I, P, P, I, F, I, P, I, I, F, P, P, F, P],
         "apc_rotary_pages_bf16_takes": [I] * 16,
         "apc_rotary_pages_bf16": [P, I, I, I, I, I, P, I, P, I, I, I, P, I, I, I, I, I, I, P, I, I, I, I, I, P, P, P, P, I,
                                   P, I, I, P, P, F, P],
@@ -155,7 +161,8 @@ class KernelTimer:
 
 _timer = None
 # entry points that launch nothing (questions about sizes): never timed
-NOT_KERNELS = {"apc_latent_attention_takes", "apc_latent_rows_bf16_takes", "apc_selective_scan_bf16_takes", "apc_attention_masked_takes", "apc_rotary_pages_bf16_takes", "apc_routed_bf16_takes", "apc_routed_max_tiles", "apc_linear_attention_bf16_takes", "apc_conv_heads_bf16_takes", "apc_attention_decode_whole_fits", "apc_attention_decode_last_fits", "apc_attention_prefill_tile_rows",
+NOT_KERNELS = {"apc_delta_rule_bf16_takes", "apc_delta_rule_fact_size", "apc_delta_rule_coef_size",
+               "apc_gated_recurrence_bf16_takes", "apc_latent_attention_takes", "apc_latent_rows_bf16_takes", "apc_selective_scan_bf16_takes", "apc_attention_masked_takes", "apc_rotary_pages_bf16_takes", "apc_routed_bf16_takes", "apc_routed_max_tiles", "apc_linear_attention_bf16_takes", "apc_conv_heads_bf16_takes", "apc_attention_decode_whole_fits", "apc_attention_decode_last_fits", "apc_attention_prefill_tile_rows",
                "apc_attention_prefill_wide_takes",
                "apc_gemm_direct_k_split", "apc_gemm_direct_emit_parts", "apc_sample_rows_scratch_kib"}
 

@@ -465,7 +465,8 @@ def masked_attention_plain(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_k
                            positions: torch.Tensor, row_seg: torch.Tensor, mask: str, mask_size: int, sink: bool,
                            scale: float, key_parts: int = 1, sinks: Optional[torch.Tensor] = None,
                            gate: Optional[torch.Tensor] = None, softcap: float = 0.0,
-                           distance_bias: Optional[tuple] = None, keep_first: int = 0) -> None:
+                           distance_bias: Optional[tuple] = None, keep_first: int = 0,
+                           out_scale: float = 1.0) -> None:
     _gpu(q, out, cache, block_table, positions, row_seg, sinks, gate)
     r1, r2 = distance_bias if distance_bias is not None else (None, None)
     _gpu(r1, r2)
@@ -488,7 +489,7 @@ def masked_attention_plain(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_k
         1 if sink else 0, _f32(sinks, n_heads, "sinks"), gate.data_ptr() if gate is not None else 0,
         _code(gate) if gate is not None else 0, _rows(gate, "head gate") if gate is not None else 0,
         float(scale), int(key_parts), float(softcap), _f32(r1, n_heads, "distance bias r1"),
-        _f32(r2, n_heads, "distance bias r2"), _stream()), "masked_attention_plain")
+        _f32(r2, n_heads, "distance bias r2"), float(out_scale), _stream()), "masked_attention_plain")
 
 
 def _check_sinks_gate(sink: bool, sinks, gate, T: int, n_heads: int) -> None:
@@ -507,23 +508,24 @@ def masked_attention(q: torch.Tensor, out: torch.Tensor, n_heads: int, n_kv_head
                      cache: torch.Tensor, page_tokens: int, block_table: torch.Tensor, step, mask: str = "causal",
                      mask_size: int = 0, sink: bool = False, scale: float = 1.0, key_parts: int = 1,
                      sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, softcap: float = 0.0,
-                     distance_bias: Optional[tuple] = None, keep_first: int = 0) -> None:
+                     distance_bias: Optional[tuple] = None, keep_first: int = 0, out_scale: float = 1.0) -> None:
     """`mask` "causal": a row sees all earlier keys and its own; "window": the last `mask_size` of them, and with
     `keep_first` n also the sequence's first n; "chunk": those of its own chunk of `mask_size` positions.  `key_parts` = M > 1: a cached key of `key_dim` elements is M keys of key_dim / M side by side, one for each of M
     softmax maps over the same values; q holds `n_heads` heads of key_dim / M, head j uses part j % M (M consecutive
     heads are the maps of one head), and `out` holds n_heads heads of value_dim (float32 or the run's type).
     `sinks` float32 [heads]: the sink's score per head (0 without).  `gate` [rows, >= heads] logits: head h of a row
     leaves multiplied by sigmoid(gate[row][h]).  `softcap` c > 0: a score s becomes c * tanh(s / c).  `distance_bias`
-    (r1, r2), float32 [heads] each: the score of a key d positions back is lowered by r1[h] * ln(1 + r2[h] * d)."""
+    (r1, r2), float32 [heads] each: the score of a key d positions back is lowered by r1[h] * ln(1 + r2[h] * d).
+    `out_scale`: a constant that `out` leaves multiplied with."""
     if _tuned_ok(q, cache) and out.dtype in (torch.bfloat16, torch.float32):
         from . import tuned
         if tuned.masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache, page_tokens,
                                        block_table, step, mask, mask_size, sink, scale, key_parts, sinks, gate,
-                                       softcap, distance_bias, keep_first):
+                                       softcap, distance_bias, keep_first, out_scale):
             return
     masked_attention_plain(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache, page_tokens, block_table,
                            step.positions, step.row_seg, mask, mask_size, sink, scale, key_parts, sinks, gate,
-                           softcap, distance_bias, keep_first)
+                           softcap, distance_bias, keep_first, out_scale)
 
 
 def rotary_pages(q: torch.Tensor, q_off: int, n_heads: int, q_dim: int, q_rot0: int, q_out: torch.Tensor,
@@ -868,12 +870,13 @@ def conv_channels(x: torch.Tensor, channels: int, conv_w: torch.Tensor, bias: Op
               f"conv_channels: state must be float32 [slots, {taps - 1}, {C}]")
     L = _lib.load("plain")
     ib = _f32(in_bias, C, "input bias")
+    fold = taps > 1 and bool(getattr(step, "decode_only", False))     # single rows: the state moves on in the same launch
     _lib.check(L.apc_conv_channels(x.data_ptr(), _code(x), ldx, T, C, ib, conv_w.data_ptr(), _f32(bias, C, "bias"), taps,
                                    state.data_ptr() if taps > 1 else 0, _i32(step.row_seg, T, "row_seg"),
                                    _i32(step.seg_row0, S, "seg_row0"), _i32(slots, S, "slots") if taps > 1 else 0,
-                                   ACTIVATIONS[activation], out.data_ptr(), _code(out), ldo, _stream()),
+                                   ACTIVATIONS[activation], 1 if fold else 0, out.data_ptr(), _code(out), ldo, _stream()),
                "conv_channels")
-    if taps > 1:
+    if taps > 1 and not fold:
         _lib.check(L.apc_conv_state(x.data_ptr(), _code(x), ldx, ib, taps, state.data_ptr(), C, S,
                                     _i32(step.seg_row0, S, "seg_row0"), _i32(step.seg_rows, S, "seg_rows"),
                                     _i32(slots, S, "slots"), _stream()), "conv_state")
@@ -1116,6 +1119,11 @@ def delta_rule(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, n_heads: 
     _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, dk, dv),
           f"delta rule: state must be float32 [slots, {H}, {dk}, {dv}]")
     S = step.n_segs
+    if _tuned_ok(rows, ba):
+        from . import tuned
+        if tuned.delta_rule_bf16(rows, ld, q_off, k_off, v_off, H, G, dk, dv, ba, ldba, a_off, b_off, A, dt_bias, state,
+                                 step, slots, out, ldo):
+            return
     L = _lib.load("plain")
     _lib.check(L.apc_delta_rule(rows.data_ptr(), _code(rows), ld, q_off, k_off, v_off, H, G, dk, dv, ba.data_ptr(),
                                 _code(ba), ldba, a_off, b_off, _f32(A, H, "A"), _f32(dt_bias, H, "dt bias"),
@@ -1141,6 +1149,10 @@ def gated_recurrence(u: torch.Tensor, z: torch.Tensor, z_bias: torch.Tensor, blo
     _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (C,),
           f"gated recurrence: state must be float32 [slots, {C}]")
     S = step.n_segs
+    if _tuned_ok(u, y, out):
+        from . import tuned
+        if tuned.gated_recurrence_bf16(u, z, z_bias, int(blocks), rate, y, y_bias, state, step, slots, out, out_scale):
+            return
     L = _lib.load("plain")
     _lib.check(L.apc_gated_recurrence(
         u.data_ptr(), _code(u), _rows(u, "u"), z.data_ptr(), _rows(z, "gate logits"), _f32(z_bias, 2 * C, "gate biases"),

@@ -467,7 +467,8 @@ MASKED_DECODE_SPLITS = 64     # at most: the adding kernel takes 64 parts
 
 def masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache, page_tokens, block_table, step,
                           mask: str, mask_size: int, sink: bool, scale: float, key_parts: int = 1, sinks=None,
-                          gate=None, softcap: float = 0.0, distance_bias=None, keep_first: int = 0) -> bool:
+                          gate=None, softcap: float = 0.0, distance_bias=None, keep_first: int = 0,
+                          out_scale: float = 1.0) -> bool:
     """Attention with a chunked or sliding mask and an optional sink on the MFMA kernels: segments of several rows on
     the tiled kernel, single rows on the kernel that cuts a row's keys into ranges.  False (nothing done) for sizes
     they do not take; the caller then runs the plain kernel."""
@@ -504,7 +505,7 @@ def masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache
             page_tokens, block_table.data_ptr(), block_table.shape[1], step.positions.data_ptr(),
             step.row_seg.data_ptr(), step.tile_row0.data_ptr(), step.tile_rows.data_ptr(), step.n_tiles, code,
             int(mask_size), keep, 1 if sink else 0, sinks_p, gate_p, ldg, float(scale), int(key_parts),
-            1 if f32 else 0, float(softcap), r1_p, r2_p, stream), "attention_masked_prefill_bf16")
+            1 if f32 else 0, float(softcap), r1_p, r2_p, float(out_scale), stream), "attention_masked_prefill_bf16")
     if step.n_decode_rows:
         n = step.n_decode_rows
         keys = min(step.max_decode_context, mask_size) if code else step.max_decode_context
@@ -517,7 +518,8 @@ def masked_attention_bf16(q, out, n_heads, n_kv_heads, key_dim, value_dim, cache
             page_tokens, block_table.data_ptr(), block_table.shape[1], step.positions.data_ptr(),
             step.row_seg.data_ptr(), step.decode_rows.data_ptr() if step.decode_rows is not None else 0, code,
             int(mask_size), keep, 1 if sink else 0, sinks_p, gate_p, ldg, float(scale), splits, parts.data_ptr(),
-            int(key_parts), 1 if f32 else 0, float(softcap), r1_p, r2_p, stream), "attention_masked_decode_bf16")
+            int(key_parts), 1 if f32 else 0, float(softcap), r1_p, r2_p, float(out_scale), stream),
+            "attention_masked_decode_bf16")
     return True
 
 
@@ -579,6 +581,53 @@ def selective_scan_bf16(x, dt, dt_bias, A, bc, D, z, state, step, slots, out) ->
         state.data_ptr(), C, N, S, _ops._i32(step.seg_row0, S, "seg_row0"), _ops._i32(step.seg_rows, S, "seg_rows"),
         _ops._i32(slots, S, "slots"), n_chunks, chunks.data_ptr(), seg_chunks.data_ptr(), ws.data_ptr(),
         sums.data_ptr(), out.data_ptr(), _ops._rows(out, "out"), _ops._stream()), "selective_scan_bf16")
+    return True
+
+
+DELTA_CHUNK_MIN_ROWS = 5     # as above, for the gated delta rule and the gated recurrence
+
+
+def delta_rule_bf16(rows, ld, q_off, k_off, v_off, H, G, dk, dv, ba, ldba, a_off, b_off, A, dt_bias, state, step, slots,
+                    out, ldo) -> bool:
+    """The gated delta rule over prompt portions in chunks of 64 rows on MFMA: every chunk's factors side by side, then a
+    walk over the chunks.  False (nothing done) for sizes the kernels do not take and for steps whose segments are all
+    short (decoded rows): the caller then runs the kernel that walks row by row."""
+    L = _lib.load("tuned")
+    if (step.max_rows < DELTA_CHUNK_MIN_ROWS or not _aligned(rows)
+            or not L.apc_delta_rule_bf16_takes(ld, q_off, k_off, H, G, dk, dv)):
+        return False
+    S = step.n_segs
+    n_chunks, chunks, seg_chunks = _row_chunks(step, rows.device)
+    fact = torch.empty(n_chunks * L.apc_delta_rule_fact_size(H), dtype=torch.bfloat16, device=rows.device)
+    coef = torch.empty(n_chunks * L.apc_delta_rule_coef_size(H), dtype=torch.float32, device=rows.device)
+    kt = torch.empty(n_chunks * G * dk * LINEAR_CHUNK_ROWS, dtype=torch.bfloat16, device=rows.device)
+    _lib.check(L.apc_delta_rule_bf16(
+        rows.data_ptr(), ld, q_off, k_off, v_off, H, G, dk, dv, ba.data_ptr(), ldba, a_off, b_off, _ops._f32(A, H, "A"),
+        _ops._f32(dt_bias, H, "dt bias"), float(dk) ** -0.5, state.data_ptr(), S, _ops._i32(step.seg_row0, S, "seg_row0"),
+        _ops._i32(step.seg_rows, S, "seg_rows"), _ops._i32(slots, S, "slots"), n_chunks, chunks.data_ptr(),
+        seg_chunks.data_ptr(), fact.data_ptr(), coef.data_ptr(), kt.data_ptr(), out.data_ptr(), ldo, _ops._stream()),
+        "delta_rule_bf16")
+    return True
+
+
+def gated_recurrence_bf16(u, z, z_bias, blocks: int, rate, y, y_bias, state, step, slots, out, out_scale: float) -> bool:
+    """The gated linear recurrence over prompt portions, chunks of 64 rows side by side (summaries, a scan over the
+    chunks, the outputs).  False (nothing done) as above."""
+    L = _lib.load("tuned")
+    T, C = out.shape
+    ldu, ldz, ldy, ldo = _ops._rows(u, "u"), _ops._rows(z, "gate logits"), _ops._rows(y, "y"), _ops._rows(out, "out")
+    if (step.max_rows < DELTA_CHUNK_MIN_ROWS or not L.apc_gated_recurrence_bf16_takes(C, blocks, ldu, ldz, ldy, ldo)
+            or any(t.data_ptr() % 4 for t in (u, y, out)) or z.data_ptr() % 8):
+        return False
+    S = step.n_segs
+    n_chunks, chunks, seg_chunks = _row_chunks(step, u.device)
+    ws = torch.empty((2, n_chunks, C), dtype=torch.float32, device=u.device)
+    _lib.check(L.apc_gated_recurrence_bf16(
+        u.data_ptr(), ldu, z.data_ptr(), ldz, _ops._f32(z_bias, 2 * C, "gate biases"), blocks, _ops._f32(rate, C, "rate"),
+        y.data_ptr(), ldy, _ops._f32(y_bias, C, "y bias"), float(out_scale), state.data_ptr(), C, S,
+        _ops._i32(step.seg_row0, S, "seg_row0"), _ops._i32(step.seg_rows, S, "seg_rows"), _ops._i32(slots, S, "slots"),
+        n_chunks, chunks.data_ptr(), seg_chunks.data_ptr(), ws[0].data_ptr(), ws[1].data_ptr(), out.data_ptr(), ldo,
+        _ops._stream()), "gated_recurrence_bf16")
     return True
 
 

@@ -23,7 +23,7 @@ The pages hold every head's key and value, put together when the row is written:
 any other attention with keys and values of different sizes."""
 from __future__ import annotations
 
-from typing import Dict, Mapping, Optional
+from typing import Dict, List, Mapping, Optional
 
 import torch
 
@@ -70,6 +70,7 @@ class SinkAttention(Mixer):
         self.k_off = self.H * self.dk
         self.v_off = self.k_off if self.values_are_keys else self.k_off + self.G * self.dk
         self.width = self.k_off + self.G * self.dk + (0 if self.values_are_keys else self.G * self.dv)
+        self.in_width, self.out_width = self.width, self.H * self.dv
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         n = self.names
@@ -89,37 +90,54 @@ class SinkAttention(Mixer):
             return PagedKeysValues(self.G, self.dk, self.dv, self.mask_size, self.keep_first)
         return PagedKeysValues(self.G, self.dk, self.dv)
 
-    def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
+    # ---- the pieces around `core`: a caller with several mixers side by side may put their matrices together
+    def in_matrices(self, tensors: Mapping[str, torch.Tensor]) -> List[torch.Tensor]:
+        """Matrices [.., hidden] whose outputs one below the other are the `in_width` columns `core` reads: q, k, v."""
+        n = self.names
+        return [tensors[n["q"]], tensors[n["k"]]] + ([] if self.values_are_keys else [tensors[n["v"]]])
+
+    def out_matrix(self, tensors: Mapping[str, torch.Tensor]) -> torch.Tensor:
+        return tensors[self.names["o"]]
+
+    def bind_core(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
         self.rt = rt
         n = self.names
         self.q_norm_w = self.k_norm_w = None
         if self.qk_norm:
             self.q_norm_w = to_device(tensors[n["q"] + n["norm"]], rt, torch.float32)
             self.k_norm_w = to_device(tensors[n["k"] + n["norm"]], rt, torch.float32)
-        mats = [tensors[n["q"]], tensors[n["k"]]] + ([] if self.values_are_keys else [tensors[n["v"]]])
-        dt = mats[0].dtype if all(m.dtype == mats[0].dtype for m in mats) else torch.float32
-        self.w_in = ops.prepare_matrix(torch.cat([to_device(m, rt, dt) for m in mats], dim=0), rt.dtype)
-        self.w_o = ops.prepare_matrix(to_device(tensors[n["o"]], rt), rt.dtype)
         self.sinks = to_device(tensors[n["sink"]], rt, torch.float32) if self.learned_sink else None
         self.cos_sin = rotary_table(self.rot, self.theta, rt, self.rope_scaling) if self.rot else None
 
-    def forward(self, h, step, cache) -> torch.Tensor:
-        """float32 [rows, hidden]: the mixer's output."""
+    def core(self, proj: torch.Tensor, step, cache, out: torch.Tensor, scale: float = 1.0) -> None:
+        """`proj` [rows, in_width] -> `out` [rows, out_width], what Wo multiplies, times `scale`."""
         pages = cache.get("mixer") if isinstance(cache, dict) else cache
         if not pages.writes:
             raise ValueError("an attention with keys and values of its own was given another entry's pages")
-        h = as_normed(h).tensor()
-        T, dev, dt = h.shape[0], h.device, self.rt.dtype
-        proj = torch.empty((T, self.width), dtype=dt, device=dev)
-        ops.linear(h, self.w_in, proj)
         q = proj[:, :self.k_off]                    # rotated where it lies: a head is read whole before it is written
         ops.rotary_pages(proj, 0, self.H, self.dk, 0, q, proj, self.k_off, self.dk, None, 0, 0, False, 0,
                          proj, self.v_off, self.dv, self.G, self.rot, self.cos_sin, step, pages.block_table, pages.kv,
                          pages.page_tokens, q_norm_w=self.q_norm_w, k_norm_w=self.k_norm_w, norm_eps=self.eps)
-        attn = torch.empty((T, self.H * self.dv), dtype=dt, device=dev)
-        ops.masked_attention(q, attn, self.H, self.G, self.dk, self.dv, pages.kv, pages.page_tokens, pages.block_table,
+        ops.masked_attention(q, out, self.H, self.G, self.dk, self.dv, pages.kv, pages.page_tokens, pages.block_table,
                              step, self.mask, self.mask_size, self.learned_sink, self.scale, sinks=self.sinks,
-                             softcap=self.softcap, keep_first=self.keep_first)
+                             softcap=self.softcap, keep_first=self.keep_first, out_scale=scale)
+
+    # ---- the mixer by itself
+    def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime) -> None:
+        self.bind_core(tensors, rt)
+        mats = self.in_matrices(tensors)
+        dt = mats[0].dtype if all(m.dtype == mats[0].dtype for m in mats) else torch.float32
+        self.w_in = ops.prepare_matrix(torch.cat([to_device(m, rt, dt) for m in mats], dim=0), rt.dtype)
+        self.w_o = ops.prepare_matrix(to_device(self.out_matrix(tensors), rt), rt.dtype)
+
+    def forward(self, h, step, cache) -> torch.Tensor:
+        """float32 [rows, hidden]: the mixer's output."""
+        h = as_normed(h).tensor()
+        T, dev, dt = h.shape[0], h.device, self.rt.dtype
+        proj = torch.empty((T, self.width), dtype=dt, device=dev)
+        ops.linear(h, self.w_in, proj)
+        attn = torch.empty((T, self.out_width), dtype=dt, device=dev)
+        self.core(proj, step, cache, attn)
         out = torch.empty((T, self.D), dtype=torch.float32, device=dev)
         ops.linear(attn, self.w_o, out)
         return out
