@@ -108,7 +108,7 @@ SIGNATURES: Dict[str, Dict[str, list]] = {
         "apc_delta_rule_coef_size": [I],
         "apc_delta_rule_bf16": [P, I, I, I, I, I, I, I, I, P, I, I, I, P, P, F, P, I, P, P, P, I, P, P, P, P, P, P, I, P],
         "apc_gated_recurrence_bf16_takes": [I, I, I, I, I, I],
-        "apc_gated_recurrence_bf16": [P, I, P, I, P, I, P, P, I, P, F, P, I, I, P, P, P, I, P, P, P, P, P, I, P],
+        "apc_gated_recurrence_bf16": [P, I, P, I, P, I, P, P, I, P, F, P, I, I, P, P, P, I, P, P, P, P, I, P],
         "apc_attention_masked_takes": [I, I, I, I, I, I],
         "apc_attention_masked_prefill_bf16": [P, I, P, I, I, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, P, P, I, F, I, I, F, P, P, F, P],
         "apc_attention_masked_decode_bf16": [P, I, P, I, I, I, I, I, I, P, I, P, I, P, P, P, I, I, I, I, P, P, I, F, I, P, I, I, F, P, P, F, P],

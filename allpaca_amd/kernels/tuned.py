@@ -621,12 +621,12 @@ def gated_recurrence_bf16(u, z, z_bias, blocks: int, rate, y, y_bias, state, ste
         return False
     S = step.n_segs
     n_chunks, chunks, seg_chunks = _row_chunks(step, u.device)
-    ws = torch.empty((2, n_chunks, C), dtype=torch.float32, device=u.device)
+    ws = torch.empty((10, n_chunks, C), dtype=torch.float32, device=u.device)
     _lib.check(L.apc_gated_recurrence_bf16(
         u.data_ptr(), ldu, z.data_ptr(), ldz, _ops._f32(z_bias, 2 * C, "gate biases"), blocks, _ops._f32(rate, C, "rate"),
         y.data_ptr(), ldy, _ops._f32(y_bias, C, "y bias"), float(out_scale), state.data_ptr(), C, S,
         _ops._i32(step.seg_row0, S, "seg_row0"), _ops._i32(step.seg_rows, S, "seg_rows"), _ops._i32(slots, S, "slots"),
-        n_chunks, chunks.data_ptr(), seg_chunks.data_ptr(), ws[0].data_ptr(), ws[1].data_ptr(), out.data_ptr(), ldo,
+        n_chunks, chunks.data_ptr(), seg_chunks.data_ptr(), ws.data_ptr(), out.data_ptr(), ldo,
         _ops._stream()), "gated_recurrence_bf16")
     return True
 

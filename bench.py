@@ -935,6 +935,144 @@ def muvorax_run(args) -> int:
     return 0
 
 
+# ---- the Natenex design beside the llama, Muvorax and Seredra decoders at equal sizes ------------------------------
+# like kernels: of the llama decoder, of Muvorax (latents, linear attention) and of Seredra (mixers side by side, scan)
+NATENEX_LIKE_KERNELS = {
+    "apc_attention_masked_prefill_bf16": (["apc_attention_prefill_bf16"], [], ["apc_attention_masked_prefill_bf16"]),
+    "apc_attention_masked_decode_bf16": (["apc_attention_decode_bf16"], [], ["apc_attention_masked_decode_bf16"]),
+    "apc_rotary_pages_bf16": (["apc_rope_kv_write_bf16", "apc_rope_kv_write"], [], ["apc_rotary_pages_bf16"]),
+    "apc_latent_attention_bf16": (["apc_attention_prefill_bf16", "apc_attention_decode_bf16"],
+                                  ["apc_latent_attention_bf16"], []),
+    "apc_latent_rows_bf16": (["apc_rope_kv_write_bf16", "apc_rope_kv_write"], ["apc_latent_rows_bf16"], []),
+    "apc_heads_gemm_bf16": (["apc_gemm_bf16", "apc_skinny_gemm_bf16"], ["apc_heads_gemm_bf16"], []),
+    "apc_delta_rule_bf16": (["apc_attention_prefill_bf16"], ["apc_linear_attention_bf16"], []),
+    "apc_delta_rule": (["apc_attention_decode_bf16"], ["apc_linear_attention"], []),
+    "apc_gated_recurrence_bf16": (["apc_attention_prefill_bf16"], ["apc_selective_scan_bf16"], ["apc_selective_scan_bf16"]),
+    "apc_gated_recurrence": (["apc_attention_decode_bf16"], ["apc_selective_scan"], ["apc_selective_scan"]),
+    "apc_conv_channels": (["apc_rope_kv_write_bf16"], ["apc_conv_channels"], ["apc_conv_channels"]),
+    "apc_gated_rmsnorm": ([], ["apc_gated_rmsnorm"], ["apc_gated_rmsnorm"]),
+    "apc_rmsnorm_add": (["apc_rmsnorm_rows"], ["apc_tanh_norm_add"], ["apc_streams_step"]),
+}
+NATENEX_TAPS, NATENEX_BLOCKS, NATENEX_KEEP = 4, 16, 64
+
+
+def natenex_configs(size: str, context: int):
+    """Four layers: mixers side by side (grouped attention over a window of half the context with 64 kept first tokens,
+    half of a head rotated, beside a gated recurrence of the model's width) with the dense feed-forward; an attention
+    over cached latents (H heads of d unrotated and d/2 rotated elements, latents of 12 d for the queries and 4 d for
+    keys and values, an output gate) with the dense feed-forward; a gated delta rule (H heads over H/2 key heads of d)
+    without one; the first layer's weights once more.  The llama, Muvorax and Seredra decoders (see there) with four
+    layers of the same widths."""
+    D, H, G, d, F, V = DESIGN_SIZES[size]
+    left = dict(heads=H, kv_heads=G, dim=d, vdim=d, scale=d ** -0.5, mask=dict(size=context // 2, keep_first=NATENEX_KEEP),
+                rot=dict(base=500000.0, dims=d // 2, scaling=dict(factor=4.0, low=1.0, high=4.0, original=2048)))
+    right = dict(width=D, blocks=NATENEX_BLOCKS, conv=NATENEX_TAPS)
+    par = dict(left=left, right=right, left_scale=0.7, right_scale=0.7)
+    lat = dict(heads=H, dim=d, rot_dim=d // 2, vdim=d, q_rank=12 * d, kv_rank=4 * d, scale=(d + d // 2) ** -0.5,
+               rot=dict(base=500000.0, dims=d // 2))
+    delta = dict(heads=H, kv_heads=H // 2, dim=d, vdim=d, conv=NATENEX_TAPS)
+    dense = dict(kind="dense", ff=F)
+    natenex = dict(architecture="Natenex", vocab=V, width=D, embedding=dict(scale=1.0), norm=dict(eps=1e-6),
+                   max_positions=2 * context + 4096,
+                   layers=[dict(type="parallel", mixer=par, mlp=dense), dict(type="latent_attention", mixer=lat, mlp=dense),
+                           dict(type="delta", mixer=delta, mlp=None),
+                           dict(type="parallel", mixer=par, mlp=dense, weights_of=0)])
+    return {"natenex": natenex, **muvorax_configs(size, context)}
+
+
+def natenex_rooflines(size, batch, context, T, points):
+    """For the kernels the design uses beside plain products and their like kernels: the bytes or the arithmetic of the
+    launches of a step over the measured time, as a share of the GPU's peak (8 TB/s, 2.5 PFLOP/s)."""
+    D, H, G, d, F, V = DESIGN_SIZES[size]
+    R, dr, Q, C, w = 4 * d, d // 2, 12 * d, D, D // NATENEX_BLOCKS
+    window, keep = context // 2, NATENEX_KEEP
+
+    def work(name, rows, keys_sum, prefill):
+        """(bytes, flops) of all of a step's launches of entry point `name` in the Natenex model."""
+        seen = (sum(min(t + 1, window + keep) for t in range(rows)) if prefill
+                else rows * min(context, window + keep))                 # keys of the windows and the kept first tokens
+        if name == "apc_attention_masked_prefill_bf16":
+            return 0, 2 * seen * H * 4 * d
+        if name == "apc_attention_masked_decode_bf16":
+            return 2 * seen * G * 2 * d * 2, 0
+        if name == "apc_rotary_pages_bf16":          # q, k, v read, q and the pages' keys and values written
+            return 2 * rows * ((H + 2 * G) * d * 2) * 2, 0
+        if name == "apc_latent_attention_bf16":
+            return (0, keys_sum * H * 2 * (2 * R + dr)) if prefill else (keys_sum * (R + dr) * 2, keys_sum * H * 2 * (2 * R + dr))
+        if name == "apc_latent_rows_bf16":
+            return rows * (2 * H * dr * 2 + 2 * (R + dr) * 2), 0
+        if name == "apc_heads_gemm_bf16":            # the latents' queries and outputs; the gates of two recurrences
+            gates = 2 * (2 * C * w * 2 + rows * (C * 2 + 2 * C * 4))
+            return 2 * H * d * R * 2 + rows * H * (d + 2 * R + dr + 2 * d) * 2 + gates, 2 * rows * H * 2 * d * R + 2 * rows * 2 * 2 * C * w
+        if name == "apc_delta_rule_bf16":            # a row: products with keys, its chunk's systems, the state both ways
+            return 0, rows * H * (2 * 2 * 32 * d + 2 * 2 * 32 * d + 3 * 2 * d * d)
+        if name == "apc_delta_rule":
+            return rows * H * d * d * 4 * 2, 0
+        if name in ("apc_gated_recurrence", "apc_gated_recurrence_bf16"):     # u, both gates, y read, the output written
+            return 2 * rows * C * (2 + 8 + 2 + 2), 0
+        if name == "apc_conv_channels":              # the recurrences' and the delta rule's channels
+            return rows * (2 * C + 2 * H * d) * (2 + 2), 0
+        if name == "apc_gated_rmsnorm":
+            return rows * H * d * (4 + 2 + 2), 0
+        if name == "apc_rmsnorm_add":                # y and x read, x and the next reader's 16-bit copy written
+            return 7 * rows * D * (4 + 4 + 4 + 2), 0
+        return None
+
+    def muvorax_work(name, rows, keys_sum, prefill):
+        if name == "apc_latent_attention_bf16":
+            return (0, 2 * keys_sum * H * 2 * (2 * R + dr)) if prefill else (2 * keys_sum * (R + dr) * 2, 0)
+        if name == "apc_latent_rows_bf16":
+            return rows * (2 * H * dr * 2 + (R + dr) * 2) * 2, 0
+        if name == "apc_heads_gemm_bf16":
+            return 2 * 2 * H * d * R * 2 + 2 * rows * H * (d + 2 * R + dr + d) * 2, 2 * 2 * rows * H * 2 * d * R
+        if name == "apc_tanh_norm_add":
+            return 8 * rows * D * (4 + 4 + 4 + 2), 0
+        return seredra_work(size, name, rows, keys_sum, prefill)
+
+    table = {}
+    for phase, rows, keys_sum in (("prefill", T, T * (T + 1) // 2), ("decode", batch, batch * context)):
+        for new, (llama, muvorax, seredra) in NATENEX_LIKE_KERNELS.items():
+            row = {}
+            for model, names in (("natenex", [new]), ("llama", llama), ("muvorax", muvorax), ("seredra", seredra)):
+                times = points[model][phase + "_kernels_us"]
+                name = next((n for n in names if n in times), None)
+                if name is None or not times[name]:
+                    continue
+                us, pre = times[name], phase == "prefill"
+                w_ = (work(name, rows, keys_sum, pre) if model == "natenex" else muvorax_work(name, rows, keys_sum, pre)
+                      if model == "muvorax" else seredra_work(size, name, rows, keys_sum, pre))
+                row[model] = {"us": round(us, 1)}
+                if w_:
+                    row[model]["share_of_peak"] = round(max(w_[0] / (us * 1e-6) / (HBM_PEAK_GBS * 1e9),
+                                                            w_[1] / (us * 1e-6) / PEAK_FLOPS["bf16"]), 4)
+            if "natenex" in row:
+                table[f"{phase}: {new}"] = row
+    return table
+
+
+def natenex_run(args) -> int:
+    T, batch, context = 2048, args.batch, args.context
+    out = {"metric": "Natenex beside the llama, Muvorax and Seredra decoders at equal sizes: prefill tok/s (one prompt of "
+                     f"2048 tokens) and decode tok/s (batch {batch}, context {context})", "unit": "tok/s", "n_gpus": 1,
+           "dtype": args.dtype, "data": "synthetic: random N(0, 0.02) weights, uniform random token ids",
+           "config": {"layers": "(windowed attention | gated recurrence) + dense, latent attention + dense, gated delta "
+                                "rule, the first layer's weights again",
+                      "window": context // 2, "keep_first": NATENEX_KEEP, "taps": NATENEX_TAPS, "blocks": NATENEX_BLOCKS,
+                      "page_tokens": 16},
+           "sizes": {}}
+    for size in args.design_sizes.split(","):
+        cfgs = natenex_configs(size, context)
+        points = {m: design_point(c, args.dtype, batch, context, args.steps, args.warmup, T) for m, c in cfgs.items()}
+        out["sizes"][size] = {
+            "shape": dict(zip(("width", "heads", "kv_heads", "head_size", "ff", "vocab"), DESIGN_SIZES[size])),
+            **points,
+            **{f"{phase}_natenex_over_{m}": round(points["natenex"][phase + "_tok_s"] / points[m][phase + "_tok_s"], 3)
+               for phase in ("prefill", "decode") for m in ("llama", "muvorax", "seredra")},
+            "like_kernels": natenex_rooflines(size, batch, context, T, points)}
+    print(json.dumps(out), flush=True)
+    return 0
+
+
 def design_point(cfg_json, dtype, batch, context, steps, warmup, T):
     """Prefill tok/s (one prompt of T tokens in one step), decode tok/s (batch x context, graphs) and the time of
     every kernel in an eager prefill step and an eager decode step of one model."""
@@ -1100,7 +1238,7 @@ def main() -> int:
                     help="for profiling: only the decode steps at --batch (as --no-points), only the 2,048-token "
                          "prefill (prints its figures as the line's value), or only the sampler over the preset's "
                          "vocabulary (microseconds a step's rows take on the GPU and on the host)")
-    ap.add_argument("--design", choices=["risizen", "gulidra", "lesarax", "seredra", "muvorax"], default=None,
+    ap.add_argument("--design", choices=["risizen", "gulidra", "lesarax", "seredra", "muvorax", "natenex"], default=None,
                     help="instead of the default workload: the named design beside the llama decoder at equal sizes "
                          "(--design-sizes), prefill and decode throughput and the times of their like kernels")
     ap.add_argument("--design-sizes", default="1b,8b", help="with --design: sizes of the comparison, of " + ",".join(DESIGN_SIZES))
@@ -1127,6 +1265,8 @@ def main() -> int:
         return seredra_run(args)
     if args.design == "muvorax":
         return muvorax_run(args)
+    if args.design == "natenex":
+        return natenex_run(args)
     if args.design:
         return design_run(args)
     if args.kernel_times:

@@ -180,7 +180,7 @@ def window_mixer(h, W, p, m, eps, positions, k, v, rnd: Callable = exact):
     T, H = h.shape[0], m["heads"]
     q = rms_norm(rnd(h @ W[p + "q"].T).reshape(T, H, m["dim"]), W[p + "q.norm"], eps)
     q = rnd(rotate_halves(q, positions, m["rot"]))
-    o = softmax_attention(q, k, v, m["scale"], int(positions[0]), m["mask"])
+    o = softmax_attention(q, k, v, m["scale"], int(positions[0]), m.get("mask"))
     return rnd(o).reshape(T, H * m["vdim"]) @ W[p + "o"].T
 
 
@@ -261,7 +261,9 @@ class Stepper:
                 st[key] = rows if key not in st else np.concatenate([st[key], rows])
 
         for i, layer in enumerate(cfg["layers"]):
-            j = layer.get("weights_of", i)
+            j = i
+            while cfg["layers"][j].get("weights_of") is not None:
+                j = cfg["layers"][j]["weights_of"]
             p, m, st = f"l{j}.mix.", layer["mixer"], self.kept[i]
             h = rnd(x)
             if layer["type"] == "parallel":
