@@ -254,55 +254,63 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
       s[it][r] = (i < dk && col) ? S[(size_t)i * dv + j] : 0.f;
     }
 
-  Frag kf[KS], qf[KS], ktf[ST][2], th[2], tl[2], ph[2], pl[2];
-  float vr[4], cb[4], ck[4], cq[4], ce[4], c_end;
-  auto load_first = [&](int c) {                  // what the right-hand side needs
+  // What a chunk reads from memory; the next chunk's is asked for when a chunk begins, so that a whole chunk's work lies
+  // between the asking and the use: without a condition (behind the last chunk it is that chunk's again) and without a
+  // step of arithmetic on the way, either of which would make the wave wait.  Elements beyond the key size are read
+  // from its first ones: the state's image has zeros there.
+  struct Chunk {
+    Frag kf[KS], qf[KS];                          // the wave's rows of keys and queries
+    Frag ktf[ST][2];                              // the wave's key elements across
+    Frag th[2], tl[2], ph[2], pl[2];              // the wave's rows of the inverse and of P
+    bf16_t vr[4];
+    float4 cb, ck, cq, ce;
+    float c_end;
+  };
+  auto load = [&](Chunk& x, int c) {
     const int r0 = base + c * C, nc = min(C, rows_all - c * C);
     const bf16_t* kr = rows + (size_t)(r0 + min(wave * 16 + li, nc - 1)) * ld + k_off + (size_t)hk * dk;
     const bf16_t* qr = kr - k_off + q_off;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
-      const int e = ks * 32 + lc * 8;
-      kf[ks] = e < dk ? load_frag(kr + e) : zero_frag();
-      qf[ks] = e < dk ? load_frag(qr + e) : zero_frag();
+      const int e = ks * 32 + lc * 8, at = e < dk ? e : 0;
+      x.kf[ks] = load_frag(kr + at);
+      x.qf[ks] = load_frag(qr + at);
     }
     const float* co = coef + ((size_t)(first + c) * H + h) * COEF + wave * 16 + lc * 4;
+    x.cb = *reinterpret_cast<const float4*>(co);
+    x.ck = *reinterpret_cast<const float4*>(co + C);
+    x.cq = *reinterpret_cast<const float4*>(co + 2 * C);
+    x.ce = *reinterpret_cast<const float4*>(co + 3 * C);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = min(wave * 16 + lc * 4 + r, nc - 1);
-      vr[r] = bf16_to_float(rows[(size_t)(r0 + t) * ld + v_off + (size_t)h * dv + jc]);
-      cb[r] = co[r];
-      ck[r] = co[C + r];
-      cq[r] = co[2 * C + r];
-      ce[r] = co[3 * C + r];
+      x.vr[r] = rows[(size_t)(r0 + t) * ld + v_off + (size_t)h * dv + jc];
     }
-    c_end = coef[((size_t)(first + c) * H + h) * COEF + NCOEF * C];
-  };
-  auto load_factors = [&](int c) {                // rows of the inverse and of P; keys across
+    x.c_end = coef[((size_t)(first + c) * H + h) * COEF + NCOEF * C];
     const bf16_t* F = fact + ((size_t)(first + c) * H + h) * FACT + (wave * 16 + li) * C + lc * 8;
 #pragma unroll
     for (int kk = 0; kk < 2; ++kk) {
-      th[kk] = load_frag(F + kk * 32);
-      tl[kk] = load_frag(F + C * C + kk * 32);
-      ph[kk] = load_frag(F + 2 * C * C + kk * 32);
-      pl[kk] = load_frag(F + 3 * C * C + kk * 32);
+      x.th[kk] = load_frag(F + kk * 32);
+      x.tl[kk] = load_frag(F + C * C + kk * 32);
+      x.ph[kk] = load_frag(F + 2 * C * C + kk * 32);
+      x.pl[kk] = load_frag(F + 3 * C * C + kk * 32);
     }
     const bf16_t* K = kt + ((size_t)(first + c) * G + hk) * dk * C;
 #pragma unroll
     for (int it = 0; it < ST; ++it) {
-      const int i = (wave * ST + it) * 16 + li;
+      const int i = (wave * ST + it) * 16 + li, at = i < dk ? i : 0;
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk) ktf[it][kk] = i < dk ? load_frag(K + (size_t)i * C + kk * 32 + lc * 8) : zero_frag();
+      for (int kk = 0; kk < 2; ++kk) x.ktf[it][kk] = load_frag(K + (size_t)at * C + kk * 32 + lc * 8);
     }
   };
-  load_first(0);
-  load_factors(0);
-  for (int c = 0; c < n; ++c) {
+  auto walk = [&](const Chunk& x, Chunk& next, int c) {
     const int nc = min(C, rows_all - c * C);
+    load(next, min(c + 1, n - 1));
 #pragma unroll
     for (int it = 0; it < ST; ++it) {
-      const int at = li * SR + (wave * ST + it) * 16 + lc * 4;
-      store_split4(Sh + at, Sl + at, s[it][0], s[it][1], s[it][2], s[it][3]);
+      const int i = (wave * ST + it) * 16 + lc * 4, at = li * SR + i;
+      const bool in = i < dk;                     // (the key size is a multiple of 8)
+      store_split4(Sh + at, Sl + at, in ? s[it][0] : 0.f, in ? s[it][1] : 0.f, in ? s[it][2] : 0.f, in ? s[it][3] : 0.f);
     }
     __syncthreads();
     // ---- S0^T k and S0^T q of the wave's rows: tile rows t, columns j
@@ -311,23 +319,23 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
     for (int ks = 0; ks < KS; ++ks) {
       const Frag fh = *reinterpret_cast<const Frag*>(Sh + li * SR + ks * 32 + lc * 8);
       const Frag fl = *reinterpret_cast<const Frag*>(Sl + li * SR + ks * 32 + lc * 8);
-      sk = mfma16(kf[ks], fh, sk);
-      o = mfma16(qf[ks], fh, o);
-      sk = mfma16(kf[ks], fl, sk);
-      o = mfma16(qf[ks], fl, o);
+      sk = mfma16(x.kf[ks], fh, sk);
+      o = mfma16(x.qf[ks], fh, o);
+      sk = mfma16(x.kf[ks], fl, sk);
+      o = mfma16(x.qf[ks], fl, o);
     }
     {
-      float x[4];
+      const float ck[4] = {x.ck.x, x.ck.y, x.ck.z, x.ck.w}, cb[4] = {x.cb.x, x.cb.y, x.cb.z, x.cb.w};
+      const float cq[4] = {x.cq.x, x.cq.y, x.cq.z, x.cq.w};
+      float y[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        x[r] = fmaf(-ck[r], sk[r], cb[r] * vr[r]);
+        y[r] = fmaf(-ck[r], sk[r], cb[r] * bf16_to_float(x.vr[r]));
         o[r] *= cq[r];
       }
       const int at = li * UR + wave * 16 + lc * 4;
-      store_split4(Rh + at, Rl + at, x[0], x[1], x[2], x[3]);
+      store_split4(Rh + at, Rl + at, y[0], y[1], y[2], y[3]);
     }
-    const float e0 = ce[0], e1 = ce[1], e2 = ce[2], e3 = ce[3], g = c_end;
-    if (c + 1 < n) load_first(c + 1);
     __syncthreads();
     // ---- the writes of the wave's rows
     {
@@ -337,24 +345,24 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
         if (kk * 32 > wave * 16 + 15) continue;    // (later rows do not enter)
         const Frag fh = *reinterpret_cast<const Frag*>(Rh + li * UR + kk * 32 + lc * 8);
         const Frag fl = *reinterpret_cast<const Frag*>(Rl + li * UR + kk * 32 + lc * 8);
-        u = mfma16(th[kk], fh, u);
-        u = mfma16(th[kk], fl, u);
-        u = mfma16(tl[kk], fh, u);
+        u = mfma16(x.th[kk], fh, u);
+        u = mfma16(x.th[kk], fl, u);
+        u = mfma16(x.tl[kk], fh, u);
       }
       const int at = li * UR + wave * 16 + lc * 4;
       store_split4(Uh + at, Ul + at, u[0], u[1], u[2], u[3]);
-      store_split4(Eh + at, El + at, u[0] * e0, u[1] * e1, u[2] * e2, u[3] * e3);
+      store_split4(Eh + at, El + at, u[0] * x.ce.x, u[1] * x.ce.y, u[2] * x.ce.z, u[3] * x.ce.w);
     }
     __syncthreads();
     // ---- the state behind the chunk, then the outputs
 #pragma unroll
     for (int it = 0; it < ST; ++it) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) s[it][r] *= g;
+      for (int r = 0; r < 4; ++r) s[it][r] *= x.c_end;
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
-        s[it] = mfma16(ktf[it][kk], *reinterpret_cast<const Frag*>(Eh + li * UR + kk * 32 + lc * 8), s[it]);
-        s[it] = mfma16(ktf[it][kk], *reinterpret_cast<const Frag*>(El + li * UR + kk * 32 + lc * 8), s[it]);
+        s[it] = mfma16(x.ktf[it][kk], *reinterpret_cast<const Frag*>(Eh + li * UR + kk * 32 + lc * 8), s[it]);
+        s[it] = mfma16(x.ktf[it][kk], *reinterpret_cast<const Frag*>(El + li * UR + kk * 32 + lc * 8), s[it]);
       }
     }
 #pragma unroll
@@ -362,11 +370,10 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
       if (kk * 32 > wave * 16 + 15) continue;
       const Frag fh = *reinterpret_cast<const Frag*>(Uh + li * UR + kk * 32 + lc * 8);
       const Frag fl = *reinterpret_cast<const Frag*>(Ul + li * UR + kk * 32 + lc * 8);
-      o = mfma16(ph[kk], fh, o);
-      o = mfma16(ph[kk], fl, o);
-      o = mfma16(pl[kk], fh, o);
+      o = mfma16(x.ph[kk], fh, o);
+      o = mfma16(x.ph[kk], fl, o);
+      o = mfma16(x.pl[kk], fh, o);
     }
-    if (c + 1 < n) load_factors(c + 1);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = wave * 16 + lc * 4 + r;
@@ -374,6 +381,12 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(
     }
     // (the state's image is written next: all reads of it lie ahead of the second barrier above; the right-hand side and
     // the writes are next stored behind the next chunk's first and second barriers)
+  };
+  Chunk a, b;
+  load(a, 0);
+  for (int c = 0; c < n; c += 2) {
+    walk(a, b, c);
+    if (c + 1 < n) walk(b, a, c + 1);
   }
 #pragma unroll
   for (int it = 0; it < ST; ++it)

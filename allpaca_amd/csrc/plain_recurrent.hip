@@ -208,6 +208,67 @@ __global__ __launch_bounds__(64) void gated_groupnorm_kernel(const float* __rest
   }
 }
 
+// The same on 16-byte accesses for groups whose size is a multiple of 4 and at most 1,024: L lanes (a power of two) a
+// group, several groups a wave, a lane's elements in registers between the sum and the scaling.
+__global__ __launch_bounds__(256) void gated_groupnorm_f4_kernel(const float* __restrict__ o, int ldo_in,
+                                                                 const float* __restrict__ w, float eps,
+                                                                 const void* __restrict__ gate, int gate_dtype, int ldg,
+                                                                 int gate_kind, void* __restrict__ out, int out_dtype,
+                                                                 int ldo, int group, int L, int per_row, long n_groups) {
+  const long g = ((long)blockIdx.x * 256 + threadIdx.x) / L;
+  const int l = threadIdx.x % L;
+  const bool on = g < n_groups;
+  const long r = on ? g / per_row : 0;
+  const int c0 = on ? (int)(g % per_row) * group : 0;
+  constexpr int VPT = 4;
+  float4 v[VPT];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    const int i = (l + j * L) * 4;
+    v[j] = i < group ? *reinterpret_cast<const float4*>(o + r * ldo_in + c0 + i) : float4{0.f, 0.f, 0.f, 0.f};
+    ss = fmaf(v[j].x, v[j].x, ss);
+    ss = fmaf(v[j].y, v[j].y, ss);
+    ss = fmaf(v[j].z, v[j].z, ss);
+    ss = fmaf(v[j].w, v[j].w, ss);
+  }
+  for (int x = L / 2; x > 0; x >>= 1) ss += __shfl_xor(ss, x, WAVE);
+  const float inv = 1.0f / sqrtf(ss / (float)group + eps);
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    const int i = (l + j * L) * 4;
+    if (!on || i >= group) continue;
+    float a[4] = {v[j].x * inv, v[j].y * inv, v[j].z * inv, v[j].w * inv};
+    if (w) {
+      const float4 ww = *reinterpret_cast<const float4*>(w + c0 + i);
+      a[0] *= ww.x; a[1] *= ww.y; a[2] *= ww.z; a[3] *= ww.w;
+    }
+    if (gate) {
+      float z[4];
+      const size_t at = (size_t)r * ldg + c0 + i;
+      if (gate_dtype == APC_F32) {
+        const float4 q = *reinterpret_cast<const float4*>((const float*)gate + at);
+        z[0] = q.x; z[1] = q.y; z[2] = q.z; z[3] = q.w;
+      } else {
+        const uint2 q = *reinterpret_cast<const uint2*>((const bf16_t*)gate + at);
+        z[0] = __uint_as_float(q.x << 16); z[1] = __uint_as_float(q.x & 0xffff0000u);
+        z[2] = __uint_as_float(q.y << 16); z[3] = __uint_as_float(q.y & 0xffff0000u);
+      }
+#pragma unroll
+      for (int x = 0; x < 4; ++x) a[x] *= gate_kind == 1 ? z[x] * sigmoid_f(z[x]) : sigmoid_f(z[x]);
+    }
+    const size_t at = (size_t)r * ldo + c0 + i;
+    if (out_dtype == APC_F32) {
+      *reinterpret_cast<float4*>((float*)out + at) = float4{a[0], a[1], a[2], a[3]};
+    } else {
+      uint2 pk;
+      pk.x = pack_bf16x2(a[0], a[1]);
+      pk.y = pack_bf16x2(a[2], a[3]);
+      *reinterpret_cast<uint2*>((bf16_t*)out + at) = pk;
+    }
+  }
+}
+
 // out[t] = (o[t] / sqrt(mean(o[t]^2) + eps)) * w * sigmoid(gate[t]), over the whole row of concatenated heads
 template <int NT>
 __global__ __launch_bounds__(NT) void gated_rmsnorm_kernel(const float* __restrict__ o, int ldo_in,
@@ -383,15 +444,27 @@ APC_EXPORT int apc_gated_rmsnorm(const float* o, int ldo_in, const float* w, flo
   if (n_rows <= 0) return 0;
   if (dim <= 0 || ldo_in < dim || ldo < dim || (gate && ldg < dim)) return APC_ERR_BAD_ARG;
   if (group < 0 || (group && dim % group) || gate_kind < 0 || gate_kind > 1) return APC_ERR_BAD_ARG;
+  auto aligned = [](const void* p, int dtype) { return ((uintptr_t)p & (dtype == APC_F32 ? 15u : 7u)) == 0; };
   if (group || !w || gate_kind) {
     const int g = group ? group : dim;
     if (dim / g > 65535) return APC_ERR_UNSUPPORTED;
+    // (which of the two kernels runs, and so the order of the additions, is fixed by the sizes and the alignment alone)
+    if (g % 4 == 0 && g <= 1024 && ldo_in % 4 == 0 && ldo % 4 == 0 && aligned(o, APC_F32) && aligned(w, APC_F32) &&
+        aligned(out, out_dtype) && (!gate || (ldg % 4 == 0 && aligned(gate, gate_dtype)))) {
+      int L = 1;
+      while (L < WAVE && L * 4 < g) L *= 2;
+      const long n_groups = (long)n_rows * (dim / g), blocks = (n_groups * L + 255) / 256;
+      if (blocks > 0x7fffffffL) return APC_ERR_UNSUPPORTED;
+      hipLaunchKernelGGL(gated_groupnorm_f4_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, o, ldo_in, w, eps, gate,
+                         gate_dtype, ldg, gate_kind, out, out_dtype, ldo, g, L, dim / g, n_groups);
+      APC_LAUNCH_CHECK();
+      return 0;
+    }
     hipLaunchKernelGGL(gated_groupnorm_kernel, dim3(n_rows, dim / g), dim3(64), 0, stream, o, ldo_in, w, eps, gate,
                        gate_dtype, ldg, gate_kind, out, out_dtype, ldo, g);
     APC_LAUNCH_CHECK();
     return 0;
   }
-  auto aligned = [](const void* p, int dtype) { return ((uintptr_t)p & (dtype == APC_F32 ? 15u : 7u)) == 0; };
   if (dim % 4 == 0 && dim <= 256 * 4 * 8 && ldo_in % 4 == 0 && ldo % 4 == 0 && aligned(o, APC_F32) && aligned(w, APC_F32) &&
       aligned(out, out_dtype) && (!gate || (ldg % 4 == 0 && aligned(gate, gate_dtype)))) {
 #define GATED_LAUNCH(VPT_)                                                                                               \
